@@ -9,8 +9,9 @@ This manager keeps those rules and adds what other layer kinds need:
 
 * **Cache groups.**  Cache entries (one per caching call of the run order) with the
   same geometry and visibility form a group; each group has a pool, a free list and
-  block tables of its own.  A group that only ever looks ``window`` keys back gives
-  pages back as soon as the window has passed them.
+  block tables of its own.  A group that only ever looks ``window`` keys back, or at the
+  keys of the current ``chunk`` of positions, gives pages back as soon as the window (or the
+  start of the next chunk) has passed them.
 * **Slots.**  Every live request holds one slot index.  Mixers with per-request state
   of fixed size get a tensor ``[max_slots, ...]`` per cache entry, zeroed when the
   slot is handed out.  GPT-2 has none; the slot then only carries the position.
@@ -42,13 +43,34 @@ class CacheGroupSpec:
     value_dim: int = 0  # head size of the values where it differs from the keys' (0: the same)
     # True: values are read from the key rows; the group keeps one pool and hands it out as both
     values_in_keys: bool = False
+    # > 0: a position sees the earlier ones of its own chunk only, chunks of this many positions
+    # counted from position 0
+    chunk: int = 0
+
+    def __post_init__(self):
+        if self.window > 0 and self.chunk > 0:
+            raise ValueError("a cache group sees a window or a chunk, not both")
+
+    @property
+    def span(self) -> int:
+        """Most keys that a position of the group sees (0: no limit)."""
+        return self.window or self.chunk
+
+    def first_visible(self, position: int) -> int:
+        """The first key that the query at ``position`` sees; it never falls as positions rise."""
+        if self.window > 0:
+            return max(0, position - self.window + 1)
+        if self.chunk > 0:
+            return position // self.chunk * self.chunk
+        return 0
 
     @property
     def value_head_dim(self) -> int:
         return self.value_dim or self.head_dim
 
     def geometry(self):
-        return (self.kv_heads, self.head_dim, self.window, self.value_head_dim, self.values_in_keys)
+        return (self.kv_heads, self.head_dim, self.window, self.value_head_dim, self.values_in_keys,
+                self.chunk)
 
 
 @dataclass(frozen=True)
@@ -142,7 +164,7 @@ class CacheManager:
                 seen.add(entry)
         self.page_size = page_size
         self.max_slots = max_slots
-        self._windowed = any(group.window > 0 for group in self.groups)
+        self._windowed = any(group.span > 0 for group in self.groups)
         self.dtype = dtype
         self.device = torch.device(device)
         self.max_positions = max_positions
@@ -199,12 +221,12 @@ class CacheManager:
         """Most pages that one request of ``length`` tokens holds in a group at any
         time, when no step brings more than ``longest_step`` tokens."""
         full = -(-length // self.page_size)
-        window = self.groups[group_index].window
-        if window <= 0:
+        span = self.groups[group_index].span
+        if span <= 0:
             return full
         step = length if longest_step is None else min(longest_step, length)
-        # keys of the step plus the window behind its first token, page-aligned slack
-        span = window + step
+        # keys of the step plus what its first token sees behind it, page-aligned slack
+        span += step
         return min(full, -(-span // self.page_size) + 1)
 
     # --------------------------------------------------------------- requests
@@ -289,11 +311,10 @@ class CacheManager:
         if not self._windowed:
             return
         for group_index, group in enumerate(self.groups):
-            if group.window <= 0:
+            if group.span <= 0:
                 continue
-            # The next query sits at position >= new_length and sees keys
-            # > position - window; keys <= new_length - window are dead.
-            last_dead = new_length - group.window
+            # the next query sits at position >= new_length: what that one does not see is dead
+            last_dead = group.first_visible(new_length) - 1
             table = record.tables[group_index]
             page = 0
             while page < len(table) and (page + 1) * self.page_size - 1 <= last_dead:

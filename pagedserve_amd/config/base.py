@@ -30,3 +30,14 @@ def require_int(raw, key, default=None, minimum=1):
     if value < minimum:
         raise ConfigError(f"config.json '{key}' must be >= {minimum}, got {value}")
     return value
+
+
+def require_number(raw, key, where, positive=True):
+    """``raw[key]`` as a float (a positive one unless told otherwise); ``where`` names the part of
+    the file in the error."""
+    value = raw.get(key) if isinstance(raw, dict) else None
+    if isinstance(value, bool) or not isinstance(value, (int, float)):
+        raise ConfigError(f"config.json {where} '{key}' must be a number, got {value!r}")
+    if positive and not value > 0:
+        raise ConfigError(f"config.json {where} '{key}' must be positive, got {value!r}")
+    return float(value)

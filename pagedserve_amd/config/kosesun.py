@@ -10,18 +10,9 @@ loader reads it from there (``decay_rank`` may name it in the file).
 from dataclasses import dataclass
 from typing import Optional, Tuple
 
-from .base import ConfigError, require_int
+from .base import ConfigError, require_int, require_number
 
 MIXERS = ("attention", "gla")
-
-
-def _number(raw, key, where, positive=True):
-    value = raw.get(key)
-    if isinstance(value, bool) or not isinstance(value, (int, float)):
-        raise ConfigError(f"config.json {where} '{key}' must be a number, got {value!r}")
-    if positive and not value > 0:
-        raise ConfigError(f"config.json {where} '{key}' must be positive, got {value!r}")
-    return float(value)
 
 
 @dataclass(frozen=True)
@@ -119,15 +110,15 @@ class KosesunConfig:
                     built = KosesunAttention(
                         heads=heads, kv_heads=kv_heads, dim=dim,
                         vdim=require_int(mixer, "vdim", default=dim),
-                        scale=_number(mixer, "scale", where + ".mixer"),
+                        scale=require_number(mixer, "scale", where + ".mixer"),
                         rot_dims=rot_dims,
-                        rot_base=_number(rot, "base", where + ".mixer.rot") if rot_dims else 10000.0,
+                        rot_base=require_number(rot, "base", where + ".mixer.rot") if rot_dims else 10000.0,
                         v_mix=bool(mixer.get("v_mix", False)))
                 else:
                     rank = mixer.get("decay_rank")
                     built = KosesunGLA(
                         heads=require_int(mixer, "heads"), dim=require_int(mixer, "dim"),
-                        vdim=require_int(mixer, "vdim"), tau=_number(mixer, "tau", where + ".mixer"),
+                        vdim=require_int(mixer, "vdim"), tau=require_number(mixer, "tau", where + ".mixer"),
                         decay_rank=None if rank is None else require_int(mixer, "decay_rank"))
             except ConfigError as error:
                 raise ConfigError(f"{where}: {error}") from None
@@ -149,9 +140,9 @@ class KosesunConfig:
             vocab=require_int(raw, "vocab"),
             width=require_int(raw, "width"),
             layers=tuple(layers),
-            norm_eps=_number(norm, "eps", "norm"),
-            embedding_scale=_number(embedding, "scale", "embedding") if "scale" in embedding else 1.0,
-            logit_softcap=0.0 if softcap is None else _number(raw, "logit_softcap", ""),
+            norm_eps=require_number(norm, "eps", "norm"),
+            embedding_scale=require_number(embedding, "scale", "embedding") if "scale" in embedding else 1.0,
+            logit_softcap=0.0 if softcap is None else require_number(raw, "logit_softcap", ""),
             streams=require_int(raw, "streams", default=0, minimum=0),
             max_positions=require_int(raw, "max_positions", default=cls.DEFAULT_MAX_POSITIONS),
         )

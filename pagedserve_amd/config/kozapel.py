@@ -10,18 +10,9 @@ The residual stream is kept in ``streams`` copies.  Every size and constant come
 from dataclasses import dataclass
 from typing import Optional, Tuple
 
-from .base import ConfigError, require_int
+from .base import ConfigError, require_int, require_number
 
 MIXERS = ("attention", "latent_attention")
-
-
-def _number(raw, key, where, positive=True):
-    value = raw.get(key) if isinstance(raw, dict) else None
-    if isinstance(value, bool) or not isinstance(value, (int, float)):
-        raise ConfigError(f"config.json {where} '{key}' must be a number, got {value!r}")
-    if positive and not value > 0:
-        raise ConfigError(f"config.json {where} '{key}' must be positive, got {value!r}")
-    return float(value)
 
 
 @dataclass(frozen=True)
@@ -101,7 +92,7 @@ def _read_mixer(kind, mixer, where, index):
     heads = require_int(mixer, "heads")
     dim = require_int(mixer, "dim")
     vdim = require_int(mixer, "vdim", default=dim)
-    scale = _number(mixer, "scale", where + ".mixer")
+    scale = require_number(mixer, "scale", where + ".mixer")
     if kind == "attention":
         kv_heads = require_int(mixer, "kv_heads", default=heads)
         if heads % kv_heads:
@@ -116,7 +107,7 @@ def _read_mixer(kind, mixer, where, index):
             if kv_from >= index:
                 raise ConfigError(f"'kv_from' {kv_from} must name an earlier layer")
         return KozapelAttention(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=scale,
-                                diff=_number(mixer, "diff", where + ".mixer", positive=False),
+                                diff=require_number(mixer, "diff", where + ".mixer", positive=False),
                                 window=window, kv_from=kv_from)
     rot_dim = require_int(mixer, "rot_dim", minimum=0)
     rot = mixer.get("rot") or {}
@@ -130,7 +121,7 @@ def _read_mixer(kind, mixer, where, index):
     return KozapelLatent(heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim,
                          kv_rank=require_int(mixer, "kv_rank"), q_rank=require_int(mixer, "q_rank"),
                          scale=scale,
-                         rot_base=_number(rot, "base", where + ".mixer.rot") if rot_dim else 10000.0)
+                         rot_base=require_number(rot, "base", where + ".mixer.rot") if rot_dim else 10000.0)
 
 
 def _read_feed_forward(mlp, where):
@@ -154,7 +145,7 @@ def _read_feed_forward(mlp, where):
         raise ConfigError(f"'router.top' {top} exceeds the experts of the {keep} groups that are kept")
     shared = mlp.get("shared")
     return KozapelFeedForward("moe", require_int(expert, "ff"), experts=experts, top=top, groups=count,
-                              keep=keep, scale=_number(router, "scale", where + ".mlp.router")
+                              keep=keep, scale=require_number(router, "scale", where + ".mlp.router")
                               if "scale" in router else 1.0,
                               shared_ff=require_int(shared, "ff") if shared else 0)
 
@@ -216,8 +207,8 @@ class KozapelConfig:
             vocab=require_int(raw, "vocab"),
             width=require_int(raw, "width"),
             layers=tuple(layers),
-            norm_eps=_number(norm, "eps", "norm"),
-            embedding_scale=_number(embedding, "scale", "embedding") if "scale" in embedding else 1.0,
+            norm_eps=require_number(norm, "eps", "norm"),
+            embedding_scale=require_number(embedding, "scale", "embedding") if "scale" in embedding else 1.0,
             streams=require_int(raw, "streams", default=0, minimum=0),
             max_positions=require_int(raw, "max_positions", default=cls.DEFAULT_MAX_POSITIONS),
         )

@@ -9,18 +9,9 @@ optional YaRN ``scaling``).  Every size and constant comes from the file.
 from dataclasses import dataclass
 from typing import Optional, Tuple
 
-from .base import ConfigError, require_int
+from .base import ConfigError, require_int, require_number
 
 MIXERS = ("rglru", "attention", "latent_attention")
-
-
-def _number(raw, key, where, positive=True):
-    value = raw.get(key) if isinstance(raw, dict) else None
-    if isinstance(value, bool) or not isinstance(value, (int, float)):
-        raise ConfigError(f"config.json {where} '{key}' must be a number, got {value!r}")
-    if positive and not value > 0:
-        raise ConfigError(f"config.json {where} '{key}' must be positive, got {value!r}")
-    return float(value)
 
 
 @dataclass(frozen=True)
@@ -135,17 +126,17 @@ def _read_rotation(raw, where, most):
         if not isinstance(scaling, dict):
             raise ConfigError(f"config.json {where} 'rot.scaling' must be an object")
         inner = where + ".rot.scaling"
-        scaling = RezelixScaling(factor=_number(scaling, "factor", inner),
-                                 original=_number(scaling, "original", inner),
-                                 fast=_number(scaling, "fast", inner),
-                                 slow=_number(scaling, "slow", inner))
-    return RezelixRotation(dims=dims, base=_number(raw, "base", where + ".rot"), scaling=scaling)
+        scaling = RezelixScaling(factor=require_number(scaling, "factor", inner),
+                                 original=require_number(scaling, "original", inner),
+                                 fast=require_number(scaling, "fast", inner),
+                                 slow=require_number(scaling, "slow", inner))
+    return RezelixRotation(dims=dims, base=require_number(raw, "base", where + ".rot"), scaling=scaling)
 
 
 def _cap(mixer, where):
     if mixer.get("softcap") in (None, 0, 0.0):
         return 0.0
-    return _number(mixer, "softcap", where)
+    return require_number(mixer, "softcap", where)
 
 
 def _read_mixer(kind, mixer, where):
@@ -165,7 +156,7 @@ def _read_mixer(kind, mixer, where):
         if vdim != dim:
             raise ConfigError(f"the values are the keys as projected: 'vdim' {vdim} must equal 'dim' {dim}")
         return RezelixAttention(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim,
-                                scale=_number(mixer, "scale", where + ".mixer"),
+                                scale=require_number(mixer, "scale", where + ".mixer"),
                                 softcap=_cap(mixer, where + ".mixer"),
                                 rot=_read_rotation(mixer.get("rot"), where + ".mixer", dim))
     rot_dim = require_int(mixer, "rot_dim", minimum=0)
@@ -174,7 +165,7 @@ def _read_mixer(kind, mixer, where):
         raise ConfigError(f"'rot.dims' {rot.dims} must equal 'rot_dim' {rot_dim}: the rotated part is rotated whole")
     return RezelixLatent(heads=heads, dim=dim, rot_dim=rot_dim, vdim=require_int(mixer, "vdim"),
                          kv_rank=require_int(mixer, "kv_rank"),
-                         scale=_number(mixer, "scale", where + ".mixer"),
+                         scale=require_number(mixer, "scale", where + ".mixer"),
                          softcap=_cap(mixer, where + ".mixer"), rot=rot)
 
 
@@ -228,7 +219,7 @@ class RezelixConfig:
             vocab=require_int(raw, "vocab"),
             width=require_int(raw, "width"),
             layers=tuple(layers),
-            norm_eps=_number(norm, "eps", "norm"),
+            norm_eps=require_number(norm, "eps", "norm"),
             max_positions=require_int(raw, "max_positions", default=cls.DEFAULT_MAX_POSITIONS),
         )
 

@@ -93,6 +93,9 @@ class LayerCall:
     # >= 0: row of the model's table of pass vectors (``ModelSpec.pass_rows``) that is added to the
     # stream of every token right before this call
     enter: int = -1
+    # True: the embedded tokens (the stream as it was before the first call) are added to the stream
+    # right before this call, ahead of the pass vector
+    add_embedding: bool = False
 
 
 @dataclass(frozen=True)
@@ -136,6 +139,8 @@ class ModelSpec:
                 raise ValueError(f"a call adds pass vector {call.enter}, the model has {self.pass_rows}")
             if call.enter >= 0 and self.streams:
                 raise ValueError("pass vectors are added to a single residual stream only")
+            if call.add_embedding and self.streams:
+                raise ValueError("the embedding is added again to a single residual stream only")
             if call.writes_cache:
                 if call.cache in writers:
                     raise ValueError(f"cache entry {call.cache} has two writers")

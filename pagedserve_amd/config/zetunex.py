@@ -10,18 +10,9 @@ constant comes from the file.
 from dataclasses import dataclass
 from typing import Optional, Tuple
 
-from .base import ConfigError, require_int
+from .base import ConfigError, require_int, require_number
 
 MIXERS = ("lightning", "parallel")
-
-
-def _number(raw, key, where, positive=True):
-    value = raw.get(key) if isinstance(raw, dict) else None
-    if isinstance(value, bool) or not isinstance(value, (int, float)):
-        raise ConfigError(f"config.json {where} '{key}' must be a number, got {value!r}")
-    if positive and not value > 0:
-        raise ConfigError(f"config.json {where} '{key}' must be positive, got {value!r}")
-    return float(value)
 
 
 @dataclass(frozen=True)
@@ -123,7 +114,7 @@ def _read_mixer(kind, mixer, where):
     return ZetunexParallel(
         left=ZetunexWindowed(heads=heads, kv_heads=kv_heads, dim=dim,
                              vdim=require_int(left, "vdim", default=dim),
-                             scale=_number(left, "scale", where + ".mixer.left"),
+                             scale=require_number(left, "scale", where + ".mixer.left"),
                              window=require_int(mask, "size", default=0, minimum=0)),
         right=ZetunexScan(inner=require_int(right, "inner"), state=require_int(right, "state"),
                           dt_rank=require_int(right, "dt_rank"), conv=require_int(right, "conv")))
@@ -150,7 +141,7 @@ def _read_feed_forward(mlp, where):
                           f"cannot give {top} per token")
     return ZetunexFeedForward(
         "moe", require_int(expert, "ff"), experts=experts, top=top, groups=count, keep=keep,
-        scale=_number(router, "scale", where + ".mlp.router") if "scale" in router else 1.0)
+        scale=require_number(router, "scale", where + ".mlp.router") if "scale" in router else 1.0)
 
 
 @dataclass(frozen=True)
@@ -210,8 +201,8 @@ class ZetunexConfig:
             vocab=require_int(raw, "vocab"),
             width=require_int(raw, "width"),
             layers=tuple(layers),
-            norm_eps=_number(norm, "eps", "norm"),
-            residual_mult=_number(raw, "residual_mult", "", positive=False) if "residual_mult" in raw else 1.0,
+            norm_eps=require_number(norm, "eps", "norm"),
+            residual_mult=require_number(raw, "residual_mult", "", positive=False) if "residual_mult" in raw else 1.0,
             loop_start=start, loop_stop=stop, loop_times=times,
             max_positions=require_int(raw, "max_positions", default=cls.DEFAULT_MAX_POSITIONS),
         )

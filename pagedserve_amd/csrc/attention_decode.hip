@@ -147,7 +147,7 @@ int ps_attention_reduce(const float* partial, void* out, int64_t out_stride, con
 }
 
 static int check_decode_sizes(const char* who, int count, int heads, int kv_heads, int head_dim,
-                              int page_size, int num_pages, int table_width, int window,
+                              int page_size, int num_pages, int table_width,
                               int splits, int waves, int dtype) {
   PS_REQUIRE(count >= 0 && heads > 0 && kv_heads > 0 && page_size > 0 && num_pages > 0 &&
                  table_width > 0,
@@ -158,7 +158,6 @@ static int check_decode_sizes(const char* who, int count, int heads, int kv_head
   PS_REQUIRE(head_dim > 0 && head_dim % 8 == 0 && head_dim <= 256,
              "%s: head_dim %d must be a multiple of 8 up to 256 (ps_attention_rowwise takes "
              "every head size)", who, head_dim);
-  PS_REQUIRE(window >= 0, "%s: negative window", who);
   PS_REQUIRE(splits >= 1 && splits <= 64 && heads <= 65535,
              "%s: splits %d / heads %d out of range", who, splits, heads);
   PS_REQUIRE(dtype == PS_F32 || dtype == PS_BF16, "%s: unknown dtype %d", who, dtype);
@@ -208,7 +207,7 @@ extern "C" int ps_attention_decode_static(const void* q, int64_t q_stride, const
                                           int page_size, int num_pages, float scale, int window,
                                           int splits, int waves, int dtype, void* stream) {
   if (check_decode_sizes("ps_attention_decode_static", count, heads, kv_heads, head_dim, page_size,
-                         num_pages, table_width, window, splits, waves, dtype))
+                         num_pages, table_width, splits, waves, dtype))
     return 1;
   PS_REQUIRE(out != nullptr, "ps_attention_decode_static: no output tensor");
   float* partial = nullptr;
@@ -248,7 +247,7 @@ extern "C" int ps_attention_decode_partial(const void* q, int64_t q_stride, cons
                                            int waves, const float* sink, float softcap, int dtype,
                                            void* stream) {
   if (check_decode_sizes("ps_attention_decode_partial", count, heads, kv_heads, head_dim,
-                         page_size, num_pages, table_width, window, splits, waves, dtype))
+                         page_size, num_pages, table_width, splits, waves, dtype))
     return 1;
   const int64_t need = (int64_t)count * heads * splits * (head_dim + 2);
   PS_REQUIRE(partial != nullptr && partial_floats >= need,
@@ -274,7 +273,7 @@ extern "C" int ps_attention_decode(const void* q, int64_t q_stride, const void* 
                                    const float* gate, int64_t gate_ld, float softcap, int dtype,
                                    void* stream) {
   if (check_decode_sizes("ps_attention_decode", count, heads, kv_heads, head_dim, page_size,
-                         num_pages, table_width, window, splits, waves, dtype))
+                         num_pages, table_width, splits, waves, dtype))
     return 1;
   PS_REQUIRE(out != nullptr, "ps_attention_decode: no output tensor");
   if (splits > 1) {

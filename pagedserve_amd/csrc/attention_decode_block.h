@@ -130,7 +130,7 @@ __device__ __forceinline__ void attention_decode_block(
   }
   const int pos = tok_pos[t];
   const int* table = tables + (int64_t)(direct ? t : tok_item[t]) * table_width;
-  const int first_key = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int first_key = first_visible_key(pos, window);
   const int end_key = pos + 1;
   int chunk = (end_key - first_key + splits - 1) / splits;
   chunk = (chunk + KEYS_PER_WAVE - 1) / KEYS_PER_WAVE * KEYS_PER_WAVE;

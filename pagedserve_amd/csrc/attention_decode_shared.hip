@@ -84,7 +84,7 @@ __global__ __launch_bounds__(256) void attention_decode_shared_kernel(const AdsA
   const int t = a.tok_list ? a.tok_list[n] : n;
   const int pos = a.tok_pos[t];
   const int* table = a.tables + (int64_t)(a.tok_item ? a.tok_item[t] : t) * a.table_width;
-  const int first_key = (a.window > 0 && pos - a.window + 1 > 0) ? pos - a.window + 1 : 0;
+  const int first_key = first_visible_key(pos, a.window);
   const int end_key = pos + 1;
   int chunk = (end_key - first_key + a.splits - 1) / a.splits;
   chunk = (chunk + ADS_KEYS - 1) / ADS_KEYS * ADS_KEYS;
@@ -267,8 +267,7 @@ extern "C" int ps_attention_decode_shared(const void* q, int64_t q_stride, const
              heads, kv_heads);
   PS_REQUIRE(head_dim > 0 && head_dim % 8 == 0 && head_dim <= 256,
              "ps_attention_decode_shared: head_dim %d must be a multiple of 8 up to 256", head_dim);
-  PS_REQUIRE(window >= 0 && splits >= 1 && splits <= 64, "ps_attention_decode_shared: window %d / splits %d",
-             window, splits);
+  PS_REQUIRE(splits >= 1 && splits <= 64, "ps_attention_decode_shared: splits %d", splits);
   PS_REQUIRE(q_stride % 8 == 0 && ((uintptr_t)q % 16) == 0 && ((uintptr_t)k_pool % 16) == 0 &&
                  ((uintptr_t)v_pool % 16) == 0,
              "ps_attention_decode_shared: queries and pools must be aligned to 16 bytes");

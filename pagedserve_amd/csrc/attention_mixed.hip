@@ -86,7 +86,7 @@ extern "C" int ps_attention_mixed(const void* q, int64_t q_stride, const void* k
              AP_TABLE_MAX, dtype, head_dim, table_width);
   PS_REQUIRE(heads % kv_heads == 0, "ps_attention_mixed: heads (%d) must be a multiple of kv_heads (%d)",
              heads, kv_heads);
-  PS_REQUIRE(window >= 0 && scale > 0.f, "ps_attention_mixed: bad window or scale");
+  PS_REQUIRE(scale > 0.f, "ps_attention_mixed: the score scale must be positive, got %g", scale);
   PS_REQUIRE(tok_list != nullptr && tok_item != nullptr,
              "ps_attention_mixed: the one-token items are given by their list and the tokens' items");
   PS_REQUIRE((int64_t)num_pages * kv_heads * page_size < ((int64_t)1 << 32),

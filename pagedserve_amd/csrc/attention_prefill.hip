@@ -65,7 +65,7 @@ extern "C" int ps_attention_prefill(const void* q, int64_t q_stride, const void*
              "ps_attention_prefill: heads (%d) must be a multiple of kv_heads (%d)", heads, kv_heads);
   PS_REQUIRE(head_dim > 0 && head_dim % 16 == 0 && head_dim <= 256,
              "ps_attention_prefill: head_dim %d must be a multiple of 16 up to 256", head_dim);
-  PS_REQUIRE(window >= 0 && tiles <= 65535, "ps_attention_prefill: bad window or too many tiles (%d)", tiles);
+  PS_REQUIRE(tiles <= 65535, "ps_attention_prefill: too many tiles (%d)", tiles);
   PS_REQUIRE(query_tile == AP_QUERIES || (query_tile == AP_QUERIES / 2 && head_dim <= 128) ||
                  (query_tile == AP_QUERIES * 2 && head_dim <= AP_LARGE_HEAD_DIM),
              "ps_attention_prefill: tiles of %d, (head sizes up to 128) %d or (head sizes up to %d) %d "

@@ -115,8 +115,10 @@ __device__ __forceinline__ void attention_prefill_block(
   const bool wave_active = q0 + wave_q * 32 < count;
   const int tile_last_q = q0 + QUERIES - 1 < count ? q0 + QUERIES - 1 : count - 1;
   const int key_end = start + tile_last_q + 1;
-  int key_begin = 0;
-  if (window > 0 && start + q0 - window + 1 > 0) key_begin = start + q0 - window + 1;
+  const int key_begin = first_visible_key(start + q0, window);
+  // the first keys that the wave's first and last query see
+  const int first_of_first = first_visible_key(wave_first, window);
+  const int first_of_last = wave_active ? first_visible_key(wave_last, window) : 0;
 
   // the block-table entries of keys key_begin .. key_end - 1
   const int first_logical = page_shift >= 0 ? (key_begin >> page_shift) : key_begin / page_size;
@@ -260,8 +262,7 @@ __device__ __forceinline__ void attention_prefill_block(
   auto wave_keys = [&](int t) { return k_first + t * AP_KEYS + wave_k * WAVE_KEYS; };
   // a wave's keys of a tile are skipped where no query of the wave can see them
   auto sees = [&](int kw) {
-    return wave_active && kw <= wave_last && kw < key_end &&
-           !(window > 0 && kw + WAVE_KEYS - 1 < wave_first - window + 1);
+    return wave_active && kw <= wave_last && kw < key_end && kw + WAVE_KEYS - 1 >= first_of_first;
   };
   auto stage_of = [&](int t) {
     return (uint32_t)(uintptr_t)(ap_lds_ptr)stages + (uint32_t)((t % STAGES) * STAGE_BYTES);
@@ -305,7 +306,7 @@ __device__ __forceinline__ void attention_prefill_block(
   auto weigh = [&](const int kw, f32x16 (&s)[KR], ValueRegs& vr) {
     // all of these keys are visible to every query of the wave: no mask
       const bool masked = kw + WAVE_KEYS - 1 > wave_first || kw + WAVE_KEYS > key_end ||
-                          (window > 0 && kw < wave_last - window + 1) || !q_valid;
+                          kw < first_of_last || !q_valid;
       // scores stay unscaled until the exponential: p = 2^(s c - m), with m kept in scaled units
       if (extra.softcap > 0.f) {
         // a cap on the scaled scores, in the unscaled scores' units
@@ -317,12 +318,13 @@ __device__ __forceinline__ void attention_prefill_block(
       }
       float tile_max = -INFINITY;
       if (__builtin_amdgcn_readfirstlane(__any(masked) ? 1 : 0)) {
+        const int q_first = q_valid ? first_visible_key(q_pos, window) : 0;
 #pragma unroll
         for (int r = 0; r < KR; ++r)
 #pragma unroll
           for (int e = 0; e < 16; ++e) {
             const int key = kw + r * 32 + (e >> 2) * 8 + half * 4 + (e & 3);
-            const bool visible = (key <= q_pos) & (window <= 0 || q_pos - key < window);
+            const bool visible = (key <= q_pos) & (key >= q_first);
             s[r][e] = visible ? s[r][e] : -INFINITY;
             tile_max = fmaxf(tile_max, s[r][e]);
           }

@@ -265,8 +265,9 @@ __device__ inline RotationPlace rotation_place(int d, int rot_dims, bool halves)
 
 // The same step for layers that treat every head on its own: the first `rot_dims` dimensions
 // of each query and key head are rotated by the token's position (pairs laid out as halves
-// or as neighbours; cosine and sine times `magnitude`), then, with head_norm, each head is
-// divided by its root mean square over its key_dim dimensions (no weight).  Values are the
+// or as neighbours; cosine and sine times `magnitude`); with head_norm each head is divided by its
+// root mean square over its key_dim dimensions, after the rotation (1) or before it (2), and
+// multiplied by a weight per dimension that all heads share (q_gamma, k_gamma; null: none).  Values are the
 // columns at v_col as projected (they may be the key columns themselves: values that are the
 // unrotated, unnormed keys).  A block per token, a wave per head in turn; a lane holds up to
 // four dimensions of the head.
@@ -275,7 +276,8 @@ __global__ __launch_bounds__(256) void attention_prepare_heads_kernel(
     const float* __restrict__ proj, int64_t ld, int q_col, int k_col, int v_col,
     T* __restrict__ q_out, int64_t q_stride, T* __restrict__ k_pool, T* __restrict__ v_pool,
     const float* __restrict__ freqs, int rot_dims, int halves, float magnitude, int head_norm,
-    float eps, const int* __restrict__ tok_item, const int* __restrict__ tok_pos,
+    const float* __restrict__ q_gamma, const float* __restrict__ k_gamma, float eps,
+    const int* __restrict__ tok_item, const int* __restrict__ tok_pos,
     const int* __restrict__ tables, int table_width, int heads, int kv_heads, int key_dim,
     int value_dim, int cache_dim, int page_size, int num_pages) {
   __shared__ float s_cos[128], s_sin[128];
@@ -300,24 +302,49 @@ __global__ __launch_bounds__(256) void attention_prepare_heads_kernel(
     const bool is_q = hh < heads;
     const int head = is_q ? hh : hh - heads;
     const float* src = row + (is_q ? q_col : k_col) + head * key_dim;
-    float value[4];
+    const float* gamma = is_q ? q_gamma : k_gamma;
+    const bool norm_first = head_norm == 2;
+    // every load of a lane's dimensions, and of the pairs' other ones, before anything waits
+    float value[4], other[4], weight[4], other_weight[4];
     float squares = 0.f;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int d = lane + 64 * r;
-      float v = 0.f;
-      if (d < key_dim) {
-        v = src[d];
-        if (d < rot_dims) {
-          const RotationPlace place = rotation_place(d, rot_dims, halves != 0);
-          v = v * s_cos[place.angle] + place.sign * src[place.partner] * s_sin[place.angle];
-        }
+      value[r] = d < key_dim ? src[d] : 0.f;
+      weight[r] = (gamma != nullptr && d < key_dim) ? gamma[d] : 1.f;
+      other[r] = 0.f;
+      other_weight[r] = 1.f;
+      if (d < rot_dims) {
+        const int partner = rotation_place(d, rot_dims, halves != 0).partner;
+        other[r] = src[partner];
+        if (gamma != nullptr) other_weight[r] = gamma[partner];
       }
-      value[r] = v;
-      squares = fmaf(v, v, squares);
+      squares = fmaf(value[r], value[r], squares);
     }
     float inv = 1.f;
-    if (head_norm) inv = 1.0f / sqrtf(wave_sum(squares) / (float)key_dim + eps);
+    if (norm_first) {
+      const float before = 1.0f / sqrtf(wave_sum(squares) / (float)key_dim + eps);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        value[r] *= before * weight[r];
+        other[r] *= before * other_weight[r];
+      }
+    }
+    squares = 0.f;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = lane + 64 * r;
+      if (d < rot_dims) {
+        const RotationPlace place = rotation_place(d, rot_dims, halves != 0);
+        value[r] = value[r] * s_cos[place.angle] + place.sign * other[r] * s_sin[place.angle];
+      }
+      squares = fmaf(value[r], value[r], squares);
+    }
+    if (head_norm == 1) {
+      inv = 1.0f / sqrtf(wave_sum(squares) / (float)key_dim + eps);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) value[r] *= weight[r];
+    }
     T* dst = nullptr;
     if (is_q) dst = q_out + (int64_t)t * q_stride + (int64_t)head * cache_dim;
     else if (stored) dst = k_pool + (((int64_t)page * kv_heads + head) * page_size + offset) * cache_dim;
@@ -341,7 +368,8 @@ __global__ __launch_bounds__(256) void attention_prepare_heads_kernel(
 extern "C" int ps_attention_prepare_heads(const float* proj, int64_t ld, int q_col, int k_col,
                                           int v_col, void* q_out, int64_t q_stride, void* k_pool,
                                           void* v_pool, const float* freqs, int rot_dims,
-                                          int halves, float magnitude, int head_norm, float eps,
+                                          int halves, float magnitude, int head_norm,
+                                          const float* q_gamma, const float* k_gamma, float eps,
                                           const int* tok_item, const int* tok_pos,
                                           const int* tables, int table_width, int tokens, int heads,
                                           int kv_heads, int key_dim, int value_dim, int cache_dim,
@@ -356,19 +384,22 @@ extern "C" int ps_attention_prepare_heads(const float* proj, int64_t ld, int q_c
              "ps_attention_prepare_heads: %d rotated dimensions do not fit heads of %d", rot_dims, key_dim);
   PS_REQUIRE(rot_dims == 0 || freqs != nullptr, "ps_attention_prepare_heads: rotation without frequencies");
   PS_REQUIRE(q_stride >= (int64_t)heads * cache_dim, "ps_attention_prepare_heads: query rows too short");
-  PS_REQUIRE(!head_norm || eps > 0.f, "ps_attention_prepare_heads: eps must be positive");
+  PS_REQUIRE(head_norm >= 0 && head_norm <= 2 && (!head_norm || eps > 0.f),
+             "ps_attention_prepare_heads: head norm %d (0: none, 1: behind the rotation, 2: ahead of it) needs a "
+             "positive eps", head_norm);
+  PS_REQUIRE(rot_dims <= 256, "ps_attention_prepare_heads: %d rotated dimensions, the kernel keeps angles for 256", rot_dims);
   PS_REQUIRE(dtype == PS_F32 || dtype == PS_BF16, "ps_attention_prepare_heads: unknown dtype %d", dtype);
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   if (dtype == PS_F32)
     hipLaunchKernelGGL(attention_prepare_heads_kernel<float>, dim3(tokens), dim3(256), 0, s, proj, ld,
                        q_col, k_col, v_col, (float*)q_out, q_stride, (float*)k_pool, (float*)v_pool,
-                       freqs, rot_dims, halves, magnitude, head_norm, eps, tok_item, tok_pos, tables,
+                       freqs, rot_dims, halves, magnitude, head_norm, q_gamma, k_gamma, eps, tok_item, tok_pos, tables,
                        table_width, heads, kv_heads, key_dim, value_dim, cache_dim, page_size, num_pages);
   else
     hipLaunchKernelGGL(attention_prepare_heads_kernel<bf16_t>, dim3(tokens), dim3(256), 0, s, proj, ld,
                        q_col, k_col, v_col, (bf16_t*)q_out, q_stride, (bf16_t*)k_pool, (bf16_t*)v_pool,
-                       freqs, rot_dims, halves, magnitude, head_norm, eps, tok_item, tok_pos, tables,
+                       freqs, rot_dims, halves, magnitude, head_norm, q_gamma, k_gamma, eps, tok_item, tok_pos, tables,
                        table_width, heads, kv_heads, key_dim, value_dim, cache_dim, page_size, num_pages);
   PS_CHECK_LAUNCH("ps_attention_prepare_heads");
   return 0;

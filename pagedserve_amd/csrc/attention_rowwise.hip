@@ -1,6 +1,6 @@
 // Paged attention, one wave per (token, head): the plain kernel of the engine.
 //
-// For the token at position p of its request it visits keys max(0, p - window + 1) .. p
+// For the token at position p of its request it visits keys first_visible_key(p, window) .. p
 // through the request's block table, 64 keys at a time: each lane scores one key
 // (q . k * scale), the wave keeps the running maximum and sum of an online softmax
 // (reference: src/kernels/triton_paged_attention.py:219-223,275-331), and each lane
@@ -34,7 +34,7 @@ __global__ __launch_bounds__(64) void attention_rowwise_kernel(
   const int lane = threadIdx.x;
   const int pos = tok_pos[t];
   const int* table = tables + (int64_t)tok_item[t] * table_width;
-  const int first_key = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int first_key = first_visible_key(pos, window);
   const int end_key = pos + 1;
 
   for (int i = lane; i < head_dim; i += 64)
@@ -114,7 +114,6 @@ extern "C" int ps_attention_rowwise(const void* q, int64_t q_stride, const void*
              heads, kv_heads);
   PS_REQUIRE(head_dim > 0 && head_dim <= 64 * AR_MAX_DIMS,
              "ps_attention_rowwise: head_dim %d must lie in 1..%d", head_dim, 64 * AR_MAX_DIMS);
-  PS_REQUIRE(window >= 0, "ps_attention_rowwise: negative window");
   PS_REQUIRE(heads <= 65535, "ps_attention_rowwise: too many heads");
   PS_REQUIRE(dtype == PS_F32 || dtype == PS_BF16, "ps_attention_rowwise: unknown dtype %d", dtype);
   if (tokens == 0) return 0;

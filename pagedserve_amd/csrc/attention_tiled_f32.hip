@@ -12,7 +12,7 @@
 // The tiles are those of the bfloat16 kernel (`tile_item`, `tile_q0`: the item of each tile and
 // its first query within the item's tokens of this step), and so are the rules: query i of an
 // item whose cached length after the step is L and which brings n tokens stands at position
-// L - n + i and sees keys max(0, position - window + 1) .. position.
+// L - n + i and sees keys first_visible_key(position, window) .. position.
 //
 // Head sizes that are multiples of 4 up to 128; others stay with the one-wave-per-token
 // kernel.
@@ -57,8 +57,7 @@ __global__ __launch_bounds__(256) void attention_tiled_f32_kernel(
   const int* table = tables + (int64_t)item * table_width;
   const int last_q = q0 + AF_TILE - 1 < count ? q0 + AF_TILE - 1 : count - 1;
   const int key_end = start + last_q + 1;
-  int key_begin = 0;
-  if (window > 0 && start + q0 - window + 1 > 0) key_begin = start + q0 - window + 1;
+  const int key_begin = first_visible_key(start + q0, window);
 
   // the tile's queries; rows beyond the item's tokens are zeros and never stored
   for (int index = tid; index < AF_TILE * d4; index += 256) {
@@ -71,9 +70,12 @@ __global__ __launch_bounds__(256) void attention_tiled_f32_kernel(
     *reinterpret_cast<float4*>(&s_q[row * STRIDE + 4 * f]) = value;
   }
 
-  int q_pos[4];
+  int q_pos[4], q_first[4];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) q_pos[i] = q0 + 4 * ty + i < count ? start + q0 + 4 * ty + i : -1;
+  for (int i = 0; i < 4; ++i) {
+    q_pos[i] = q0 + 4 * ty + i < count ? start + q0 + 4 * ty + i : -1;
+    q_first[i] = q_pos[i] < 0 ? 0 : first_visible_key(q_pos[i], window);
+  }
   float run_max[4], run_sum[4];
   float4 acc[DV][4];
 #pragma unroll
@@ -145,7 +147,7 @@ __global__ __launch_bounds__(256) void attention_tiled_f32_kernel(
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         const int key = k0 + tx + 16 * j;
-        const bool visible = key_ok[j] && key <= q_pos[i] && (window <= 0 || q_pos[i] - key < window);
+        const bool visible = key_ok[j] && key <= q_pos[i] && key >= q_first[i];
         float score = s[i][j] * scale;
         if (extra.softcap > 0.f) score = capped_score(score, extra.softcap);
         s[i][j] = visible ? score : -INFINITY;
@@ -247,7 +249,7 @@ extern "C" int ps_attention_tiled_f32(const void* q, int64_t q_stride, const voi
              "(ps_attention_rowwise takes every size)", head_dim, AF_MAX_DIM);
   PS_REQUIRE(heads % kv_heads == 0,
              "ps_attention_tiled_f32: heads (%d) must be a multiple of kv_heads (%d)", heads, kv_heads);
-  PS_REQUIRE(window >= 0 && scale > 0.f, "ps_attention_tiled_f32: bad window or scale");
+  PS_REQUIRE(scale > 0.f, "ps_attention_tiled_f32: the score scale must be positive, got %g", scale);
   PS_REQUIRE((q_stride % 4) == 0 && (out_stride % 4) == 0 && ((uintptr_t)q % 16) == 0 &&
                  ((uintptr_t)out % 16) == 0 && ((uintptr_t)k_pool % 16) == 0 &&
                  ((uintptr_t)v_pool % 16) == 0,

@@ -199,6 +199,18 @@ __device__ inline float gelu_erf_f(float u) {
   return 0.5f * u * (1.0f + erff(u * 0.7071067811865476f));
 }
 
+// The gated unit act(g) * u of feed-forwards with two first matrices:
+//   g' = min(g, limit),  u' = clamp(u, -limit, limit),  g' sigmoid(slope g') (u' + shift)
+// (limit infinite, slope 1, shift 0: silu(g) * u).
+struct GateForm {
+  float limit, slope, shift;
+};
+__device__ inline float gated_unit(float g, float u, const GateForm form) {
+  g = fminf(g, form.limit);
+  u = fminf(fmaxf(u, -form.limit), form.limit);
+  return g / (1.0f + expf(-form.slope * g)) * (u + form.shift);
+}
+
 template <int EPI>
 __device__ inline float apply_activation(float v) {
   if (EPI == PS_EPI_GELU_TANH) return gelu_tanh_f(v);
@@ -208,6 +220,16 @@ __device__ inline float apply_activation(float v) {
     return r * r;
   }
   return v;
+}
+
+// The first key that the query at position `pos` sees; the last one is its own.  `window` says
+// which, in one number: > 0, the last `window` positions; 0, all of them; < 0, those of its own
+// chunk, the positions being cut into chunks of -window counted from position 0.  It never
+// falls as `pos` rises, which the tiled kernels rely on.
+__host__ __device__ inline int first_visible_key(int pos, int window) {
+  if (window > 0) return pos - window + 1 > 0 ? pos - window + 1 : 0;
+  if (window < 0) return pos - (int)((unsigned)pos % (unsigned)-window);
+  return 0;
 }
 
 // What an attention kernel may be given beside its operands: a sink (one float per head whose

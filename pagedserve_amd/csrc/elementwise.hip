@@ -52,15 +52,15 @@ int ps_compute_units() {
 // ---------------------------------------------------------------- embedding
 // h0[t] = scale * wte[id[t]] + wpe[pos[t]]  (reference: src/model/paged_decoder.py:306-314,
 // where the scale is 1); with norm_gamma, the row is then RMS-normed in float in the same
-// launch: h0 <- h0 / sqrt(mean(h0^2) + eps) * norm_gamma.
+// launch: h0 <- h0 / sqrt(mean(h0^2) + eps) * norm_gamma.  `copy`: the rows are written there too.
 // The id of token t is ids[t], or carried[src[t]] where src[t] >= 0: a token that an earlier
 // step chose on the device and that the host has not seen yet.
 template <typename T>
 __global__ void embed_kernel(const T* __restrict__ table, const T* __restrict__ pos_table,
                              const int* __restrict__ ids, const int* __restrict__ src,
                              const int* __restrict__ carried, const int* __restrict__ positions,
-                             float* __restrict__ out, int width, int vocab, float scale,
-                             const float* __restrict__ norm_gamma, float norm_eps) {
+                             float* __restrict__ out, float* __restrict__ copy, int width, int vocab,
+                             float scale, const float* __restrict__ norm_gamma, float norm_eps) {
   __shared__ float scratch[16];
   const int t = blockIdx.x;
   int id = ids[t];
@@ -78,16 +78,19 @@ __global__ void embed_kernel(const T* __restrict__ table, const T* __restrict__ 
   } else {
     for (int i = threadIdx.x; i < width; i += blockDim.x) dst[i] = to_float<T>(row[i]) * scale;
   }
-  if (norm_gamma == nullptr) return;
   // (each thread reads back what it wrote itself)
-  float sum = 0.f;
-  for (int i = threadIdx.x; i < width; i += blockDim.x) sum = fmaf(dst[i], dst[i], sum);
-  const float inv = 1.0f / sqrtf(block_sum(sum, scratch) / (float)width + norm_eps);
-  for (int i = threadIdx.x; i < width; i += blockDim.x) dst[i] = dst[i] * inv * norm_gamma[i];
+  if (norm_gamma != nullptr) {
+    float sum = 0.f;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) sum = fmaf(dst[i], dst[i], sum);
+    const float inv = 1.0f / sqrtf(block_sum(sum, scratch) / (float)width + norm_eps);
+    for (int i = threadIdx.x; i < width; i += blockDim.x) dst[i] = dst[i] * inv * norm_gamma[i];
+  }
+  if (copy != nullptr)
+    for (int i = threadIdx.x; i < width; i += blockDim.x) copy[(int64_t)t * width + i] = dst[i];
 }
 
 extern "C" int ps_embed(const void* table, const void* pos_table, const int* ids, const int* src,
-                        const int* carried, const int* positions, float* out, int tokens,
+                        const int* carried, const int* positions, float* out, float* copy, int tokens,
                         int width, int vocab, int max_positions, float scale,
                         const float* norm_gamma, float norm_eps, int dtype, void* stream) {
   PS_REQUIRE(tokens >= 0 && width > 0 && vocab > 0, "ps_embed: bad sizes (tokens %d, width %d)",
@@ -101,12 +104,12 @@ extern "C" int ps_embed(const void* table, const void* pos_table, const int* ids
   hipStream_t s = (hipStream_t)stream;
   if (dtype == PS_F32)
     hipLaunchKernelGGL(embed_kernel<float>, dim3(tokens), dim3(threads), 0, s, (const float*)table,
-                       (const float*)pos_table, ids, src, carried, positions, out, width, vocab,
+                       (const float*)pos_table, ids, src, carried, positions, out, copy, width, vocab,
                        scale, norm_gamma, norm_eps);
   else
     hipLaunchKernelGGL(embed_kernel<bf16_t>, dim3(tokens), dim3(threads), 0, s,
                        (const bf16_t*)table, (const bf16_t*)pos_table, ids, src, carried,
-                       positions, out, width, vocab, scale, norm_gamma, norm_eps);
+                       positions, out, copy, width, vocab, scale, norm_gamma, norm_eps);
   PS_CHECK_LAUNCH("ps_embed");
   return 0;
 }

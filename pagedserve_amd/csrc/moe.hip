@@ -11,7 +11,11 @@
 // added to the scores for the choice only (the weights use the scores without it; closed
 // experts count as minus infinity, since corrected scores may be negative); a group's score as
 // the sum of its `group_top` largest choice scores; weights divided by their sum (+ 1e-20).
-// Option of the experts: the plain form W_down,e relu(W_up,e x)^2 with one first matrix.
+// (weights as softmax over the chosen experts' logits alone: score 2, where the choice is by the
+// logits themselves).
+// Options of the experts: other constants of the gated unit (common.h: GateForm); the plain form
+// W_down,e relu(W_up,e x)^2 with one first matrix; one more expert, of an inner width and constants
+// of its own, that every token uses, with the weight one or sigmoid of a row's product with x.
 #include <math.h>
 
 #include "common.h"
@@ -21,13 +25,14 @@
 
 // What a router does beyond the softmax choice.
 struct RouteOptions {
-  int sigmoid;                 // scores are sigmoid(z) instead of softmax(z)
+  int score;                   // s: 0 softmax(z), 1 sigmoid(z), 2 z itself, the weights softmax over the chosen
   const float* correction;     // added to the scores for the choice (null: none)
   int group_top;               // a group's score: the sum of this many largest choice scores
   int normalise;               // the chosen weights are divided by their sum
-  int fixed;                   // experts behind the routed ones that every token uses with weight 1:
-                               // a row of ids and weights is [top chosen | fixed], the fixed ones
-                               // numbered from `experts` on
+  int fixed;                   // 1: a row of ids and weights is [top chosen | the expert numbered
+                               // `experts`, which every token uses], else [top chosen]
+  const float* gate;           // a row of the width: that expert's weight is sigmoid(gate . x) (null: 1)
+  float* gate_out;             // without `fixed`: where sigmoid(gate . x) of each token goes instead
 };
 
 // The sum of the `count` largest of choice[first .. first + size - 1].  The numbers are walked in
@@ -84,22 +89,24 @@ __global__ __launch_bounds__(64) void moe_route_kernel(
     const T* __restrict__ x, int64_t x_ld, const float* __restrict__ w, int width, int experts,
     int groups, int keep, int top, float scale, RouteOptions options, int* __restrict__ ids,
     float* __restrict__ weights) {
-  __shared__ float s_score[MOE_MAX_EXPERTS];
+  __shared__ float s_score[MOE_MAX_EXPERTS + 1];
   __shared__ float s_choice[MOE_MAX_EXPERTS];
   __shared__ unsigned char s_open[MOE_MAX_EXPERTS];
   const int64_t t = blockIdx.x;
   const int lane = threadIdx.x;
   const T* row = x + t * x_ld;
-  for (int e = 0; e < experts; ++e) {
-    const float sum = wave_sum(router_dot<T>(row, w + (int64_t)e * width, width, lane));
+  const int rows = experts + (options.gate != nullptr ? 1 : 0);
+  for (int e = 0; e < rows; ++e) {
+    const float* w_row = e < experts ? w + (int64_t)e * width : options.gate;
+    const float sum = wave_sum(router_dot<T>(row, w_row, width, lane));
     if (lane == 0) s_score[e] = sum;
   }
   __syncthreads();
   if (lane != 0) return;
   const int cols = top + options.fixed;
-  if (options.sigmoid) {
+  if (options.score == 1) {
     for (int e = 0; e < experts; ++e) s_score[e] = 1.0f / (1.0f + expf(-s_score[e]));
-  } else {
+  } else if (options.score == 0) {
     float top_z = -INFINITY;
     for (int e = 0; e < experts; ++e) top_z = fmaxf(top_z, s_score[e]);
     float total = 0.f;
@@ -149,11 +156,26 @@ __global__ __launch_bounds__(64) void moe_route_kernel(
     weights[t * cols + j] = own;
     chosen_sum += own;
   }
-  const float factor = options.normalise ? scale / (chosen_sum + 1e-20f) : scale;
-  for (int j = 0; j < top; ++j) weights[t * cols + j] *= factor;
-  for (int j = 0; j < options.fixed; ++j) {
-    ids[t * cols + top + j] = experts + j;
-    weights[t * cols + top + j] = 1.0f;
+  if (options.score == 2) {
+    float top_z = -INFINITY;
+    for (int j = 0; j < top; ++j) top_z = fmaxf(top_z, weights[t * cols + j]);
+    chosen_sum = 0.f;
+    for (int j = 0; j < top; ++j) {
+      const float p = expf(weights[t * cols + j] - top_z);
+      weights[t * cols + j] = p;
+      chosen_sum += p;
+    }
+    for (int j = 0; j < top; ++j) weights[t * cols + j] *= scale / chosen_sum;
+  } else {
+    const float factor = options.normalise ? scale / (chosen_sum + 1e-20f) : scale;
+    for (int j = 0; j < top; ++j) weights[t * cols + j] *= factor;
+  }
+  const float gate = options.gate != nullptr ? 1.0f / (1.0f + expf(-s_score[experts])) : 1.0f;
+  if (options.fixed) {
+    ids[t * cols + top] = experts;
+    weights[t * cols + top] = gate;
+  } else if (options.gate_out != nullptr) {
+    options.gate_out[t] = gate;
   }
 }
 
@@ -165,22 +187,27 @@ __global__ __launch_bounds__(256) void moe_route_wave_kernel(
     const T* __restrict__ x, int64_t x_ld, const float* __restrict__ w, int width, int experts,
     int groups, int keep, int top, float scale, RouteOptions options, int* __restrict__ ids,
     float* __restrict__ weights) {
-  __shared__ float s_score[64];
+  __shared__ float s_score[65];
   __shared__ float s_group[64];
   const int64_t t = blockIdx.x;
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
   const T* row = x + t * x_ld;
-  for (int e = wave; e < experts; e += 4) {
-    const float sum = wave_sum(router_dot<T>(row, w + (int64_t)e * width, width, lane));
+  const int rows = experts + (options.gate != nullptr ? 1 : 0);
+  for (int e = wave; e < rows; e += 4) {
+    const float* w_row = e < experts ? w + (int64_t)e * width : options.gate;
+    const float sum = wave_sum(router_dot<T>(row, w_row, width, lane));
     if (lane == 0) s_score[e] = sum;
   }
   __syncthreads();
   // (all four waves choose, from the same numbers; the first one writes)
   const bool mine = lane < experts;
   const float z = mine ? s_score[lane] : -INFINITY;
+  const float gate_z = options.gate != nullptr ? s_score[experts] : 0.f;
   __syncthreads();
   float score;
-  if (options.sigmoid) {
+  if (options.score == 2) {
+    score = mine ? z : 0.f;
+  } else if (options.score == 1) {
     score = mine ? 1.0f / (1.0f + expf(-z)) : 0.f;
   } else {
     const float p = mine ? expf(z - wave_max(z)) : 0.f;
@@ -218,26 +245,47 @@ __global__ __launch_bounds__(256) void moe_route_wave_kernel(
       if (wave == 0) ids[t * cols + j] = chosen;
     }
   }
-  const float own = (slot >= 0 && score == score) ? score : 0.f;
+  float own = (slot >= 0 && score == score) ? score : 0.f;
+  if (options.score == 2) {
+    const float top_z = wave_max(slot >= 0 ? own : -INFINITY);
+    own = slot >= 0 ? expf(own - top_z) : 0.f;
+  }
   const float chosen_sum = wave_sum(own);
   if (slot >= 0 && wave == 0) {
-    weights[t * cols + slot] = options.normalise ? own / (chosen_sum + 1e-20f) * scale : own * scale;
+    const bool normed = options.normalise || options.score == 2;
+    weights[t * cols + slot] = normed ? own / (chosen_sum + 1e-20f) * scale : own * scale;
   }
-  if (wave == 1 && lane < options.fixed) {
-    ids[t * cols + top + lane] = experts + lane;
-    weights[t * cols + top + lane] = 1.0f;
+  if (wave == 1 && lane == 0 && (options.fixed || options.gate_out != nullptr)) {
+    const float gate = options.gate != nullptr ? 1.0f / (1.0f + expf(-gate_z)) : 1.0f;
+    if (options.fixed) {
+      ids[t * cols + top] = experts;
+      weights[t * cols + top] = gate;
+    } else {
+      options.gate_out[t] = gate;
+    }
   }
 }
 
-// What a hidden column becomes: silu(g) * u of the gated form, relu(g)^2 of the plain one.
+// What a hidden column becomes: the gated unit of the gated form, relu(g)^2 of the plain one.
 template <bool GATED>
-__device__ inline float moe_activation(float g, float u) {
-  if (GATED) return g / (1.0f + expf(-g)) * u;
+__device__ inline float moe_activation(float g, float u, const GateForm form) {
+  if (GATED) return gated_unit(g, u, form);
   const float r = fmaxf(g, 0.f);
   return r * r;
 }
 
-// hidden[(t, j), c] = silu(W_gate,e[c] . x_t) * (W_up,e[c] . x_t) for e = ids[t, j].  The
+// The expert that every token uses beside the routed ones, in the row kernels: it is the last of a
+// token's choices (inner 0: there is none).  A token's hidden rows lie one behind the other,
+// [routed choices][inner] and then this expert's.
+template <typename T>
+struct ExtraExpert {
+  const T* w1;         // as an expert's first matrices, of its own inner width
+  const T* w2;         // [width][inner]
+  int inner;
+  GateForm form;
+};
+
+// hidden[(t, j), c] = unit(W_gate,e[c] . x_t, W_up,e[c] . x_t) for e = ids[t, j].  The
 // experts' first matrices lie one behind the other, [experts][gate rows | up rows][width].
 // A block of four waves per (token, choice) and 4 * ROWS hidden columns; the lanes share a dot
 // product's width.  GATED false: the plain form, hidden = relu(W_up,e[c] . x_t)^2, the experts' first
@@ -245,16 +293,19 @@ __device__ inline float moe_activation(float g, float u) {
 template <typename T, int ROWS, bool GATED>
 __global__ __launch_bounds__(256) void moe_hidden_kernel(
     const T* __restrict__ x, int64_t x_ld, const T* __restrict__ w1, const int* __restrict__ ids,
-    T* __restrict__ hidden, int width, int inner, int experts, const T* __restrict__ w1x) {
+    T* __restrict__ hidden, int width, int inner, GateForm form, const ExtraExpert<T> extra) {
   extern __shared__ float s_x[];
   // (blockIdx.x: the token, blockIdx.z: which of its choices)
-  const int64_t row_index = (int64_t)blockIdx.x * gridDim.z + blockIdx.z;
-  int e = ids[row_index];
-  // (experts numbered from `experts` on lie in a tensor of their own)
-  if (e >= experts) {
-    e = w1x != nullptr ? e - experts : 0;
-    if (w1x != nullptr) w1 = w1x;
+  int e = ids[(int64_t)blockIdx.x * gridDim.z + blockIdx.z];
+  const int routed = extra.inner > 0 ? gridDim.z - 1 : gridDim.z;
+  T* own = hidden + (int64_t)blockIdx.x * (routed * inner + extra.inner) + (int64_t)blockIdx.z * inner;
+  if ((int)blockIdx.z == routed) {
+    e = 0;
+    w1 = extra.w1;
+    inner = extra.inner;
+    form = extra.form;
   }
+  if ((int)blockIdx.y * 4 * ROWS >= inner) return;     // (the grid is cut for the wider of the two)
   const T* x_row = x + (int64_t)blockIdx.x * x_ld;
   for (int d = threadIdx.x; d < width; d += 256) s_x[d] = to_float<T>(x_row[d]);
   __syncthreads();
@@ -273,7 +324,7 @@ __global__ __launch_bounds__(256) void moe_hidden_kernel(
     }
     g = wave_sum(g);
     if (GATED) u = wave_sum(u);
-    if (lane == 0) hidden[row_index * inner + c] = from_float<T>(moe_activation<GATED>(g, u));
+    if (lane == 0) own[c] = from_float<T>(moe_activation<GATED>(g, u, form));
   }
 }
 
@@ -283,11 +334,12 @@ template <typename T, int ROWS>
 __global__ __launch_bounds__(256) void moe_down_kernel(
     const T* __restrict__ hidden, const T* __restrict__ w2, const int* __restrict__ ids,
     const float* __restrict__ weights, float* __restrict__ y, int width, int inner, int top,
-    int experts, const T* __restrict__ w2x) {
-  extern __shared__ float s_h[];        // [top][inner]
+    const ExtraExpert<T> extra) {
+  extern __shared__ float s_h[];        // [routed choices][inner], then the extra expert's
   const int64_t t = blockIdx.x;
-  for (int i = threadIdx.x; i < top * inner; i += 256)
-    s_h[i] = to_float<T>(hidden[t * top * inner + i]);
+  const int routed = extra.inner > 0 ? top - 1 : top;
+  const int held = routed * inner + extra.inner;
+  for (int i = threadIdx.x; i < held; i += 256) s_h[i] = to_float<T>(hidden[t * held + i]);
   __syncthreads();
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
   const int first = (blockIdx.y * 4 + wave) * ROWS;
@@ -296,12 +348,12 @@ __global__ __launch_bounds__(256) void moe_down_kernel(
     if (d >= width) break;
     float total = 0.f;
     for (int j = 0; j < top; ++j) {
-      const int e = ids[t * top + j];
-      const T* w_row = (e < experts || w2x == nullptr)
-                           ? w2 + ((int64_t)(e < experts ? e : 0) * width + d) * inner
-                           : w2x + ((int64_t)(e - experts) * width + d) * inner;
+      const bool is_extra = j == routed;
+      const int columns = is_extra ? extra.inner : inner;
+      const T* w_row = is_extra ? extra.w2 + (int64_t)d * columns
+                                : w2 + ((int64_t)ids[t * top + j] * width + d) * inner;
       float sum = 0.f;
-      for (int c = lane; c < inner; c += 64) sum = fmaf(to_float<T>(w_row[c]), s_h[j * inner + c], sum);
+      for (int c = lane; c < columns; c += 64) sum = fmaf(to_float<T>(w_row[c]), s_h[j * inner + c], sum);
       total = fmaf(weights[t * top + j], wave_sum(sum), total);
     }
     if (lane == 0) y[t * width + d] += total;
@@ -309,9 +361,10 @@ __global__ __launch_bounds__(256) void moe_down_kernel(
 }
 
 extern "C" int ps_moe_route(const void* x, int64_t x_ld, const float* w, int tokens, int width,
-                            int experts, int groups, int keep, int top, float scale, int sigmoid,
-                            const float* correction, int group_top, int normalise, int fixed, int* ids,
-                            float* weights, int dtype, void* stream) {
+                            int experts, int groups, int keep, int top, float scale, int score,
+                            const float* correction, int group_top, int normalise, int fixed,
+                            const float* gate, float* gate_out, int* ids, float* weights, int dtype,
+                            void* stream) {
   PS_REQUIRE(tokens >= 0 && width > 0 && experts > 0 && experts <= MOE_MAX_EXPERTS,
              "ps_moe_route: %d experts, at most %d", experts, MOE_MAX_EXPERTS);
   PS_REQUIRE(groups >= 1 && experts % groups == 0 && keep >= 1 && keep <= groups,
@@ -323,8 +376,11 @@ extern "C" int ps_moe_route(const void* x, int64_t x_ld, const float* w, int tok
              "ps_moe_route: a group's score sums its %d largest scores, 1 to 8 are taken", group_top);
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-  PS_REQUIRE(fixed >= 0 && fixed <= 64, "ps_moe_route: %d fixed experts, up to 64 are taken", fixed);
-  const RouteOptions options = {sigmoid, correction, group_top, normalise, fixed};
+  PS_REQUIRE(score >= 0 && score <= 2, "ps_moe_route: score %d (0: softmax, 1: sigmoid, 2: softmax over the chosen)", score);
+  PS_REQUIRE(fixed == 0 || fixed == 1, "ps_moe_route: %d experts for every token, one at most", fixed);
+  PS_REQUIRE(gate_out == nullptr || (gate != nullptr && !fixed),
+             "ps_moe_route: gates go to rows of their own only without a fixed expert");
+  const RouteOptions options = {score, correction, group_top, normalise, fixed, gate, gate_out};
   if (experts <= 64) {
     if (dtype == PS_F32)
       hipLaunchKernelGGL(moe_route_wave_kernel<float>, dim3(tokens), dim3(256), 0, s, (const float*)x,
@@ -370,14 +426,18 @@ __device__ inline void load8<float>(const float* p, float (&v)[8]) {
 template <typename T, int ROWS, bool GATED>
 __global__ __launch_bounds__(256) void moe_hidden_wide_kernel(
     const T* __restrict__ x, int64_t x_ld, const T* __restrict__ w1, const int* __restrict__ ids,
-    T* __restrict__ hidden, int width, int inner, int experts, const T* __restrict__ w1x) {
+    T* __restrict__ hidden, int width, int inner, GateForm form, const ExtraExpert<T> extra) {
   extern __shared__ float s_x[];
-  const int64_t row_index = (int64_t)blockIdx.x * gridDim.z + blockIdx.z;
-  int e = ids[row_index];
-  if (e >= experts) {
-    e = w1x != nullptr ? e - experts : 0;
-    if (w1x != nullptr) w1 = w1x;
+  int e = ids[(int64_t)blockIdx.x * gridDim.z + blockIdx.z];
+  const int routed = extra.inner > 0 ? gridDim.z - 1 : gridDim.z;
+  T* own = hidden + (int64_t)blockIdx.x * (routed * inner + extra.inner) + (int64_t)blockIdx.z * inner;
+  if ((int)blockIdx.z == routed) {
+    e = 0;
+    w1 = extra.w1;
+    inner = extra.inner;
+    form = extra.form;
   }
+  if ((int)blockIdx.y * 4 * ROWS >= inner) return;
   const T* x_row = x + (int64_t)blockIdx.x * x_ld;
   for (int d = threadIdx.x; d < width; d += 256) s_x[d] = to_float<T>(x_row[d]);
   __syncthreads();
@@ -414,7 +474,7 @@ __global__ __launch_bounds__(256) void moe_hidden_wide_kernel(
   for (int r = 0; r < ROWS; ++r) {
     const float gs = wave_sum(g[r]), us = GATED ? wave_sum(u[r]) : 0.f;
     if (lane == 0 && first + r < inner)
-      hidden[row_index * inner + first + r] = from_float<T>(moe_activation<GATED>(gs, us));
+      own[first + r] = from_float<T>(moe_activation<GATED>(gs, us, form));
   }
 }
 
@@ -423,11 +483,12 @@ template <typename T, int ROWS>
 __global__ __launch_bounds__(256) void moe_down_wide_kernel(
     const T* __restrict__ hidden, const T* __restrict__ w2, const int* __restrict__ ids,
     const float* __restrict__ weights, float* __restrict__ y, int width, int inner, int top,
-    int experts, const T* __restrict__ w2x) {
-  extern __shared__ float s_h[];        // [top][inner]
+    const ExtraExpert<T> extra) {
+  extern __shared__ float s_h[];        // [routed choices][inner], then the extra expert's
   const int64_t t = blockIdx.x;
-  for (int i = threadIdx.x; i < top * inner; i += 256)
-    s_h[i] = to_float<T>(hidden[t * top * inner + i]);
+  const int routed = extra.inner > 0 ? top - 1 : top;
+  const int held = routed * inner + extra.inner;
+  for (int i = threadIdx.x; i < held; i += 256) s_h[i] = to_float<T>(hidden[t * held + i]);
   __syncthreads();
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
   const int first = (blockIdx.y * 4 + wave) * ROWS;
@@ -436,7 +497,9 @@ __global__ __launch_bounds__(256) void moe_down_wide_kernel(
 #pragma unroll
   for (int r = 0; r < ROWS; ++r) total[r] = 0.f;
   for (int j = 0; j < top; ++j) {
-    const int e = ids[t * top + j];
+    const bool is_extra = j == routed;
+    const int columns = is_extra ? extra.inner : inner;
+    const T* matrix = is_extra ? extra.w2 : w2 + (int64_t)ids[t * top + j] * width * inner;
     const float weight = weights[t * top + j];
     float sum[ROWS];
     const T* rows[ROWS];
@@ -444,10 +507,9 @@ __global__ __launch_bounds__(256) void moe_down_wide_kernel(
     for (int r = 0; r < ROWS; ++r) {
       sum[r] = 0.f;
       const int d = first + r < width ? first + r : width - 1;
-      rows[r] = (e < experts || w2x == nullptr) ? w2 + ((int64_t)(e < experts ? e : 0) * width + d) * inner
-                                                : w2x + ((int64_t)(e - experts) * width + d) * inner;
+      rows[r] = matrix + (int64_t)d * columns;
     }
-    for (int c = lane * 8; c < inner; c += 512) {
+    for (int c = lane * 8; c < columns; c += 512) {
       float hv[8];
 #pragma unroll
       for (int i = 0; i < 8; ++i) hv[i] = s_h[j * inner + c + i];
@@ -512,7 +574,7 @@ typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 moe_bf16x8;
 
 // A tile of 128 sorted pairs times 128 weight rows of the tile's expert, k in stages of 32.
 // HIDDEN: the weight rows are 64 gate rows and the 64 up rows of the same hidden columns, and
-// hidden[pair, column] = silu(gate) * up; the rows of A are the pairs' tokens (pair / top).
+// hidden[pair, column] = unit(gate, up); the rows of A are the pairs' tokens (pair / top).
 // MODE 2, the plain form's hidden rows: 128 up rows, hidden[pair, column] = relu(up)^2 (a tile of
 // pairs is staged once for twice the columns).
 // MODE 0: 64 output columns (so that the narrower product still gives every compute unit a
@@ -523,7 +585,7 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
     const bf16_t* __restrict__ a, int64_t lda, const bf16_t* __restrict__ w, int64_t expert_stride,
     int w_rows, int k, const int* __restrict__ order, const int* __restrict__ tile_expert, int top,
     const float* __restrict__ weights, bf16_t* __restrict__ hidden, float* __restrict__ out,
-    int64_t out_ld) {
+    int64_t out_ld, const GateForm form) {
   const int e = tile_expert[blockIdx.x];
   if (e < 0) return;
   __shared__ __attribute__((aligned(16))) unsigned char lds[2][(MOE_TILE + 128) * MOE_LDS_STRIDE];
@@ -643,13 +705,13 @@ __global__ __launch_bounds__(256) void moe_grouped_kernel(
     if (HIDDEN) {
       const int col = n0 + wave_n * 32 + (lane & 31);
       const float g = acc[r][0][i], u = acc[r][1][i];
-      if (col < columns) hidden[(int64_t)pair * columns + col] = from_float<bf16_t>(g / (1.0f + expf(-g)) * u);
+      if (col < columns) hidden[(int64_t)pair * columns + col] = from_float<bf16_t>(gated_unit(g, u, form));
     } else if (MODE == 2) {
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
         const int col = n0 + j * 64 + wave_n * 32 + (lane & 31);
         if (col < columns)
-          hidden[(int64_t)pair * columns + col] = from_float<bf16_t>(moe_activation<false>(acc[r][j][i], 0.f));
+          hidden[(int64_t)pair * columns + col] = from_float<bf16_t>(moe_activation<false>(acc[r][j][i], 0.f, form));
       }
     } else {
       const int col = n0 + wave_n * 32 + (lane & 31);
@@ -671,44 +733,52 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
 
 extern "C" int ps_moe_experts(const void* x, int64_t x_ld, const void* w1, const void* w2,
                               const int* ids, const float* weights, void* hidden, float* y,
-                              int tokens, int width, int inner, int top, int gated, int experts,
-                              const void* w1x, const void* w2x, int dtype, void* stream) {
+                              int tokens, int width, int inner, int top, int gated, float limit,
+                              float slope, float shift, const void* w1x, const void* w2x, int inner_x,
+                              float limit_x, int dtype, void* stream) {
   PS_REQUIRE(tokens >= 0 && width > 0 && inner > 0 && top > 0 && top <= 65535,
              "ps_moe_experts: bad sizes");
-  PS_REQUIRE((size_t)width * 4 <= 64 * 1024 && (size_t)top * inner * 4 <= 64 * 1024,
-             "ps_moe_experts: width %d or %d x %d hidden columns do not fit LDS", width, top, inner);
+  PS_REQUIRE(inner_x >= 0 && (inner_x == 0 || (top > 1 && w1x != nullptr && w2x != nullptr)),
+             "ps_moe_experts: an expert for every token needs its matrices and its place behind the chosen ones");
+  const int held = (inner_x > 0 ? top - 1 : top) * inner + inner_x;      // hidden columns of a token
+  PS_REQUIRE((size_t)width * 4 <= 64 * 1024 && (size_t)held * 4 <= 64 * 1024,
+             "ps_moe_experts: width %d or %d hidden columns of a token do not fit LDS", width, held);
+  PS_REQUIRE(limit > 0.f && (inner_x == 0 || limit_x > 0.f), "ps_moe_experts: limits must be positive");
   PS_REQUIRE(dtype == PS_F32 || dtype == PS_BF16, "ps_moe_experts: unknown dtype %d", dtype);
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-  const bool wide1 = width % 8 == 0 && x_ld % 8 == 0, wide2 = inner % 8 == 0;
+  const bool wide1 = width % 8 == 0 && x_ld % 8 == 0, wide2 = inner % 8 == 0 && inner_x % 8 == 0;
+  const int widest = inner > inner_x ? inner : inner_x;
+  const GateForm form = {limit, slope, shift};
   // hidden columns / output columns per wave: four, or two while that still leaves the chip
   // short of blocks (a handful of decoded tokens)
   const bool few = (int64_t)tokens * ((width + 15) / 16) < 4 * ps_compute_units();
 #define PS_MOE_HIDDEN(T, ROWS, GATED)                                                              \
   do {                                                                                             \
-    const dim3 grid1(tokens, (inner + 4 * ROWS - 1) / (4 * ROWS), top);                            \
+    const dim3 grid1(tokens, (widest + 4 * ROWS - 1) / (4 * ROWS), top);                            \
     if (wide1)                                                                                     \
       hipLaunchKernelGGL((moe_hidden_wide_kernel<T, ROWS, GATED>), grid1, dim3(256),               \
                          (size_t)width * 4, s, (const T*)x, x_ld, (const T*)w1, ids, (T*)hidden,   \
-                         width, inner, experts, (const T*)w1x);                                    \
+                         width, inner, form, extra);                                               \
     else                                                                                           \
       hipLaunchKernelGGL((moe_hidden_kernel<T, ROWS, GATED>), grid1, dim3(256), (size_t)width * 4, \
-                         s, (const T*)x, x_ld, (const T*)w1, ids, (T*)hidden, width, inner,        \
-                         experts, (const T*)w1x);                                                  \
+                         s, (const T*)x, x_ld, (const T*)w1, ids, (T*)hidden, width, inner, form,  \
+                         extra);                                                                   \
   } while (0)
 #define PS_MOE_ROWS(T, ROWS)                                                                       \
   do {                                                                                             \
+    const ExtraExpert<T> extra = {(const T*)w1x, (const T*)w2x, inner_x, {limit_x, slope, shift}}; \
     const dim3 grid2(tokens, (width + 4 * ROWS - 1) / (4 * ROWS));                                 \
     if (gated) PS_MOE_HIDDEN(T, ROWS, true);                                                       \
     else PS_MOE_HIDDEN(T, ROWS, false);                                                            \
     if (wide2)                                                                                     \
-      hipLaunchKernelGGL((moe_down_wide_kernel<T, ROWS>), grid2, dim3(256), (size_t)top * inner * 4, \
+      hipLaunchKernelGGL((moe_down_wide_kernel<T, ROWS>), grid2, dim3(256), (size_t)held * 4,     \
                          s, (const T*)hidden, (const T*)w2, ids, weights, y, width, inner, top,    \
-                         experts, (const T*)w2x);                                                  \
+                         extra);                                                                   \
     else                                                                                           \
-      hipLaunchKernelGGL((moe_down_kernel<T, ROWS>), grid2, dim3(256), (size_t)top * inner * 4, s, \
+      hipLaunchKernelGGL((moe_down_kernel<T, ROWS>), grid2, dim3(256), (size_t)held * 4, s,       \
                          (const T*)hidden, (const T*)w2, ids, weights, y, width, inner, top,       \
-                         experts, (const T*)w2x);                                                  \
+                         extra);                                                                   \
   } while (0)
   if (dtype == PS_F32) {
     if (few) PS_MOE_ROWS(float, 2);
@@ -731,13 +801,15 @@ extern "C" int ps_moe_experts_grouped(const void* x, int64_t x_ld, const void* w
                                       const int* ids, const float* weights, void* hidden,
                                       float* out, int* order, int* tile_expert, float* y,
                                       int tokens, int width, int inner, int experts, int top,
-                                      int gated, void* stream) {
+                                      int gated, float limit, float slope, float shift, void* stream) {
   PS_REQUIRE(tokens >= 0 && width > 0 && inner > 0 && top > 0 && experts > 0 &&
                  experts <= MOE_MAX_EXPERTS, "ps_moe_experts_grouped: bad sizes");
   PS_REQUIRE(width % 8 == 0 && inner % 8 == 0 && x_ld % 8 == 0,
              "ps_moe_experts_grouped: width %d and inner width %d must be multiples of 8", width, inner);
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
+  PS_REQUIRE(limit > 0.f, "ps_moe_experts_grouped: the limit must be positive");
+  const GateForm form = {limit, slope, shift};
   const int pairs = tokens * top;
   const int tiles = ps_moe_grouped_tiles(pairs, experts);
   hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(1024), 0, s, ids, pairs, experts, order, tile_expert,
@@ -746,16 +818,16 @@ extern "C" int ps_moe_experts_grouped(const void* x, int64_t x_ld, const void* w
     hipLaunchKernelGGL(moe_grouped_kernel<1>, dim3(tiles, (inner + 63) / 64), dim3(256), 0, s,
                        (const bf16_t*)x, x_ld, (const bf16_t*)w1, (int64_t)2 * inner * width, 2 * inner,
                        width, order, tile_expert, top, weights, (bf16_t*)hidden, (float*)nullptr,
-                       (int64_t)0);
+                       (int64_t)0, form);
   else
     hipLaunchKernelGGL(moe_grouped_kernel<2>, dim3(tiles, (inner + 127) / 128), dim3(256), 0, s,
                        (const bf16_t*)x, x_ld, (const bf16_t*)w1, (int64_t)inner * width, inner,
                        width, order, tile_expert, top, weights, (bf16_t*)hidden, (float*)nullptr,
-                       (int64_t)0);
+                       (int64_t)0, form);
   hipLaunchKernelGGL(moe_grouped_kernel<0>, dim3(tiles, (width + 63) / 64), dim3(256), 0, s,
                      (const bf16_t*)hidden, (int64_t)inner, (const bf16_t*)w2, (int64_t)width * inner,
                      width, inner, order, tile_expert, top, weights, (bf16_t*)nullptr, out,
-                     (int64_t)width);
+                     (int64_t)width, form);
   hipLaunchKernelGGL(moe_combine_kernel, dim3(tokens), dim3(256), 0, s, out, y, width, top);
   PS_CHECK_LAUNCH("ps_moe_experts_grouped");
   return 0;

@@ -24,7 +24,7 @@ int ps_device_info(int* compute_units, int* lds_bytes, char* arch, int arch_len)
 // where id(t) = ids[t], or carried[src[t]] if src is given and src[t] >= 0.  norm_gamma (null:
 // none): the row is then RMS-normed, out / sqrt(mean(out^2) + norm_eps) * norm_gamma.
 int ps_embed(const void* table, const void* pos_table, const int* ids, const int* src,
-             const int* carried, const int* positions, float* out, int tokens, int width,
+             const int* carried, const int* positions, float* out, float* copy, int tokens, int width,
              int vocab, int max_positions, float scale, const float* norm_gamma, float norm_eps,
              int dtype, void* stream);
 
@@ -114,8 +114,9 @@ int ps_kv_write(const void* k, const void* v, int64_t stride, void* k_pool, void
                 void* stream);
 
 // Attention of `tokens` tokens of the step (those listed in tok_list, or all when it is
-// null) over their requests' cached keys 0..position (or the last `window` of them), one
-// wave per (token, head).  Any head_dim from 1 to 256; heads must be a multiple of kv_heads.
+// null) over their requests' cached keys up to their own position, one wave per (token, head).
+// window says which of them: > 0, the last `window`; 0, all; < 0, those of the token's own chunk
+// (positions cut into chunks of -window from 0 on).  The same in the attention kernels below.  Any head_dim from 1 to 256; heads must be a multiple of kv_heads.
 // sink: null, or one float per head that enters the softmax's denominator as exp(sink[head])
 // (a score without key or value, not scaled); gate: null, or a float per token and head, rows
 // gate_ld apart: the output of token t and head h is multiplied by sigmoid(gate[t * gate_ld + h]);
@@ -294,13 +295,15 @@ int ps_attention_prepare(const float* proj, int64_t ld, int q_col, int k_col, in
                          int store, int q_dim, int q_maps, int dtype, void* stream);
 // The same step for layers that treat every head on its own: the first rot_dims dimensions of
 // each query and key head rotated (halves != 0: dimension i with i + rot_dims / 2, else 2i with
-// 2i + 1; cosine and sine times magnitude), then, with head_norm, every head divided by its root
-// mean square over key_dim (no weight); values: the columns at v_col as projected (v_col may be
+// 2i + 1; cosine and sine times magnitude); head_norm: every head divided by its root mean square
+// over key_dim and multiplied by q_gamma / k_gamma (a float per dimension, null for ones), 1 behind
+// the rotation, 2 ahead of it, 0 not at all; values: the columns at v_col as projected (v_col may be
 // k_col: values that are the keys before rotation and norm).  cache_dim up to 256.
 int ps_attention_prepare_heads(const float* proj, int64_t ld, int q_col, int k_col, int v_col,
                                void* q_out, int64_t q_stride, void* k_pool, void* v_pool,
                                const float* freqs, int rot_dims, int halves, float magnitude,
-                               int head_norm, float eps, const int* tok_item, const int* tok_pos,
+                               int head_norm, const float* q_gamma, const float* k_gamma, float eps,
+                               const int* tok_item, const int* tok_pos,
                                const int* tables, int table_width, int tokens, int heads,
                                int kv_heads, int key_dim, int value_dim, int cache_dim,
                                int page_size, int num_pages, int dtype, void* stream);
@@ -386,15 +389,19 @@ int ps_selective_scan(const void* x, const float* dt, const float* bc, int64_t b
                       const float* step_bias, int low_col, int rank, int dtype, void* stream);
 
 // ---- a stream whose sublayers add into a scratch row ------------------------------------------
-// h += factor * column_scale * y + bias (y, bias: null for none; column_scale: a float per
-// column, null for ones); zero[...] = 0 (may be y); if gamma:
-// normed = h / sqrt(mean(h^2) + eps) * gamma.
+// h += factor * column_scale * y + rows + bias (y, rows: a float row per token, bias: one row for
+// all; null for none; column_scale: a float per column, null for ones); zero[...] = 0 (may be y);
+// if gamma: normed = h / sqrt(mean(h^2) + eps) * gamma; if gamma2: normed2 = the same * gamma2.
 int ps_stream_step(float* h, const float* y, float factor, const float* column_scale,
-                   const float* bias, const float* gamma, float eps, void* normed, float* zero,
-                   int tokens, int width, int out_dtype, void* stream);
-// out[t, c] = silu(gu[t * ld + c]) * gu[t * ld + inner + c].
+                   const float* rows, const float* bias, const float* gamma, float eps, void* normed,
+                   const float* gamma2, void* normed2, float* zero, int tokens, int width,
+                   int out_dtype, void* stream);
+// out[t, c] = unit(gu[t * ld + c], gu[t * ld + inner + c]) (* row_scale[t], unless null) with
+// unit(g, u) = g' sigmoid(slope g') (u' + shift), g' = min(g, limit), u' = clamp(u, -limit, limit):
+// silu(g) * u for an infinite limit, slope 1 and shift 0.  activation 1: gelu_tanh(g) * u.
 int ps_silu_gate(const float* gu, int64_t ld, void* out, int64_t out_ld, int tokens, int inner,
-                 int activation, int dtype, void* stream);
+                 int activation, float limit, float slope, float shift, const float* row_scale,
+                 int dtype, void* stream);
 // p[t * ld + first + c] = silu(...) in place for c < count.
 int ps_silu_columns(float* p, int64_t ld, int first, int count, int tokens, void* stream);
 // y += share * (rms_norm(a) * wa + rms_norm(b) * wb) over rows of width floats; a and b are cleared.
@@ -425,18 +432,27 @@ int ps_lru_scan(const float* proj, int64_t ld, int y_col, int x_col, const float
 
 // ---- mixture of experts ------------------------------------------------------------------------
 // ids / weights [tokens, top]: the experts that each row of x chooses and s * scale of each
-// (softmax over all experts of the 32-bit logits w x; only experts of the keep best of groups
-// equal groups of neighbours, a group's score being its largest s).
+// (score 0: softmax over all experts of the 32-bit logits w x, 1: their sigmoid, 2: the logits, the
+// weights then being the softmax over the chosen ones; only experts of the keep best of groups
+// equal groups of neighbours, a group's score being the sum of its group_top largest s).  correction:
+// added to s for the choice only; normalise: weights divided by their sum before scale.  fixed 1: a
+// row has one more place, for the expert numbered `experts` that every token uses, with the weight
+// sigmoid(gate . x) (gate: a row of the width; null: weight 1); fixed 0: those weights go to
+// gate_out [tokens], unless null.
 int ps_moe_route(const void* x, int64_t x_ld, const float* w, int tokens, int width, int experts,
-                 int groups, int keep, int top, float scale, int sigmoid, const float* correction,
-                 int group_top, int normalise, int fixed, int* ids, float* weights, int dtype,
-                 void* stream);
-// y[t] += sum_j weights[t, j] W2[e] (silu(W1[e][:inner] x_t) * (W1[e][inner:] x_t)), e = ids[t, j];
-// w1: [experts, 2 * inner, width], w2: [experts, width, inner]; hidden: [tokens * top, inner] scratch.
+                 int groups, int keep, int top, float scale, int score, const float* correction,
+                 int group_top, int normalise, int fixed, const float* gate, float* gate_out, int* ids,
+                 float* weights, int dtype, void* stream);
+// y[t] += sum_j weights[t, j] W2[e] unit(W1[e][:inner] x_t, W1[e][inner:] x_t), e = ids[t, j], with
+// ps_silu_gate's unit; gated 0: W2[e] relu(W1[e] x_t)^2.
+// w1: [experts, 2 * inner, width], w2: [experts, width, inner].  inner_x > 0: the last of a token's
+// `top` places is an expert for every token of that inner width, w1x [2 * inner_x, width], w2x
+// [width, inner_x], with a limit of its own.  hidden: scratch of tokens * (inner per routed place +
+// inner_x).
 int ps_moe_experts(const void* x, int64_t x_ld, const void* w1, const void* w2, const int* ids,
                    const float* weights, void* hidden, float* y, int tokens, int width, int inner,
-                   int top, int gated, int experts, const void* w1x, const void* w2x, int dtype,
-                   void* stream);
+                   int top, int gated, float limit, float slope, float shift, const void* w1x,
+                   const void* w2x, int inner_x, float limit_x, int dtype, void* stream);
 // The same for many rows in bfloat16 (width and inner multiples of 8): the (token, choice) pairs
 // are sorted by expert into tiles of 128 and multiplied on the matrix cores.  order:
 // [tiles * 128] int and tile_expert: [tiles] int scratch with tiles = ps_moe_grouped_tiles(tokens *
@@ -445,7 +461,7 @@ int ps_moe_grouped_tiles(int pairs, int experts);
 int ps_moe_experts_grouped(const void* x, int64_t x_ld, const void* w1, const void* w2, const int* ids,
                            const float* weights, void* hidden, float* out, int* order,
                            int* tile_expert, float* y, int tokens, int width, int inner, int experts,
-                           int top, int gated, void* stream);
+                           int top, int gated, float limit, float slope, float shift, void* stream);
 
 // Differential attention behind the attention kernels: ctx holds two softmax maps per head over
 // the same values, cache_dim wide: map m of head h at head `m * heads + h` (map_major) or at head

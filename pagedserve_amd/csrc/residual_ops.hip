@@ -6,13 +6,14 @@
 #include "pagedserve_hip.h"
 
 // One pass over the stream's rows, every piece optional:
-//   h <- h + factor * column_scale * y + bias;   zero <- 0 (may be y);
-//   normed <- h / sqrt(mean(h^2) + eps) * gamma
+//   h <- h + factor * column_scale * y + rows + bias;   zero <- 0 (may be y);
+//   normed <- h / sqrt(mean(h^2) + eps) * gamma;   normed2 <- the same * gamma2
 // (column_scale: a float per column, null for ones).  A block per token.
 template <typename T>
 __global__ __launch_bounds__(256) void stream_step_kernel(
     float* __restrict__ h, const float* y, float factor, const float* __restrict__ column_scale,
-    const float* __restrict__ bias, const float* __restrict__ gamma, float eps, T* __restrict__ normed, float* zero, int width) {
+    const float* __restrict__ rows, const float* __restrict__ bias, const float* __restrict__ gamma, float eps,
+    T* __restrict__ normed, const float* __restrict__ gamma2, T* __restrict__ normed2, float* zero, int width) {
   __shared__ float scratch[16];
   const int64_t t = blockIdx.x;
   float* row = h + t * width;
@@ -20,29 +21,37 @@ __global__ __launch_bounds__(256) void stream_step_kernel(
   for (int d = threadIdx.x; d < width; d += blockDim.x) {
     float v = row[d];
     if (y != nullptr) v = fmaf(column_scale ? factor * column_scale[d] : factor, y[t * width + d], v);
+    if (rows != nullptr) v += rows[t * width + d];
     if (bias != nullptr) v += bias[d];
-    if (y != nullptr || bias != nullptr) row[d] = v;
+    if (y != nullptr || rows != nullptr || bias != nullptr) row[d] = v;
     if (zero != nullptr) zero[t * width + d] = 0.f;
     sum = fmaf(v, v, sum);
   }
   if (gamma == nullptr) return;
   const float inv = 1.0f / sqrtf(block_sum(sum, scratch) / (float)width + eps);
   // (each thread reads back what it wrote itself)
-  for (int d = threadIdx.x; d < width; d += blockDim.x)
-    normed[t * width + d] = from_float<T>(row[d] * inv * gamma[d]);
+  for (int d = threadIdx.x; d < width; d += blockDim.x) {
+    const float v = row[d] * inv;
+    normed[t * width + d] = from_float<T>(v * gamma[d]);
+    if (gamma2 != nullptr) normed2[t * width + d] = from_float<T>(v * gamma2[d]);
+  }
 }
 
-// out[t, c] = act(gu[t, c]) * gu[t, inner + c]; act: silu, or (GELU) the tanh form of gelu
+// out[t, c] = unit(gu[t, c], gu[t, inner + c]) (common.h: GateForm), or (GELU) gelu_tanh(gu[t, c]) *
+// gu[t, inner + c]; times row_scale[t] where that is given
 template <typename T, bool GELU>
 __global__ __launch_bounds__(256) void silu_gate_kernel(const float* __restrict__ gu, int64_t ld,
                                                         T* __restrict__ out, int64_t out_ld,
-                                                        int inner) {
+                                                        int inner, const GateForm form,
+                                                        const float* __restrict__ row_scale) {
   const int64_t t = blockIdx.x;
   const int c = blockIdx.y * 256 + threadIdx.x;
   if (c >= inner) return;
   const float g = gu[t * ld + c];
   const float u = gu[t * ld + inner + c];
-  out[t * out_ld + c] = from_float<T>((GELU ? gelu_tanh_f(g) : g / (1.0f + expf(-g))) * u);
+  float v = GELU ? gelu_tanh_f(g) * u : gated_unit(g, u, form);
+  if (row_scale != nullptr) v *= row_scale[t];
+  out[t * out_ld + c] = from_float<T>(v);
 }
 
 // p[t, c] <- silu(p[t, c]) for columns first .. first + count - 1 of rows ld floats apart
@@ -80,26 +89,30 @@ __global__ __launch_bounds__(256) void pair_norm_mix_kernel(
 }
 
 extern "C" int ps_stream_step(float* h, const float* y, float factor, const float* column_scale,
-                              const float* bias, const float* gamma, float eps, void* normed,
-                              float* zero, int tokens, int width, int out_dtype, void* stream) {
+                              const float* rows, const float* bias, const float* gamma, float eps,
+                              void* normed, const float* gamma2, void* normed2, float* zero, int tokens,
+                              int width, int out_dtype, void* stream) {
   PS_REQUIRE(tokens >= 0 && width > 0, "ps_stream_step: bad sizes");
   PS_REQUIRE(gamma == nullptr || (normed != nullptr && eps > 0.f),
              "ps_stream_step: a norm needs an output and a positive eps");
+  PS_REQUIRE(gamma2 == nullptr || (gamma != nullptr && normed2 != nullptr),
+             "ps_stream_step: a second scale goes with the first and needs an output");
   PS_REQUIRE(out_dtype == PS_F32 || out_dtype == PS_BF16, "ps_stream_step: unknown dtype %d", out_dtype);
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   if (out_dtype == PS_F32)
     hipLaunchKernelGGL(stream_step_kernel<float>, dim3(tokens), dim3(256), 0, s, h, y, factor,
-                       column_scale, bias, gamma, eps, (float*)normed, zero, width);
+                       column_scale, rows, bias, gamma, eps, (float*)normed, gamma2, (float*)normed2, zero, width);
   else
     hipLaunchKernelGGL(stream_step_kernel<bf16_t>, dim3(tokens), dim3(256), 0, s, h, y, factor,
-                       column_scale, bias, gamma, eps, (bf16_t*)normed, zero, width);
+                       column_scale, rows, bias, gamma, eps, (bf16_t*)normed, gamma2, (bf16_t*)normed2, zero, width);
   PS_CHECK_LAUNCH("ps_stream_step");
   return 0;
 }
 
 extern "C" int ps_silu_gate(const float* gu, int64_t ld, void* out, int64_t out_ld, int tokens,
-                            int inner, int activation, int dtype, void* stream) {
+                            int inner, int activation, float limit, float slope, float shift,
+                            const float* row_scale, int dtype, void* stream) {
   PS_REQUIRE(tokens >= 0 && inner > 0 && ld >= 2 * (int64_t)inner && out_ld >= inner,
              "ps_silu_gate: bad sizes");
   PS_REQUIRE(dtype == PS_F32 || dtype == PS_BF16, "ps_silu_gate: unknown dtype %d", dtype);
@@ -107,14 +120,16 @@ extern "C" int ps_silu_gate(const float* gu, int64_t ld, void* out, int64_t out_
   hipStream_t s = (hipStream_t)stream;
   const dim3 grid(tokens, (inner + 255) / 256);
   PS_REQUIRE(activation == 0 || activation == 1, "ps_silu_gate: activation %d (0: silu, 1: gelu_tanh)", activation);
+  PS_REQUIRE(limit > 0.f, "ps_silu_gate: the limit must be positive");
+  const GateForm form = {limit, slope, shift};
   if (dtype == PS_F32 && activation)
-    hipLaunchKernelGGL((silu_gate_kernel<float, true>), grid, dim3(256), 0, s, gu, ld, (float*)out, out_ld, inner);
+    hipLaunchKernelGGL((silu_gate_kernel<float, true>), grid, dim3(256), 0, s, gu, ld, (float*)out, out_ld, inner, form, row_scale);
   else if (dtype == PS_F32)
-    hipLaunchKernelGGL((silu_gate_kernel<float, false>), grid, dim3(256), 0, s, gu, ld, (float*)out, out_ld, inner);
+    hipLaunchKernelGGL((silu_gate_kernel<float, false>), grid, dim3(256), 0, s, gu, ld, (float*)out, out_ld, inner, form, row_scale);
   else if (activation)
-    hipLaunchKernelGGL((silu_gate_kernel<bf16_t, true>), grid, dim3(256), 0, s, gu, ld, (bf16_t*)out, out_ld, inner);
+    hipLaunchKernelGGL((silu_gate_kernel<bf16_t, true>), grid, dim3(256), 0, s, gu, ld, (bf16_t*)out, out_ld, inner, form, row_scale);
   else
-    hipLaunchKernelGGL((silu_gate_kernel<bf16_t, false>), grid, dim3(256), 0, s, gu, ld, (bf16_t*)out, out_ld, inner);
+    hipLaunchKernelGGL((silu_gate_kernel<bf16_t, false>), grid, dim3(256), 0, s, gu, ld, (bf16_t*)out, out_ld, inner, form, row_scale);
   PS_CHECK_LAUNCH("ps_silu_gate");
   return 0;
 }

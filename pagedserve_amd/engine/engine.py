@@ -95,7 +95,7 @@ class Engine:
             if max_context <= 0:
                 raise ValueError("max_context must be positive")
             self.max_positions = min(self.max_positions, int(max_context))
-        if groups and not any(group.window > 0 for group in groups):
+        if groups and not any(group.span > 0 for group in groups):
             smallest = num_pages if isinstance(num_pages, int) else min(num_pages)
             self.max_positions = min(self.max_positions, smallest * page_size)
         self.cache = CacheManager(groups, num_pages, page_size, max_requests, self.dtype,

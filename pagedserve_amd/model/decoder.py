@@ -15,7 +15,7 @@ from ..config.spec import ModelSpec
 from ..ops import kernels
 from ..parts import (ARRANGEMENTS, EMBEDDINGS, HEADS, NORMS, POSITIONS, ROLES, CacheView,
                      PagedKVSpec, SlotStateSpec, build_part)
-from ..parts.block import STREAM_BIAS
+from ..parts.block import STREAM_BIAS, STREAM_ROWS
 from ..weights.loader import VECTOR, ParamSpec
 
 
@@ -59,6 +59,10 @@ class DecoderModel:
                     or not getattr(self.embedding, "takes_norm", False)):
                 raise ValueError("the embedding's norm must be an RMS norm without a shift, on a single "
                                  "stream, with an embedding that norms in its own launch")
+        # whether the embedded rows are kept beside the stream, for calls that add them again
+        self.keeps_embedding = any(call.add_embedding for call in spec.schedule)
+        if self.keeps_embedding and not getattr(self.embedding, "takes_copy", False):
+            raise ValueError("a call that adds the embedding again needs an embedding that keeps its rows")
         # Queries of a prompt portion are handed to the mixers in tiles; each mixer says which
         # size (or sizes) its kernel takes, and the step lists the tiles once per size that is
         # asked for.
@@ -146,13 +150,12 @@ class DecoderModel:
         for entry, spec in flat:
             if isinstance(spec, PagedKVSpec):
                 by_geometry.setdefault((spec.kv_heads, spec.head_dim, spec.window, spec.value_dim,
-                                        spec.values_in_keys), []).append(entry)
+                                        spec.values_in_keys, spec.chunk), []).append(entry)
             elif isinstance(spec, SlotStateSpec):
                 states.append(StateSpec(entry, tuple(spec.shape), spec.dtype))
             elif spec is not None:
                 raise TypeError(f"unknown cache spec {spec!r}")
-        groups = [CacheGroupSpec(tuple(entries), kv_heads, head_dim, window, value_dim, shared)
-                  for (kv_heads, head_dim, window, value_dim, shared), entries in by_geometry.items()]
+        groups = [CacheGroupSpec(tuple(entries), *geometry) for geometry, entries in by_geometry.items()]
         return groups, states
 
     def cache_views(self, cache) -> List[CacheView]:
@@ -204,23 +207,27 @@ class DecoderModel:
             kernels.streams_expand(embedded, h, tokens, width, streams)
         else:
             h = ctx.workspace.first_rows("residual", width, torch.float32, tokens)
+            options = {}
             if self.embedding_norm is not None:
-                self.embedding.forward(ctx, self.position.embedding_table(), h,
-                                       norm=self.embedding_norm.gamma_eps())
-            else:
-                self.embedding.forward(ctx, self.position.embedding_table(), h)
+                options["norm"] = self.embedding_norm.gamma_eps()
+            if self.keeps_embedding:
+                options["copy"] = embedded = ctx.workspace.first_rows("embedded", width, torch.float32, tokens)
+            self.embedding.forward(ctx, self.position.embedding_table(), h, **options)
         schedule = self.spec.schedule
         for index, (call, view) in enumerate(zip(schedule, views)):
             block = self.blocks[call.block]
-            if call.enter >= 0:
-                # the pass vector: a block that folds it into its first launch takes it, else a
-                # launch of its own adds it
+            if call.enter >= 0 or call.add_embedding:
+                # the embedding again and the pass vector: a block that folds them into its first
+                # launch takes them, else a launch of its own adds them
+                bias = self.pass_rows[call.enter] if call.enter >= 0 else None
+                rows = embedded if call.add_embedding else None
                 if getattr(block, "takes_stream_bias", False):
                     if ctx.extra is None:
                         ctx.extra = {}
-                    ctx.extra[STREAM_BIAS] = self.pass_rows[call.enter]
+                    ctx.extra[STREAM_BIAS] = bias
+                    ctx.extra[STREAM_ROWS] = rows
                 else:
-                    kernels.stream_step(h, tokens, width, bias=self.pass_rows[call.enter])
+                    kernels.stream_step(h, tokens, width, bias=bias, rows=rows)
             block.forward(h, ctx, view)
             # a block may leave its last write to the block that follows, if that one takes it
             if hasattr(block, "finish"):

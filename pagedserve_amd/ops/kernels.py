@@ -21,7 +21,7 @@ EPILOGUES = {"none": 0, "gelu_tanh": 1, "gelu_erf": 2, "residual": 3, "relu2": 4
 _DTYPE_CODE = {torch.float32: F32, torch.bfloat16: BF16}
 
 _SIGNATURES = {
-    "ps_embed": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+    "ps_embed": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                  c_int, c_int, c_int, c_float, c_void_p, c_float, c_int, c_void_p],
     "ps_norm": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_float, c_int,
                 c_int, c_void_p],
@@ -60,8 +60,8 @@ _SIGNATURES = {
     "ps_conv_silu": [c_void_p, c_int64, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p,
                      c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ps_attention_prepare_heads": [c_void_p, c_int64, c_int, c_int, c_int, c_void_p, c_int64, c_void_p,
-                                   c_void_p, c_void_p, c_int, c_int, c_float, c_int, c_float, c_void_p,
-                                   c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                                   c_void_p, c_void_p, c_int, c_int, c_float, c_int, c_void_p, c_void_p,
+                                   c_float, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                                    c_int, c_int, c_int, c_void_p],
     "ps_latent_prepare": [c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_void_p, c_int64, c_void_p, c_void_p,
                           c_float, c_void_p, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_int,
@@ -76,19 +76,22 @@ _SIGNATURES = {
                           c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                           c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
                           c_int, c_int, c_int, c_void_p],
-    "ps_stream_step": [c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_float, c_void_p,
-                       c_void_p, c_int, c_int, c_int, c_void_p],
+    "ps_stream_step": [c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p, c_void_p, c_float,
+                       c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
     "ps_silu_columns": [c_void_p, c_int64, c_int, c_int, c_int, c_void_p],
-    "ps_silu_gate": [c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_int, c_int, c_void_p],
+    "ps_silu_gate": [c_void_p, c_int64, c_void_p, c_int64, c_int, c_int, c_int, c_float, c_float,
+                     c_float, c_void_p, c_int, c_void_p],
     "ps_pair_norm_mix": [c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_float, c_void_p, c_int,
                          c_int, c_void_p],
     "ps_moe_route": [c_void_p, c_int64, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
-                     c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p],
+                     c_int, c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                     c_void_p],
     "ps_moe_experts_grouped": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
-                               c_int, c_void_p],
+                               c_int, c_float, c_float, c_float, c_void_p],
     "ps_moe_experts": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
-                       c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int, c_void_p],
+                       c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_void_p, c_void_p,
+                       c_int, c_float, c_int, c_void_p],
     "ps_gla_output": [c_void_p, c_void_p, c_float, c_void_p, c_int64, c_void_p, c_int64, c_int,
                       c_int, c_int, c_int, c_void_p],
     "ps_softcap": [c_void_p, c_int64, c_int, c_int, c_float, c_void_p],
@@ -206,11 +209,12 @@ def _ptr(tensor):
     return 0 if tensor is None else tensor.data_ptr()
 
 
-def embed(table, pos_table, ids, positions, out, token_src=None, carried=None, scale=1.0, norm=None):
+def embed(table, pos_table, ids, positions, out, token_src=None, carried=None, scale=1.0, norm=None, copy=None):
     """out[t] = scale * table[id(t)] + pos_table[positions[t]] as float (pos_table may be None).
     id(t) is ``ids[t]``, or ``carried[token_src[t]]`` where ``token_src[t] >= 0``: a token
     that an earlier step chose on the device.  ``norm = (gamma, eps)``: every row is then
-    RMS-normed in the same launch, ``out / sqrt(mean(out^2) + eps) * gamma``."""
+    RMS-normed in the same launch, ``out / sqrt(mean(out^2) + eps) * gamma``.  ``copy``: float rows
+    that get the result too (a model that adds it to the stream again later)."""
     _check(table, "table", ndim=2)
     _check(ids, "ids", torch.int32, 1)
     _check(out, "out", torch.float32, 2)
@@ -238,9 +242,11 @@ def embed(table, pos_table, ids, positions, out, token_src=None, carried=None, s
     if norm is not None:
         gamma, eps = norm
         _float_vector(gamma, "norm gamma", width)
+    if copy is not None:
+        _float_rows(copy, "copy", tokens, width)
     _call("ps_embed", table.data_ptr(), _ptr(pos_table), ids.data_ptr(), _ptr(token_src),
           _ptr(carried if token_src is not None else None),
-          _ptr(positions if pos_table is not None else None), out.data_ptr(), tokens, width,
+          _ptr(positions if pos_table is not None else None), out.data_ptr(), _ptr(copy), tokens, width,
           table.shape[0], max_positions, float(scale), _ptr(gamma), float(eps),
           dtype_code(table.dtype), _stream())
     return out
@@ -1342,12 +1348,13 @@ def differential_merge(partial, count, splits, lam, factor, eps, gate, out, head
 
 def attention_prepare_heads(proj, columns, q_out, k_pool, v_pool, tok_item, tok_pos, tables, heads,
                             key_dim, value_dim, freqs=None, rot_dims=0, halves=True, magnitude=1.0,
-                            head_norm=False, eps=1e-6):
+                            head_norm=False, eps=1e-6, norm_first=False, q_gamma=None, k_gamma=None):
     """``attention_prepare`` for layers that treat every head on its own: rotation of the first
     ``rot_dims`` dimensions of each head (``halves``: dimension i with i + rot_dims / 2, else 2i
     with 2i + 1; cosine and sine times ``magnitude``), then ``head_norm``: each head divided by its
-    root mean square over ``key_dim`` (no weight).  ``columns = (q_col, k_col, v_col)``; the value
-    columns are stored as projected and may be the key columns."""
+    root mean square over ``key_dim`` and multiplied by ``q_gamma`` / ``k_gamma`` (a float per dimension,
+    None for ones); ``norm_first``: that ahead of the rotation.  ``columns = (q_col, k_col, v_col)``; the
+    value columns are stored as projected and may be the key columns."""
     _check(proj, "proj", torch.float32, 2)
     _check(q_out, "q_out", ndim=2)
     pages, kv_heads, page_size, cache_dim = _check_pools(k_pool, v_pool, q_out.dtype)
@@ -1364,9 +1371,13 @@ def attention_prepare_heads(proj, columns, q_out, k_pool, v_pool, tok_item, tok_
     _check_step_index(tok_item, tok_pos, tables, tokens)
     if rot_dims:
         _float_vector(freqs, "freqs", rot_dims // 2)
+    for name, gamma in (("q_gamma", q_gamma), ("k_gamma", k_gamma)):
+        if gamma is not None:
+            _float_vector(gamma, name, key_dim)
     _call("ps_attention_prepare_heads", proj.data_ptr(), ld, q_col, k_col, v_col, q_out.data_ptr(),
           _rows(q_out, "q_out"), k_pool.data_ptr(), v_pool.data_ptr(), _ptr(freqs), int(rot_dims),
-          1 if halves else 0, float(magnitude), 1 if head_norm else 0, float(eps), tok_item.data_ptr(),
+          1 if halves else 0, float(magnitude), (2 if norm_first else 1) if head_norm else 0,
+          _ptr(q_gamma), _ptr(k_gamma), float(eps), tok_item.data_ptr(),
           tok_pos.data_ptr(), tables.data_ptr(), tables.shape[1], tokens, heads, kv_heads, key_dim,
           value_dim, cache_dim, page_size, pages, dtype_code(q_out.dtype), _stream())
 
@@ -1699,12 +1710,13 @@ def selective_scan(x, dt, bc, b_col, c_col, proj, u_col, z_col, a_log, skip, sta
           dtype_code(x.dtype), _stream())
 
 
-def stream_step(h, tokens, width, add=None, bias=None, norm=None, zero=None):
+def stream_step(h, tokens, width, add=None, bias=None, norm=None, zero=None, rows=None, norm2=None):
     """One pass over the float stream ``h`` (``[>= tokens, width]``), every piece optional:
     ``add = (y, factor)``: ``h += factor * y``, or ``add = (y, factor, column_scale)`` with a float
-    per column: ``h += factor * column_scale * y``; ``bias``: a float row added to every token;
+    per column: ``h += factor * column_scale * y``; ``rows``: a float row per token that is added;
+    ``bias``: a float row added to every token;
     ``norm = (gamma, eps, normed)``: the RMS norm of the new ``h`` times ``gamma`` goes to ``normed``
-    (engine dtype); ``zero``: a float ``[tokens, width]`` buffer that is cleared (it may be ``y``)."""
+    (engine dtype); ``norm2 = (gamma2, normed2)``: the same norm times ``gamma2`` to ``normed2``; ``zero``: a float ``[tokens, width]`` buffer that is cleared (it may be ``y``)."""
     _float_rows(h, "h", tokens, width)
     y, factor, gamma, eps, normed, code, column_scale = None, 0.0, None, 1.0, None, F32, None
     if add is not None:
@@ -1722,18 +1734,45 @@ def stream_step(h, tokens, width, add=None, bias=None, norm=None, zero=None):
         if normed.shape[0] < tokens or normed.shape[1] != width or not normed.is_contiguous():
             raise KernelError("stream_step: normed must be contiguous [>= tokens, width]")
         code = dtype_code(normed.dtype)
+    gamma2 = normed2 = None
+    if norm2 is not None:
+        gamma2, normed2 = norm2
+        _float_vector(gamma2, "gamma2", width)
+        if norm is None:
+            raise KernelError("stream_step: a second norm goes with a first")
+        _check(normed2, "normed2", normed.dtype, 2)
+        if normed2.shape[0] < tokens or normed2.shape[1] != width or not normed2.is_contiguous():
+            raise KernelError("stream_step: normed2 must be contiguous [>= tokens, width]")
     if zero is not None:
         _float_rows(zero, "zero", tokens, width)
-    _call("ps_stream_step", h.data_ptr(), _ptr(y), float(factor), _ptr(column_scale), _ptr(bias), _ptr(gamma), float(eps),
-          _ptr(normed), _ptr(zero), tokens, width, code, _stream())
+    if rows is not None:
+        _float_rows(rows, "rows", tokens, width)
+    _call("ps_stream_step", h.data_ptr(), _ptr(y), float(factor), _ptr(column_scale), _ptr(rows), _ptr(bias),
+          _ptr(gamma), float(eps), _ptr(normed), _ptr(gamma2), _ptr(normed2), _ptr(zero), tokens, width, code,
+          _stream())
 
 
 GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
 
+# constants of the gated unit ``g' sigmoid(slope g') (u' + shift)`` with ``g' = min(g, limit)`` and
+# ``u' = clamp(u, -limit, limit)`` (csrc/common.h: GateForm); these are ``silu(g) * u``
+PLAIN_GATE = (float("inf"), 1.0, 0.0)
 
-def silu_gate(gu, out, activation="silu"):
+
+def _gate_form(form):
+    """(limit, slope, shift) of the gated unit, checked."""
+    limit, slope, shift = (float(value) for value in form)
+    if not limit > 0.0:
+        raise KernelError(f"the limit of a gated unit must be positive (inf: none), got {limit}")
+    return limit, slope, shift
+
+
+def silu_gate(gu, out, activation="silu", form=PLAIN_GATE, row_scale=None):
     """``out[t, c] = act(gu[t, c]) * gu[t, inner + c]`` for float ``gu`` of ``2 * inner`` columns;
-    ``act``: ``silu`` or ``gelu_tanh``."""
+    ``act``: ``silu`` (with the unit's other constants as ``form = (limit, slope, shift)``) or
+    ``gelu_tanh``.  ``row_scale``: a float per row that multiplies it."""
+    if row_scale is not None:
+        _float_vector(row_scale, "row_scale", gu.shape[0])
     if activation not in GATE_ACTIVATIONS:
         raise KernelError(f"silu_gate: activation {activation!r}; known: {', '.join(GATE_ACTIVATIONS)}")
     _check(gu, "gu", torch.float32, 2)
@@ -1742,7 +1781,8 @@ def silu_gate(gu, out, activation="silu"):
     if gu.shape[1] != 2 * inner or out.shape[0] < tokens or out.shape[1] != inner:
         raise KernelError("silu_gate: gu must hold twice out's columns")
     _call("ps_silu_gate", gu.data_ptr(), _rows(gu, "gu"), out.data_ptr(), _rows(out, "out"), tokens,
-          inner, GATE_ACTIVATIONS[activation], dtype_code(out.dtype), _stream())
+          inner, GATE_ACTIVATIONS[activation], *_gate_form(form), _ptr(row_scale), dtype_code(out.dtype),
+          _stream())
 
 
 def silu_columns(rows, first, count):
@@ -1765,16 +1805,29 @@ def pair_norm_mix(a, b, weight_a, weight_b, eps, share, y, tokens, width):
           float(eps), float(share), y.data_ptr(), tokens, width, _stream())
 
 
-def moe_route(x, router, groups, keep, top, scale, ids, weights, sigmoid=False, correction=None,
-              group_top=1, normalise=False, fixed=0):
+ROUTE_SCORES = {"softmax": 0, "sigmoid": 1, "chosen_softmax": 2}
+
+
+def moe_route(x, router, groups, keep, top, scale, ids, weights, score="softmax", correction=None,
+              group_top=1, normalise=False, fixed=False, gate=None, gate_out=None):
     """The experts that every row of ``x`` chooses (``ids``, int32 ``[tokens, top]``) and their
-    weights (float): softmax (or ``sigmoid``) over all experts of the 32-bit logits, group-limited
-    choice, the scores times ``scale`` (``csrc/moe.hip``).  ``correction``: a float per expert
+    weights (float): softmax over all experts (or ``sigmoid``) of the 32-bit logits, group-limited
+    choice, the scores times ``scale`` (``csrc/moe.hip``); ``chosen_softmax``: the choice by the logits
+    themselves, the weights the softmax over the chosen ones.  ``correction``: a float per expert
     that is added to the scores for the choice only; ``group_top``: a group's score is the sum of
     that many of its largest choice scores; ``normalise``: the chosen scores are divided by
-    their sum before ``scale``.  ``fixed``: that many more columns of ``ids`` and ``weights`` are
-    filled with the numbers ``experts, experts + 1, ..`` and the weight one (experts that every token
-    uses, for ``moe_experts(extra=...)``)."""
+    their sum before ``scale``.  ``fixed``: ``ids`` and ``weights`` have one more column, for an expert
+    that every token uses (``moe_experts(extra=...)``): the number ``experts`` and the weight one, or
+    ``sigmoid(gate . x)`` of a float row ``gate``; without ``fixed``, those weights go to ``gate_out``
+    (float ``[>= tokens]``)."""
+    if score not in ROUTE_SCORES:
+        raise KernelError(f"moe_route: unknown score {score!r}; known: {', '.join(ROUTE_SCORES)}")
+    if gate is not None:
+        _float_vector(gate, "gate", x.shape[1])
+    if gate_out is not None:
+        if fixed or gate is None:
+            raise KernelError("moe_route: gates go to rows of their own only without a fixed expert")
+        _float_vector(gate_out, "gate_out", x.shape[0])
     if correction is not None:
         _float_vector(correction, "correction", router.shape[0])
     if not 1 <= int(group_top) <= 8:
@@ -1788,12 +1841,12 @@ def moe_route(x, router, groups, keep, top, scale, ids, weights, sigmoid=False, 
     _check(ids, "ids", torch.int32, 2)
     _check(weights, "weights", torch.float32, 2)
     for tensor in (ids, weights):
-        if tensor.shape[0] < tokens or tensor.shape[1] != top + fixed or not tensor.is_contiguous():
+        if tensor.shape[0] < tokens or tensor.shape[1] != top + (1 if fixed else 0) or not tensor.is_contiguous():
             raise KernelError("moe_route: ids and weights must be contiguous [>= tokens, top + fixed]")
     _call("ps_moe_route", x.data_ptr(), x.stride(0), router.data_ptr(), tokens, width, experts,
-          int(groups), int(keep), int(top), float(scale), 1 if sigmoid else 0, _ptr(correction),
-          int(group_top), 1 if normalise else 0, int(fixed), ids.data_ptr(), weights.data_ptr(),
-          dtype_code(x.dtype), _stream())
+          int(groups), int(keep), int(top), float(scale), ROUTE_SCORES[score], _ptr(correction),
+          int(group_top), 1 if normalise else 0, 1 if fixed else 0, _ptr(gate), _ptr(gate_out),
+          ids.data_ptr(), weights.data_ptr(), dtype_code(x.dtype), _stream())
 
 
 MOE_TILE = 128            # pairs per tile of the sorted path (csrc/moe.hip)
@@ -1809,7 +1862,8 @@ def moe_grouped_tiles(pairs, experts) -> int:
     return -(-pairs // MOE_TILE) + experts
 
 
-def moe_experts_grouped(x, w1, w2, ids, weights, hidden, out, order, tile_expert, y, gated=True):
+def moe_experts_grouped(x, w1, w2, ids, weights, hidden, out, order, tile_expert, y, gated=True,
+                        form=PLAIN_GATE):
     """``moe_experts`` for many rows in bfloat16: the pairs sorted by expert, the products on the
     matrix cores.  ``out``: float ``[>= tokens * top, width]``, ``order``: int32 ``[>= tiles * MOE_TILE]``,
     ``tile_expert``: int32 ``[>= tiles]`` scratch with ``tiles = moe_grouped_tiles(tokens * top, experts)``."""
@@ -1828,8 +1882,8 @@ def moe_experts_grouped(x, w1, w2, ids, weights, hidden, out, order, tile_expert
         raise KernelError("moe_experts_grouped: ids and weights must be contiguous [tokens, top]")
     tiles = moe_grouped_tiles(tokens * top, experts)
     _check(hidden, "hidden", x.dtype, 2)
-    if hidden.shape[0] < tokens * top or hidden.shape[1] != inner or not hidden.is_contiguous():
-        raise KernelError("moe_experts_grouped: hidden must be contiguous [>= tokens * top, inner]")
+    if hidden.numel() < tokens * top * inner or not hidden.is_contiguous():
+        raise KernelError("moe_experts_grouped: hidden must be contiguous with room for tokens * top * inner")
     _float_rows(out, "out", tokens * top, width)
     _check(order, "order", torch.int32, 1)
     _check(tile_expert, "tile_expert", torch.int32, 1)
@@ -1838,15 +1892,18 @@ def moe_experts_grouped(x, w1, w2, ids, weights, hidden, out, order, tile_expert
     _float_rows(y, "y", tokens, width)
     _call("ps_moe_experts_grouped", x.data_ptr(), x.stride(0), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(),
           weights.data_ptr(), hidden.data_ptr(), out.data_ptr(), order.data_ptr(), tile_expert.data_ptr(),
-          y.data_ptr(), tokens, width, inner, experts, top, 1 if gated else 0, _stream())
+          y.data_ptr(), tokens, width, inner, experts, top, 1 if gated else 0, *_gate_form(form), _stream())
 
 
-def moe_experts(x, w1, w2, ids, weights, hidden, y, gated=True, extra=None):
-    """``y[t] += sum_j weights[t, j] W2[e] (silu(W1[e][:inner] x_t) * (W1[e][inner:] x_t))`` with
-    ``e = ids[t, j]``; ``w1``: ``[experts, 2 * inner, width]``, ``w2``: ``[experts, width, inner]``.
+def moe_experts(x, w1, w2, ids, weights, hidden, y, gated=True, extra=None, form=PLAIN_GATE,
+                extra_limit=float("inf")):
+    """``y[t] += sum_j weights[t, j] W2[e] unit(W1[e][:inner] x_t, W1[e][inner:] x_t)`` with
+    ``e = ids[t, j]``; ``w1``: ``[experts, 2 * inner, width]``, ``w2``: ``[experts, width, inner]``;
+    ``form``: the constants of the gated unit.
     ``gated=False``: the plain form ``W2[e] relu(W1[e] x_t)^2`` with ``w1 [experts, inner, width]``.
-    ``extra = (w1x, w2x)``: experts numbered from ``experts`` on, in tensors of their own of the same
-    form (``moe_route(fixed=...)`` names them for every token)."""
+    ``extra = (w1x, w2x)``: the expert in the last column of ``ids``, which every token uses
+    (``moe_route(fixed=True)``), of the same form but an inner width and a limit of its own: ``w1x [2 *
+    inner_x, width]`` (plain: ``[inner_x, width]``), ``w2x [width, inner_x]``."""
     _check(x, "x", ndim=2)
     tokens, width = x.shape
     _check(w1, "w1", x.dtype, 3)
@@ -1859,22 +1916,26 @@ def moe_experts(x, w1, w2, ids, weights, hidden, y, gated=True, extra=None):
     _check(ids, "ids", torch.int32, 2)
     _check(weights, "weights", torch.float32, 2)
     _check(hidden, "hidden", x.dtype, 2)
-    if hidden.shape[0] < tokens * top or hidden.shape[1] != inner or not hidden.is_contiguous():
-        raise KernelError("moe_experts: hidden must be contiguous [>= tokens * top, inner]")
     if not (ids.is_contiguous() and weights.is_contiguous()) or weights.shape[1] != top:
         raise KernelError("moe_experts: ids and weights must be contiguous [tokens, top]")
     w1x = w2x = None
+    inner_x = 0
     if extra is not None:
         w1x, w2x = extra
-        _check(w1x, "extra w1", x.dtype, 3)
-        _check(w2x, "extra w2", x.dtype, 3)
-        if (tuple(w1x.shape[1:]) != tuple(w1.shape[1:]) or tuple(w2x.shape[1:]) != tuple(w2.shape[1:])
-                or w1x.shape[0] != w2x.shape[0] or not (w1x.is_contiguous() and w2x.is_contiguous())):
-            raise KernelError("moe_experts: the extra experts must have the form of the others")
+        _check(w1x, "extra w1", x.dtype, 2)
+        _check(w2x, "extra w2", x.dtype, 2)
+        inner_x = w2x.shape[1]
+        if (tuple(w1x.shape) != ((2 if gated else 1) * inner_x, width) or w2x.shape[0] != width or top < 2
+                or not (w1x.is_contiguous() and w2x.is_contiguous())):
+            raise KernelError("moe_experts: the expert for every token must have the form of the others")
+    held = (top - 1 if inner_x else top) * inner + inner_x
+    if hidden.numel() < tokens * held or not hidden.is_contiguous():
+        raise KernelError(f"moe_experts: hidden must be contiguous with room for {held} columns per token")
     _float_rows(y, "y", tokens, width)
     _call("ps_moe_experts", x.data_ptr(), x.stride(0), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(),
           weights.data_ptr(), hidden.data_ptr(), y.data_ptr(), tokens, width, inner, top,
-          1 if gated else 0, experts, _ptr(w1x), _ptr(w2x), dtype_code(x.dtype), _stream())
+          1 if gated else 0, *_gate_form(form), _ptr(w1x), _ptr(w2x), inner_x, float(extra_limit),
+          dtype_code(x.dtype), _stream())
 
 
 def gla_output(o, weight, eps, gate, out, heads, value_dim):

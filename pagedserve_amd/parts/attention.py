@@ -5,7 +5,7 @@ import torch
 from ..ops import kernels
 from ..weights.loader import MATRIX, VECTOR, ParamSpec
 from .base import Mixer, PagedKVSpec, site_memo
-from .position import rotary_frequencies
+from .position import banded_frequencies, rotary_frequencies
 from .registry import register_mixer
 
 
@@ -44,16 +44,22 @@ class Attention(Mixer):
       (which then speaks for the packed projection alone).
     * ``rotary_layout``: ``"neighbours"`` (dimension 2i with 2i+1) or ``"halves"`` (dimension i
       with i + rotary_dims / 2); ``rotary_scaling = (factor, original, fast, slow)`` stretches
-      the frequencies and scales cosine and sine (``parts/position.py: rotary_frequencies``).
-    * ``head_norm``: after the rotation every query and key head is divided by its own root
-      mean square (no weight, ``norm_eps``).
+      the frequencies and scales cosine and sine (``parts/position.py: rotary_frequencies``);
+      ``rotary_bands = (factor, low, high, original)`` stretches them by wavelength
+      (``banded_frequencies`` there).
+    * ``head_norm``: every query and key head is divided by its own root mean square over
+      ``head_dim`` (``norm_eps``): ``True`` or ``"after"``, after the rotation, without a weight;
+      ``"before"``, before the rotation, with a weight per dimension that all heads share
+      (``q_norm.gamma``, ``k_norm.gamma``).
+    * ``chunk``: a query at position p sees the keys ``p // chunk * chunk .. p`` only: positions are
+      cut into chunks counted from 0, and none looks into the chunk before its own.
     * ``values_from_keys``: there is no value projection; the values are the keys as projected,
       before rotation and norm (the packed product is ``[q | k]``).
     * ``score_cap``: ``c > 0``: a scaled score ``s`` enters the softmax as ``c tanh(s / c)``.
     * ``pad_heads``: heads are cached with their size rounded up to a multiple of this (zeros
       behind), so that a head size which the tiled kernels do not take still runs on them.
 
-    ``rotary_layout="halves"``, ``rotary_scaling``, ``head_norm`` and ``values_from_keys`` go
+    ``rotary_layout="halves"``, ``rotary_scaling``, ``rotary_bands``, ``head_norm`` and ``values_from_keys`` go
     through the launch that treats every head on its own (``kernels.attention_prepare_heads``);
     that one does not norm over the whole projection or mix values.
     """
@@ -72,13 +78,20 @@ class Attention(Mixer):
 
     VALUE_MIXES = ("none", "source", "mix")
 
+    chunk = 0      # (mixers that are built on this one and set no chunk of their own)
+
+    @property
+    def span(self) -> int:
+        """Which keys a query sees, as the kernels take it (csrc/common.h: first_visible_key)."""
+        return -self.chunk if self.chunk else self.window
+
     def __init__(self, width: int, dtype, heads: int, kv_heads: int, head_dim: int, scale: float,
                  window: int = 0, bias: bool = True, value_dim: int = 0, qk_norm: bool = False,
                  norm_eps: float = 1e-6, rotary_dims: int = 0, rotary_base: float = 10000.0,
                  sink: bool = False, value_mix: str = "none", head_gate: bool = False,
                  out_bias=None, rotary_layout: str = "neighbours", rotary_scaling=None,
-                 head_norm: bool = False, values_from_keys: bool = False, score_cap: float = 0.0,
-                 pad_heads: int = 0):
+                 head_norm=False, values_from_keys: bool = False, score_cap: float = 0.0,
+                 pad_heads: int = 0, chunk: int = 0, rotary_bands=None):
         if heads % kv_heads != 0:
             raise ValueError(f"heads ({heads}) must be a multiple of kv_heads ({kv_heads})")
         if not 0 < head_dim <= 256:
@@ -97,6 +110,9 @@ class Attention(Mixer):
         self.value_dim = value_dim or head_dim
         self.scale = float(scale)
         self.window = int(window)
+        self.chunk = int(chunk)
+        if self.window < 0 or self.chunk < 0 or (self.window and self.chunk):
+            raise ValueError("attention sees a window or a chunk of positions (0: neither), not both")
         self.bias = bias
         # (the output projection's bias goes with the packed projection's unless named apart)
         self.out_has_bias = bool(bias) if out_bias is None else bool(out_bias)
@@ -111,7 +127,13 @@ class Attention(Mixer):
             raise ValueError(f"rotary_layout {rotary_layout!r}; known: neighbours, halves")
         self.rotary_halves = rotary_layout == "halves"
         self.rotary_scaling = None if rotary_scaling is None else tuple(float(v) for v in rotary_scaling)
+        if head_norm not in (False, True, "after", "before"):
+            raise ValueError(f"head_norm {head_norm!r}; known: True or after, before, False")
         self.head_norm = bool(head_norm)
+        self.norm_before = head_norm == "before"
+        self.rotary_bands = None if rotary_bands is None else tuple(float(v) for v in rotary_bands)
+        if self.rotary_bands is not None and self.rotary_scaling is not None:
+            raise ValueError("frequencies are stretched one way or the other, not both")
         self.values_from_keys = bool(values_from_keys)
         self.score_cap = float(score_cap or 0.0)
         if self.score_cap < 0:
@@ -120,7 +142,7 @@ class Attention(Mixer):
             raise ValueError("values that are the keys have the keys' head size")
         # the launch that treats every head on its own
         self.head_wise = (self.head_norm or self.values_from_keys or self.rotary_scaling is not None
-                          or (self.rotary_halves and self.rotary_dims > 0))
+                          or self.rotary_bands is not None or (self.rotary_halves and self.rotary_dims > 0))
         if self.head_wise and (self.qk_norm or value_mix != "none"):
             raise ValueError("a norm over the whole projection and mixed values do not go with "
                              "rotary halves, scaled frequencies, head norms or values from keys")
@@ -169,6 +191,9 @@ class Attention(Mixer):
         if self.qk_norm:
             params["q_norm.gamma"] = ParamSpec((self.heads * self.key_dim,), VECTOR)
             params["k_norm.gamma"] = ParamSpec((self.kv_heads * self.key_dim,), VECTOR)
+        elif self.norm_before:
+            params["q_norm.gamma"] = ParamSpec((self.key_dim,), VECTOR)
+            params["k_norm.gamma"] = ParamSpec((self.key_dim,), VECTOR)
         if self.has_sink:
             params["sink"] = ParamSpec((self.heads,), VECTOR)
         if self.value_mix == "mix":
@@ -194,8 +219,11 @@ class Attention(Mixer):
         self.rotary_magnitude = 1.0
         if self.rotary_dims:
             # base^(-2i/dims), worked out in 64-bit and rounded once; the angle is float(p) * f
-            freqs, self.rotary_magnitude = rotary_frequencies(self.rotary_dims, self.rotary_base,
-                                                              self.rotary_scaling)
+            if self.rotary_bands is not None:
+                freqs = banded_frequencies(self.rotary_dims, self.rotary_base, *self.rotary_bands)
+            else:
+                freqs, self.rotary_magnitude = rotary_frequencies(self.rotary_dims, self.rotary_base,
+                                                                  self.rotary_scaling)
             self.freqs = freqs.to(torch.float32).to(self.out_weight.device)
         # copies in the layout that the products of few rows (decode steps) read fastest
         self.qkv_packed = kernels.pack_decode_weight(self.qkv_weight)
@@ -205,7 +233,7 @@ class Attention(Mixer):
         self._memo_attention.clear()
 
     def cache_spec(self):
-        return PagedKVSpec(self.kv_heads, self.head_dim, self.window)
+        return PagedKVSpec(self.kv_heads, self.head_dim, self.window, chunk=self.chunk)
 
     def _project_prepared(self, x, ctx, cache, tables):
         """Projection in float, then norm, rotation, value mixing and cache write in one launch;
@@ -227,7 +255,8 @@ class Attention(Mixer):
                 proj, (q_col, k_col, v_col), q, cache.k_pool, cache.v_pool, ctx.tok_item, ctx.positions,
                 tables, self.heads, self.key_dim, self.value_dim, freqs=self.freqs,
                 rot_dims=self.rotary_dims, halves=self.rotary_halves, magnitude=self.rotary_magnitude,
-                head_norm=self.head_norm, eps=self.norm_eps)
+                head_norm=self.head_norm, eps=self.norm_eps, norm_first=self.norm_before,
+                q_gamma=self.q_gamma, k_gamma=self.k_gamma)
             return q, (proj[:, gate_col:gate_col + self.heads] if self.head_gate else None)
         kernels.attention_prepare(
             proj, (q_col, k_col, v_col), q, cache.k_pool, cache.v_pool, ctx.tok_item, ctx.positions,
@@ -297,7 +326,7 @@ class Attention(Mixer):
             partial = self._range_records(ctx)
             kernels.attention_decode_partial(q, cache.k_pool, cache.v_pool, partial, ctx.tok_item,
                                              ctx.positions, tables, self.heads, self.scale, splits,
-                                             window=self.window, waves=4, sink=sink, softcap=self.score_cap)
+                                             window=self.span, waves=4, sink=sink, softcap=self.score_cap)
             kernels.attention_merge_linear(partial, singles, self.heads, self.head_dim, splits,
                                            self.out_weight, self.out_packed, self.out_bias, residual)
             return
@@ -307,7 +336,7 @@ class Attention(Mixer):
             tile_item, tile_q0 = ctx.query_tiles[kernels.PREFILL_TILE]
             kernels.attention_mixed(q, cache.k_pool, cache.v_pool, context, ctx.single_tokens,
                                     ctx.tok_item, ctx.positions, tile_item, tile_q0, ctx.cu_tokens,
-                                    ctx.kv_lens, tables, self.heads, self.scale, self.window,
+                                    ctx.kv_lens, tables, self.heads, self.scale, self.span,
                                     memo=site_memo(self._memo_attention, ctx.workspace),
                                     shared=ctx.shared_calls, sink=sink, gate=gates, softcap=self.score_cap)
             return self._project_out(context, residual, ctx)
@@ -317,7 +346,7 @@ class Attention(Mixer):
                                             None if singles == tokens else ctx.tok_item, ctx.positions,
                                             tables, self.heads, self.scale,
                                             self._shared_splits(singles, ctx.max_kv_len),
-                                            self._range_records(ctx), window=self.window,
+                                            self._range_records(ctx), window=self.span,
                                             tok_list=None if singles == tokens else ctx.single_tokens,
                                             gate=gates, softcap=self.score_cap)
         elif singles:
@@ -338,7 +367,7 @@ class Attention(Mixer):
             kernels.attention_decode(q, cache.k_pool, cache.v_pool, context,
                                      None if direct else ctx.tok_item,
                                      ctx.positions, tables, self.heads, self.scale, splits,
-                                     partial=partial, window=self.window, waves=waves,
+                                     partial=partial, window=self.span, waves=waves,
                                      tok_list=None if singles == tokens else ctx.single_tokens,
                                      sink=sink, gate=gates, softcap=self.score_cap)
         whole = singles == 0
@@ -355,7 +384,7 @@ class Attention(Mixer):
                 tile_item, tile_q0 = ctx.query_tiles[size]
             kernels.attention_prefill(q, cache.k_pool, cache.v_pool, context, tile_item,
                                       tile_q0, ctx.cu_tokens, ctx.kv_lens, tables,
-                                      self.heads, self.scale, self.window,
+                                      self.heads, self.scale, self.span,
                                       max_kv_len=ctx.max_kv_len, query_tile=size,
                                       memo=site_memo(self._memo_attention, ctx.workspace),
                                       shared=ctx.shared_calls, sink=sink, gate=gates, softcap=self.score_cap)
@@ -367,15 +396,15 @@ class Attention(Mixer):
             if tile_item.numel():
                 kernels.attention_tiled_f32(q, cache.k_pool, cache.v_pool, context, tile_item, tile_q0,
                                             ctx.cu_tokens, ctx.kv_lens, tables, self.heads, self.scale,
-                                            self.window, sink=sink, gate=gates, softcap=self.score_cap)
+                                            self.span, sink=sink, gate=gates, softcap=self.score_cap)
             if not singles and ctx.single_tokens is not None and ctx.single_tokens.numel():
                 kernels.attention_rowwise(q, cache.k_pool, cache.v_pool, context, ctx.tok_item,
-                                          ctx.positions, tables, self.heads, self.scale, self.window,
+                                          ctx.positions, tables, self.heads, self.scale, self.span,
                                           tok_list=None if ctx.single_tokens.numel() == tokens
                                           else ctx.single_tokens, sink=sink, gate=gates, softcap=self.score_cap)
         elif singles < tokens:
             kernels.attention_rowwise(q, cache.k_pool, cache.v_pool, context, ctx.tok_item,
-                                      ctx.positions, tables, self.heads, self.scale, self.window,
+                                      ctx.positions, tables, self.heads, self.scale, self.span,
                                       tok_list=None if whole else ctx.portion_tokens, sink=sink, gate=gates, softcap=self.score_cap)
         self._project_out(context, residual, ctx)
 
@@ -393,11 +422,16 @@ class Attention(Mixer):
         against 0.958 ms)."""
         if not (self.fuse_mixed and kernels.mixed_supported(self.dtype, self.head_dim, tables.shape[1])):
             return False
-        visible = ctx.max_kv_len if self.window <= 0 else min(ctx.max_kv_len, self.window)
+        visible = self._visible(ctx.max_kv_len)
         if 4 * singles * self.heads < kernels.compute_units() and visible > 512:
             return False
         large_tiles = ctx.query_tiles[kernels.PREFILL_LARGE_TILE][0].numel()
         return not kernels.prefill_large_tile_pays(self.heads, self.head_dim, large_tiles, ctx.max_kv_len)
+
+    def _visible(self, max_kv_len: int) -> int:
+        """Most keys that a query of a step sees whose longest request has ``max_kv_len``."""
+        limit = self.window or self.chunk
+        return min(max_kv_len, limit) if limit else max_kv_len
 
     def _range_records(self, ctx):
         """Scratch for one record per (token, head, key range): always asked for at its largest
@@ -420,7 +454,7 @@ class Attention(Mixer):
         About three blocks of four waves per compute unit, never more ranges than the keys of
         the longest request can feed; and not where the projection's blocks would read more
         than 12 MB of records between them (wide models)."""
-        visible = max_kv_len if self.window <= 0 else min(max_kv_len, self.window)
+        visible = self._visible(max_kv_len)
         pairs = count * self.heads
         units = kernels.compute_units()
         most = max(1, -(-visible // kernels.decode_keys_per_block(self.head_dim, 4)))
@@ -443,7 +477,7 @@ class Attention(Mixer):
         """Ranges per request of the decode kernel whose blocks serve a group's heads together:
         about two blocks per compute unit, no range shorter than a tile of keys, and never more
         records than the scratch holds (six per unit beside one per token and head)."""
-        visible = max_kv_len if self.window <= 0 else min(max_kv_len, self.window)
+        visible = self._visible(max_kv_len)
         units = kernels.compute_units()
         group = self.heads // self.kv_heads
         blocks = count * self.kv_heads * -(-group // kernels.SHARED_DECODE_HEADS)
@@ -473,7 +507,7 @@ class Attention(Mixer):
         Never more ranges than the keys of the longest request can feed, and never more than
         six blocks per unit beside one per pair (the scratch for the records is sized for
         that)."""
-        visible = max_kv_len if self.window <= 0 else min(max_kv_len, self.window)
+        visible = self._visible(max_kv_len)
         pairs = count * self.heads
         units = kernels.compute_units()
         if 2 * pairs >= 7 * units:

@@ -36,7 +36,8 @@ from ..weights.loader import ParamSpec
 
 @dataclass(frozen=True)
 class PagedKVSpec:
-    """A mixer that caches keys and values of every (or the last ``window``) positions."""
+    """A mixer that caches keys and values of every position, of the last ``window`` ones, or of
+    those of the current chunk of ``chunk`` positions."""
 
     kv_heads: int
     head_dim: int
@@ -45,6 +46,7 @@ class PagedKVSpec:
     # True: the values are read from the cached key rows themselves (a latent that is key and
     # value at once): the entry has one pool, handed out as both
     values_in_keys: bool = False
+    chunk: int = 0         # > 0: only keys of the query's own chunk of that many positions are ever read
 
 
 @dataclass(frozen=True)

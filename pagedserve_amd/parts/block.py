@@ -136,6 +136,7 @@ class HyperConnectedMixerBlock(HyperConnectedBlock):
 
 _SCALED_ADD = "scaled_add"    # key of ``ctx.extra``: (y, factor) of a block that is not added to the stream yet
 STREAM_BIAS = "stream_bias"   # key of ``ctx.extra``: a float row that the next block adds to every token
+STREAM_ROWS = "stream_rows"   # key of ``ctx.extra``: float rows, one per token, that the next block adds
 
 
 @register_arrangement("parallel_scaled")
@@ -178,8 +179,9 @@ class ParallelScaledBlock:
             ctx.extra = {}
         gamma, eps = self.norm1.gamma_eps()
         add = ctx.extra.pop(_SCALED_ADD, None)
-        kernels.stream_step(h, tokens, self.width, add=add, bias=ctx.extra.pop(STREAM_BIAS, None),
-                            norm=(gamma, eps, normed), zero=None if add is None else add[0])
+        kernels.stream_step(h, tokens, self.width, add=add, rows=ctx.extra.pop(STREAM_ROWS, None),
+                            bias=ctx.extra.pop(STREAM_BIAS, None), norm=(gamma, eps, normed),
+                            zero=None if add is None else add[0])
         self.mixer.forward(normed, y, ctx, cache)
         if self.feed_forward is not None:
             self.feed_forward.forward(normed, y, ctx)
@@ -191,6 +193,51 @@ class ParallelScaledBlock:
         add = ctx.extra.pop(_SCALED_ADD, None) if ctx.extra else None
         if add is not None:
             kernels.stream_step(h, ctx.tokens, self.width, add=add, zero=add[0])
+
+
+@register_arrangement("parallel_two_norms")
+class ParallelTwoNormsBlock:
+    """``h += mixer(norm1(h)) + feed_forward(norm2(h))``, both norms of the same ``h``: they divide
+    by one root mean square and differ in their scales, so one launch writes both normed rows
+    (and first adds what the model puts before a pass, ``ctx.extra[STREAM_ROWS]`` and
+    ``[STREAM_BIAS]``).  Both inputs are made before either sublayer runs, which then add straight
+    into the stream."""
+
+    roles = {"norm1": "norm", "mixer": "mixer", "norm2": "norm", "feed_forward": "feed_forward"}
+    takes_stream_bias = True
+
+    def __init__(self, width, dtype, parts):
+        self.width = width
+        self.dtype = dtype
+        self._parts = dict(parts)
+        self.norm1 = parts["norm1"]
+        self.mixer = parts["mixer"]
+        self.norm2 = parts["norm2"]
+        self.feed_forward = parts["feed_forward"]
+        if not (hasattr(self.norm1, "gamma_eps") and hasattr(self.norm2, "gamma_eps")
+                and self.norm1.eps == self.norm2.eps):
+            raise ValueError("a parallel block of two norms needs RMS norms without a shift and of one eps")
+
+    @property
+    def graph_safe(self):
+        return all(getattr(part, "graph_safe", False) for part in self._parts.values())
+
+    def parts(self):
+        return dict(self._parts)
+
+    def forward(self, h, ctx, cache):
+        tokens = ctx.tokens
+        normed1 = ctx.workspace.first_rows("normed", self.width, self.dtype, tokens)
+        normed2 = ctx.workspace.first_rows("normed2", self.width, self.dtype, tokens)
+        extra = ctx.extra or {}
+        gamma1, eps = self.norm1.gamma_eps()
+        gamma2, _ = self.norm2.gamma_eps()
+        kernels.stream_step(h, tokens, self.width, rows=extra.pop(STREAM_ROWS, None),
+                            bias=extra.pop(STREAM_BIAS, None), norm=(gamma1, eps, normed1),
+                            norm2=(gamma2, normed2))
+        self.mixer.forward(normed1, h, ctx, cache)
+        self.feed_forward.forward(normed2, h, ctx)
+        return h
 
 
 @register_arrangement("pre_norm_scaled")

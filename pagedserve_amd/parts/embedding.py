@@ -11,7 +11,8 @@ class TokenLookup(Embedding):
     """``h[t] = scale * table[id[t]] + position_table[pos[t]]`` in float
     (src/model/paged_decoder.py:306-314, where the scale is 1).  A token id may be "what the
     last step chose for row r", which the kernel reads from the device.  ``norm = (gamma, eps)``:
-    the rows are RMS-normed in the same launch (a model that norms its embedding)."""
+    the rows are RMS-normed in the same launch (a model that norms its embedding).  ``copy``: float
+    rows that get the result too (a model that adds it to the stream again before later passes)."""
 
     graph_safe = True
 
@@ -25,11 +26,12 @@ class TokenLookup(Embedding):
         return {"table": ParamSpec((self.vocab_size, self.width), TABLE)}
 
     takes_norm = True
+    takes_copy = True
 
-    def forward(self, ctx, position_table, out, norm=None):
+    def forward(self, ctx, position_table, out, norm=None, copy=None):
         return kernels.embed(self.table, position_table, ctx.token_ids, ctx.positions, out,
                              token_src=ctx.token_src, carried=ctx.carried_tokens, scale=self.scale,
-                             norm=norm)
+                             norm=norm, copy=copy)
 
 
 @register_head("linear")

@@ -37,6 +37,29 @@ class NoPositions(PositionEncoding):
         self.max_positions = max_positions
 
 
+def banded_frequencies(dims: int, base: float, factor: float, low: float, high: float, original: float):
+    """Frequencies of the ``dims / 2`` rotated pairs as 64-bit floats, ``f_i = base^(-2i / dims)``
+    stretched by wavelength as Llama 3.1 does: with ``t = original f / (2 pi)`` turns over
+    ``original`` positions, a pair of more than ``high`` turns keeps its frequency, one of fewer than
+    ``low`` turns ``factor`` times slower, and between the two the frequency is ``(1 - s) f / factor + s
+    f`` with ``s = (t - low) / (high - low)``."""
+    import math
+
+    import torch
+
+    out = []
+    for i in range(dims // 2):
+        f = float(base) ** (-2.0 * i / dims)
+        turns = original * f / (2.0 * math.pi)
+        if turns < low:
+            f = f / factor
+        elif turns <= high and high > low:
+            s = (turns - low) / (high - low)
+            f = (1.0 - s) * f / factor + s * f
+        out.append(f)
+    return torch.tensor(out, dtype=torch.float64)
+
+
 def rotary_frequencies(dims: int, base: float, scaling=None):
     """(frequencies of the ``dims / 2`` rotated pairs as 64-bit floats, factor on cosine and sine).
 
