@@ -34,6 +34,7 @@ One JSON line is printed:
     python bench.py --design zetunex [--sizes small,medium,small_many_experts]   Zetunex beside Kosesun at equal size
     python bench.py --design rezelix [--sizes small,medium,small_wide_heads]     Rezelix beside Zetunex at equal size
     python bench.py --design kozapel [--sizes small,medium,small_narrow_maps]    Kozapel beside Kosesun at equal size
+    python bench.py --design malalix [--sizes small,medium,small_passed_twice,small_wide_heads]  Malalix beside Zetunex at equal size
 
 ``--kernels`` times every kernel of a decode step (1, 8 and 64 requests over 1,024 keys), of
 the prefill step (2 x 1,024 tokens) and of a mixed step (32 decoded tokens beside a portion of
@@ -641,8 +642,39 @@ KOZAPEL_SIZES = {
     "small_narrow_maps": (kozapel_shape(768, 12, 12, 12, 32, 64, 3072, 50257, rank=96, rot_dim=32),
                           kosesun_shape(768, 12, 12, 12, 64, 64, 3072, 50257)),
 }
+
+
+def malalix_shape(width, layers, heads, kv_heads, dim, vdim, ff, vocab, chunk=512, experts=8, top=2, passes=1):
+    """A Malalix configuration of a real model's layer sizes: attention with grouped heads inside
+    chunks, half of every head rotated, and in every layer ``experts`` experts of which ``top``
+    together are as wide as a dense feed-forward of ``ff`` would be, beside a shared one as wide as
+    one of them.  ``passes``: that many passes over ``layers / passes`` layers."""
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": dim ** -0.5,
+             "mask": {"size": chunk},
+             "rot": {"dims": dim // 2, "base": 500000.0,
+                     "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    mlp = {"kind": "moe", "expert": {"ff": ff // top, "limit": 7.0}, "router": {"experts": experts, "top": top},
+           "shared": {"ff": ff // top, "limit": 7.0}}
+    listed = [{"type": "attention", "mixer": mixer, "mlp": mlp} for _ in range(layers // passes)]
+    return {"architecture": "Malalix", "vocab": vocab, "width": width, "layers": listed, "norm": {"eps": 1e-6},
+            "loop": {"start": 0, "stop": len(listed), "times": passes}}
+
+
+# name -> (Malalix configuration, the Zetunex configuration of equal width, number of layer runs,
+# heads, inner width and vocabulary)
+MALALIX_SIZES = {
+    "small": (malalix_shape(768, 12, 12, 4, 64, 64, 3072, 50257), zetunex_shape(768, 12, 12, 4, 64, 3072, 50257)),
+    "medium": (malalix_shape(1024, 24, 16, 4, 64, 64, 4096, 50257), zetunex_shape(1024, 24, 16, 4, 64, 4096, 50257)),
+    # six layers, passed twice
+    "small_passed_twice": (malalix_shape(768, 12, 12, 4, 64, 64, 3072, 50257, passes=2),
+                           zetunex_shape(768, 12, 12, 4, 64, 3072, 50257)),
+    # heads of 128 with values of 64, four of sixteen experts per token
+    "small_wide_heads": (malalix_shape(768, 12, 6, 2, 128, 64, 3072, 50257, experts=16, top=4),
+                         zetunex_shape(768, 12, 6, 2, 128, 3072, 50257, experts=16, top=4)),
+}
 DESIGNS = {"kosesun": (("kosesun", "gpt2"), DESIGN_SIZES), "zetunex": (("zetunex", "kosesun"), ZETUNEX_SIZES),
-           "rezelix": (("rezelix", "zetunex"), REZELIX_SIZES), "kozapel": (("kozapel", "kosesun"), KOZAPEL_SIZES)}
+           "rezelix": (("rezelix", "zetunex"), REZELIX_SIZES), "kozapel": (("kozapel", "kosesun"), KOZAPEL_SIZES),
+           "malalix": (("malalix", "zetunex"), MALALIX_SIZES)}
 
 
 def design_comparison(args):
@@ -749,7 +781,7 @@ def main(argv=None):
     parser.add_argument("--rows", default="1,8,64", help="decode batch sizes of --kernels")
     parser.add_argument("--only", help="--kernels: only kernels whose name holds one of these (comma-separated)")
     parser.add_argument("--no-prefill", action="store_true", help="--kernels: decode tables only")
-    parser.add_argument("--design", choices=("kosesun", "zetunex", "rezelix", "kozapel"), default=None,
+    parser.add_argument("--design", choices=tuple(DESIGNS), default=None,
                         help="prefill and decode throughput of this design beside the closest other one at equal size")
     parser.add_argument("--sizes", default="small,small_narrow,medium", help="--design: which sizes")
     args = parser.parse_args(argv)

@@ -269,10 +269,10 @@ __device__ inline RotationPlace rotation_place(int d, int rot_dims, bool halves)
 // root mean square over its key_dim dimensions, after the rotation (1) or before it (2), and
 // multiplied by a weight per dimension that all heads share (q_gamma, k_gamma; null: none).  Values are the
 // columns at v_col as projected (they may be the key columns themselves: values that are the
-// unrotated, unnormed keys).  A block per token, a wave per head in turn; a lane holds up to
-// four dimensions of the head.
-template <typename T>
-__global__ __launch_bounds__(256) void attention_prepare_heads_kernel(
+// unrotated, unnormed keys).  A block per token; a wave takes HB heads (of queries, keys or values)
+// at a time, all of whose loads are on their way together, a lane NR dimensions of each.
+template <typename T, int NR, int HB>
+__global__ __launch_bounds__(1024) void attention_prepare_heads_kernel(
     const float* __restrict__ proj, int64_t ld, int q_col, int k_col, int v_col,
     T* __restrict__ q_out, int64_t q_stride, T* __restrict__ k_pool, T* __restrict__ v_pool,
     const float* __restrict__ freqs, int rot_dims, int halves, float magnitude, int head_norm,
@@ -283,12 +283,49 @@ __global__ __launch_bounds__(256) void attention_prepare_heads_kernel(
   __shared__ float s_cos[128], s_sin[128];
   const int t = blockIdx.x;
   const float* row = proj + (int64_t)t * ld;
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), waves = blockDim.x >> 6;
+  const int total = heads + 2 * kv_heads;      // query heads, key heads, value heads
+  float value[HB][NR], other[HB][NR];          // a lane's dimensions, and the other ones of their pairs
+  int partner[NR];
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    const int d = lane + 64 * r;
+    partner[r] = d < rot_dims ? rotation_place(d, rot_dims, halves != 0).partner : -1;
+  }
+  auto load = [&](const int base) {
+#pragma unroll
+    for (int b = 0; b < HB; ++b) {
+      const int hh = base + b * waves;
+      const bool is_v = hh >= heads + kv_heads;
+      const int own = is_v ? value_dim : key_dim;
+      const float* src = is_v ? row + v_col + (hh - heads - kv_heads) * value_dim
+                              : (hh < heads ? row + q_col + hh * key_dim : row + k_col + (hh - heads) * key_dim);
+#pragma unroll
+      for (int r = 0; r < NR; ++r) {
+        const int d = lane + 64 * r;
+        value[b][r] = hh < total && d < own ? src[d] : 0.f;
+        other[b][r] = hh < total && !is_v && partner[r] >= 0 ? src[partner[r]] : 0.f;
+      }
+    }
+  };
+  load(wave);
   const int pos = tok_pos[t];
   const int logical = pos / page_size;
   int page = -1;
   if (logical < table_width) page = tables[(int64_t)tok_item[t] * table_width + logical];
   const bool stored = page >= 0 && page < num_pages;
   const int offset = pos - logical * page_size;
+  // weights of a lane's dimensions: of the queries' norm, of the keys', and of the pairs' other ones
+  float q_weight[NR], k_weight[NR], q_other[NR], k_other[NR];
+#pragma unroll
+  for (int r = 0; r < NR; ++r) {
+    const int d = lane + 64 * r;
+    q_weight[r] = q_gamma != nullptr && d < key_dim ? q_gamma[d] : 1.f;
+    k_weight[r] = k_gamma != nullptr && d < key_dim ? k_gamma[d] : 1.f;
+    q_other[r] = q_gamma != nullptr && partner[r] >= 0 ? q_gamma[partner[r]] : 1.f;
+    k_other[r] = k_gamma != nullptr && partner[r] >= 0 ? k_gamma[partner[r]] : 1.f;
+  }
   for (int i = threadIdx.x; i < rot_dims / 2; i += blockDim.x) {
     float sn, cs;
     sincosf((float)pos * freqs[i], &sn, &cs);
@@ -296,72 +333,68 @@ __global__ __launch_bounds__(256) void attention_prepare_heads_kernel(
     s_sin[i] = sn * magnitude;
   }
   __syncthreads();
-  const int lane = threadIdx.x & 63;
-  const int wave = threadIdx.x >> 6, waves = blockDim.x >> 6;
-  for (int hh = wave; hh < heads + kv_heads; hh += waves) {
-    const bool is_q = hh < heads;
-    const int head = is_q ? hh : hh - heads;
-    const float* src = row + (is_q ? q_col : k_col) + head * key_dim;
-    const float* gamma = is_q ? q_gamma : k_gamma;
-    const bool norm_first = head_norm == 2;
-    // every load of a lane's dimensions, and of the pairs' other ones, before anything waits
-    float value[4], other[4], weight[4], other_weight[4];
-    float squares = 0.f;
+  float turn_cos[NR], turn_sin[NR];      // (the sine with its sign)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int d = lane + 64 * r;
-      value[r] = d < key_dim ? src[d] : 0.f;
-      weight[r] = (gamma != nullptr && d < key_dim) ? gamma[d] : 1.f;
-      other[r] = 0.f;
-      other_weight[r] = 1.f;
-      if (d < rot_dims) {
-        const int partner = rotation_place(d, rot_dims, halves != 0).partner;
-        other[r] = src[partner];
-        if (gamma != nullptr) other_weight[r] = gamma[partner];
-      }
-      squares = fmaf(value[r], value[r], squares);
-    }
-    float inv = 1.f;
-    if (norm_first) {
-      const float before = 1.0f / sqrtf(wave_sum(squares) / (float)key_dim + eps);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        value[r] *= before * weight[r];
-        other[r] *= before * other_weight[r];
-      }
-    }
-    squares = 0.f;
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int d = lane + 64 * r;
-      if (d < rot_dims) {
-        const RotationPlace place = rotation_place(d, rot_dims, halves != 0);
-        value[r] = value[r] * s_cos[place.angle] + place.sign * other[r] * s_sin[place.angle];
-      }
-      squares = fmaf(value[r], value[r], squares);
-    }
-    if (head_norm == 1) {
-      inv = 1.0f / sqrtf(wave_sum(squares) / (float)key_dim + eps);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) value[r] *= weight[r];
-    }
-    T* dst = nullptr;
-    if (is_q) dst = q_out + (int64_t)t * q_stride + (int64_t)head * cache_dim;
-    else if (stored) dst = k_pool + (((int64_t)page * kv_heads + head) * page_size + offset) * cache_dim;
-    if (dst != nullptr) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int d = lane + 64 * r;
-        if (d < cache_dim) dst[d] = from_float<T>(value[r] * inv);   // (zeros behind key_dim)
-      }
+  for (int r = 0; r < NR; ++r) {
+    const int d = lane + 64 * r;
+    turn_cos[r] = 1.f;
+    turn_sin[r] = 0.f;
+    if (d < rot_dims) {
+      const RotationPlace place = rotation_place(d, rot_dims, halves != 0);
+      turn_cos[r] = s_cos[place.angle];
+      turn_sin[r] = place.sign * s_sin[place.angle];
     }
   }
-  if (!stored) return;
-  for (int i = threadIdx.x; i < kv_heads * cache_dim; i += blockDim.x) {
-    const int head = i / cache_dim;
-    const int d = i - head * cache_dim;
-    const float v = d < value_dim ? row[v_col + head * value_dim + d] : 0.f;
-    v_pool[(((int64_t)page * kv_heads + head) * page_size + offset) * cache_dim + d] = from_float<T>(v);
+  for (int base = wave; base < total; base += waves * HB) {
+    if (base != wave) load(base);
+#pragma unroll
+    for (int b = 0; b < HB; ++b) {
+      const int hh = base + b * waves;
+      if (hh >= total) break;
+      const bool is_q = hh < heads, is_v = hh >= heads + kv_heads;
+      float out[NR];
+      if (is_v) {
+#pragma unroll
+        for (int r = 0; r < NR; ++r) out[r] = value[b][r];
+      } else {
+        float before = 1.f, after = 1.f;
+        if (head_norm == 2) {
+          float squares = 0.f;
+#pragma unroll
+          for (int r = 0; r < NR; ++r) squares = fmaf(value[b][r], value[b][r], squares);
+          before = 1.0f / sqrtf(wave_sum(squares) / (float)key_dim + eps);
+        }
+#pragma unroll
+        for (int r = 0; r < NR; ++r) {
+          float v = value[b][r], o = other[b][r];
+          if (head_norm == 2) {
+            v *= before * (is_q ? q_weight[r] : k_weight[r]);
+            o *= before * (is_q ? q_other[r] : k_other[r]);
+          }
+          out[r] = v * turn_cos[r] + o * turn_sin[r];
+        }
+        if (head_norm == 1) {
+          float squares = 0.f;
+#pragma unroll
+          for (int r = 0; r < NR; ++r) squares = fmaf(out[r], out[r], squares);
+          after = 1.0f / sqrtf(wave_sum(squares) / (float)key_dim + eps);
+#pragma unroll
+          for (int r = 0; r < NR; ++r) out[r] *= after * (is_q ? q_weight[r] : k_weight[r]);
+        }
+      }
+      T* dst = nullptr;
+      if (is_q) dst = q_out + (int64_t)t * q_stride + (int64_t)hh * cache_dim;
+      else if (stored)
+        dst = (is_v ? v_pool : k_pool) +
+              (((int64_t)page * kv_heads + (is_v ? hh - heads - kv_heads : hh - heads)) * page_size + offset) * cache_dim;
+      if (dst != nullptr) {
+#pragma unroll
+        for (int r = 0; r < NR; ++r) {
+          const int d = lane + 64 * r;
+          if (d < cache_dim) dst[d] = from_float<T>(out[r]);   // (zeros behind the head's own size)
+        }
+      }
+    }
   }
 }
 
@@ -391,16 +424,25 @@ extern "C" int ps_attention_prepare_heads(const float* proj, int64_t ld, int q_c
   PS_REQUIRE(dtype == PS_F32 || dtype == PS_BF16, "ps_attention_prepare_heads: unknown dtype %d", dtype);
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-  if (dtype == PS_F32)
-    hipLaunchKernelGGL(attention_prepare_heads_kernel<float>, dim3(tokens), dim3(256), 0, s, proj, ld,
-                       q_col, k_col, v_col, (float*)q_out, q_stride, (float*)k_pool, (float*)v_pool,
-                       freqs, rot_dims, halves, magnitude, head_norm, q_gamma, k_gamma, eps, tok_item, tok_pos, tables,
-                       table_width, heads, kv_heads, key_dim, value_dim, cache_dim, page_size, num_pages);
-  else
-    hipLaunchKernelGGL(attention_prepare_heads_kernel<bf16_t>, dim3(tokens), dim3(256), 0, s, proj, ld,
-                       q_col, k_col, v_col, (bf16_t*)q_out, q_stride, (bf16_t*)k_pool, (bf16_t*)v_pool,
-                       freqs, rot_dims, halves, magnitude, head_norm, q_gamma, k_gamma, eps, tok_item, tok_pos, tables,
-                       table_width, heads, kv_heads, key_dim, value_dim, cache_dim, page_size, num_pages);
+  // few tokens: a wave per head where the block has room; many fill the chip with four waves each
+  const int total = heads + 2 * kv_heads;
+  const int threads = tokens <= 256 ? 64 * (total < 16 ? total : 16) : 256;
+#define PS_PREPARE_HEADS(T, NR, HB)                                                                \
+  hipLaunchKernelGGL((attention_prepare_heads_kernel<T, NR, HB>), dim3(tokens), dim3(threads), 0, s, proj, \
+                     ld, q_col, k_col, v_col, (T*)q_out, q_stride, (T*)k_pool, (T*)v_pool, freqs,   \
+                     rot_dims, halves, magnitude, head_norm, q_gamma, k_gamma, eps, tok_item,       \
+                     tok_pos, tables, table_width, heads, kv_heads, key_dim, value_dim, cache_dim,  \
+                     page_size, num_pages)
+#define PS_PREPARE_HEADS_OF(T)                       \
+  do {                                               \
+    if (cache_dim <= 64) PS_PREPARE_HEADS(T, 1, 5);  \
+    else if (cache_dim <= 128) PS_PREPARE_HEADS(T, 2, 3); \
+    else PS_PREPARE_HEADS(T, 4, 2);                  \
+  } while (0)
+  if (dtype == PS_F32) PS_PREPARE_HEADS_OF(float);
+  else PS_PREPARE_HEADS_OF(bf16_t);
+#undef PS_PREPARE_HEADS_OF
+#undef PS_PREPARE_HEADS
   PS_CHECK_LAUNCH("ps_attention_prepare_heads");
   return 0;
 }

@@ -533,6 +533,206 @@ __global__ __launch_bounds__(256) void moe_down_wide_kernel(
   }
 }
 
+// ---- few rows in bfloat16: by expert, on the matrix cores ---------------------------------------
+// A group of a step's tokens: up to 16 (the columns of a product) and up to 64 (token, routed choice)
+// pairs (a lane each).  An expert's rows are read once per group, for all its tokens that chose it.
+#define MOE_GROUP 16
+
+typedef __attribute__((__vector_size__(4 * sizeof(float)))) float moe_f32x4;
+typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 moe_bf16x8;
+
+// The experts that a wave's group of tokens chose, a pair per lane: pair p is choice p % top of
+// the group's token p / top (-1 behind the last pair).
+__device__ inline int group_choice(const int* __restrict__ ids, int t0, int pairs, int top, int cols, int lane) {
+  const int t = lane / top;
+  return lane < pairs ? ids[(int64_t)(t0 + t) * cols + (lane - t * top)] : -1;
+}
+
+// Eight bfloat16 of a row from place k on (zeros behind its end).
+__device__ inline moe_bf16x8 moe_operand(const bf16_t* row, int k, int end) {
+  uint4 raw = {0u, 0u, 0u, 0u};
+  if (k < end) raw = *reinterpret_cast<const uint4*>(row + k);
+  return *reinterpret_cast<const moe_bf16x8*>(&raw);
+}
+
+#define MOE_STEPS 6      // k steps of 32 whose loads a wave has on their way together
+
+// The hidden rows.  Block (columns, slot, group) does the expert of the group's pair `slot` if that
+// is the first pair with it, for all of the group's tokens that chose it (the last slot: the
+// extra expert, for all of them).  S[weight row][token] = W X^T with v_mfma_f32_16x16x32_bf16: two tiles
+// of 16 weight rows, the gate and the up rows of 16 hidden columns (the plain form: 32 columns); the
+// four waves share k between them and meet in LDS.  (Columns run fastest: workgroups go round the XCDs,
+// and slots running fastest would leave a step whose tokens agree on two experts to two XCDs.)
+template <bool GATED>
+__global__ __launch_bounds__(256) void moe_hidden_group_kernel(
+    const bf16_t* __restrict__ x, int64_t x_ld, const bf16_t* __restrict__ w1, const int* __restrict__ ids,
+    bf16_t* __restrict__ hidden, int tokens, int group, int width, int inner, int top, GateForm form,
+    const ExtraExpert<bf16_t> extra) {
+  __shared__ float s_acc[4][8][64];
+  const int t0 = blockIdx.z * group;
+  const int count = tokens - t0 < group ? tokens - t0 : group;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / 64), lane = threadIdx.x % 64;
+  const int r = lane & 15, g = lane >> 4;
+  const int slot = blockIdx.y;
+  const bool has_extra = extra.inner > 0;
+  const int held = top * inner + extra.inner;
+  const bool is_extra = has_extra && slot == (int)gridDim.y - 1;
+  const int pairs = count * top;
+  const int columns = is_extra ? extra.inner : inner;
+  const int first = blockIdx.x * (GATED ? 16 : 32);
+  if (first >= columns || (!is_extra && slot >= pairs)) return;
+  const bf16_t* matrix = extra.w1;
+  // which of its choices is this expert, by token (of the column r): a bit each
+  unsigned long long own = 1ull;
+  int base = top * inner;
+  if (!is_extra) {
+    const int mine = group_choice(ids, t0, pairs, top, top + (has_extra ? 1 : 0), lane);
+    const int e = __builtin_amdgcn_readlane(mine, slot);
+    const unsigned long long takers = __ballot(mine == e);
+    if (__builtin_ctzll(takers) < slot) return;      // (an earlier pair's block does it)
+    matrix = w1 + (int64_t)e * (GATED ? 2 : 1) * inner * width;
+    own = r < count ? (takers >> (r * top)) & (~0ull >> (64 - top)) : 0ull;
+    base = 0;
+  } else {
+    form = extra.form;
+  }
+  const bf16_t* rows[2];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int c = first + (GATED ? 0 : 16 * j) + r;
+    rows[j] = matrix + ((int64_t)(GATED ? j * columns : 0) + (c < columns ? c : columns - 1)) * width;
+  }
+  const bf16_t* token = x + (int64_t)(t0 + (r < count ? r : 0)) * x_ld;
+  const int steps = (width + 31) / 32, share = (steps + 3) / 4;
+  const int end = min((wave + 1) * share * 32, width);
+  moe_f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+  for (int k0 = wave * share * 32; k0 < end; k0 += MOE_STEPS * 32) {
+    moe_bf16x8 fa[2][MOE_STEPS], fb[MOE_STEPS];
+#pragma unroll
+    for (int s = 0; s < MOE_STEPS; ++s) {
+      const int k = k0 + s * 32 + 8 * g;
+      fa[0][s] = moe_operand(rows[0], k, end);
+      fa[1][s] = moe_operand(rows[1], k, end);
+      fb[s] = moe_operand(token, k, end);
+    }
+#pragma unroll
+    for (int s = 0; s < MOE_STEPS; ++s) {
+      acc[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[0][s], fb[s], acc[0], 0, 0, 0);
+      acc[1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[1][s], fb[s], acc[1], 0, 0, 0);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    s_acc[wave][i][lane] = acc[0][i];
+    s_acc[wave][4 + i][lane] = acc[1][i];
+  }
+  __syncthreads();
+  // wave i finishes element i of both tiles: weight row 4 g + i, token r
+  const int i = wave;
+  float a = 0.f, b = 0.f;
+#pragma unroll
+  for (int w = 0; w < 4; ++w) {
+    a += s_acc[w][i][lane];
+    b += s_acc[w][4 + i][lane];
+  }
+  if (r >= count) return;
+  const int c = first + 4 * g + i;
+  bf16_t* row = hidden + (int64_t)(t0 + r) * held + base;
+  for (; own != 0; own &= own - 1) {
+    bf16_t* at = row + __builtin_ctzll(own) * inner * (is_extra ? 0 : 1);
+    if (GATED) {
+      if (c < columns) at[c] = from_float<bf16_t>(moe_activation<true>(a, b, form));
+    } else {
+      if (c < columns) at[c] = from_float<bf16_t>(moe_activation<false>(a, 0.f, form));
+      if (c + 16 < columns) at[c + 16] = from_float<bf16_t>(moe_activation<false>(b, 0.f, form));
+    }
+  }
+}
+
+#define MOE_PIECE 256        // hidden columns of an expert that a wave of the kernel below takes at a time
+#define MOE_DOWN_WAVES 8
+
+// The down projection: block (16 output columns, share, group).  The waves of all shares divide the
+// pieces of MOE_PIECE hidden columns of all experts that the group chose; Y^T[column][token] of a
+// piece, times each token's weight of the expert, is summed over a block's waves in LDS and over the
+// shares with float atomics.
+__global__ __launch_bounds__(64 * MOE_DOWN_WAVES) void moe_down_group_kernel(
+    const bf16_t* __restrict__ hidden, const bf16_t* __restrict__ w2, const int* __restrict__ ids,
+    const float* __restrict__ weights, float* __restrict__ y, int tokens, int group, int width,
+    int inner, int top, const ExtraExpert<bf16_t> extra) {
+  __shared__ float s_sum[MOE_DOWN_WAVES][4][64];
+  const int t0 = blockIdx.z * group;
+  const int count = tokens - t0 < group ? tokens - t0 : group;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / 64), lane = threadIdx.x % 64;
+  const int r = lane & 15, g = lane >> 4;
+  const int cols = top + (extra.inner > 0 ? 1 : 0);
+  const int pairs = count * top;
+  const int held = top * inner + extra.inner;
+  const int first = blockIdx.x * 16;
+  const int mine = group_choice(ids, t0, pairs, top, cols, lane);
+  // the first pair of every expert that was chosen
+  bool again = lane >= pairs;
+  for (int p = 0; p + 1 < pairs; ++p) again |= lane > p && mine == __builtin_amdgcn_readlane(mine, p);
+  const unsigned long long firsts = __ballot(!again);
+  const int experts = __builtin_popcountll(firsts);
+  const int per_expert = (inner + MOE_PIECE - 1) / MOE_PIECE;
+  const int pieces = experts * per_expert + (extra.inner + MOE_PIECE - 1) / MOE_PIECE;
+  const int column = first + r < width ? first + r : width - 1;
+  const int t = t0 + (r < count ? r : 0);
+  moe_f32x4 sum = {0.f, 0.f, 0.f, 0.f};
+  for (int p = blockIdx.y * MOE_DOWN_WAVES + wave; p < pieces; p += gridDim.y * MOE_DOWN_WAVES) {
+    const bool is_extra = p >= experts * per_expert;
+    const int which = is_extra ? experts : p / per_expert;
+    const int columns = is_extra ? extra.inner : inner;
+    const int k0 = (p - which * per_expert) * MOE_PIECE;
+    const bf16_t* matrix = extra.w2;
+    const bf16_t* row = hidden + (int64_t)t * held;
+    float weight = 0.f;
+    bool chose = r < count;
+    if (!is_extra) {
+      unsigned long long left = firsts;
+      for (int skip = 0; skip < which; ++skip) left &= left - 1;
+      const int e = __builtin_amdgcn_readlane(mine, __builtin_ctzll(left));
+      const unsigned long long takers = __ballot(mine == e);
+      unsigned long long own = chose ? (takers >> (r * top)) & (~0ull >> (64 - top)) : 0ull;
+      matrix = w2 + (int64_t)e * width * inner;
+      chose = own != 0;
+      if (chose) row += __builtin_ctzll(own) * inner;
+      // (the rows of an expert that a token names twice are alike)
+      for (; own != 0; own &= own - 1) weight += weights[(int64_t)t * cols + __builtin_ctzll(own)];
+    } else {
+      row += top * inner;
+      if (chose) weight = weights[(int64_t)t * cols + top];
+    }
+    const bf16_t* w_row = matrix + (int64_t)column * columns;
+    const int end = chose ? columns : 0;      // (a token that did not choose the expert: zeros)
+    moe_bf16x8 fa[MOE_PIECE / 32], fb[MOE_PIECE / 32];
+#pragma unroll
+    for (int s = 0; s < MOE_PIECE / 32; ++s) {
+      const int k = k0 + s * 32 + 8 * g;
+      fa[s] = moe_operand(w_row, k, columns);
+      fb[s] = moe_operand(row, k, end);
+    }
+    moe_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < MOE_PIECE / 32; ++s)
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[s], fb[s], acc, 0, 0, 0);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) sum[i] = fmaf(weight, acc[i], sum[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) s_sum[wave][i][lane] = sum[i];
+  __syncthreads();
+  // thread (i, lane): column 4 g + i, token r
+  if (wave >= 4 || r >= count || first + 4 * g + wave >= width) return;
+  float total = 0.f;
+#pragma unroll
+  for (int w = 0; w < MOE_DOWN_WAVES; ++w) total += s_sum[w][wave][lane];
+  float* at = y + (int64_t)(t0 + r) * width + first + 4 * g + wave;
+  if (gridDim.y == 1) *at += total;
+  else unsafeAtomicAdd(at, total);
+}
+
 // ---- many rows: the (token, choice) pairs sorted by expert, products on the matrix cores -------
 #define MOE_TILE 128     // pairs per tile; an expert's pairs are padded up to whole tiles
 
@@ -568,7 +768,6 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
 }
 
 typedef __attribute__((__vector_size__(16 * sizeof(float)))) float moe_f32x16;
-typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 moe_bf16x8;
 #define MOE_LDS_STRIDE 80   // bytes between rows of a stage (64 bytes of k, padded)
 #define MOE_DEPTH 4         // k tiles whose global loads are in flight
 
@@ -741,8 +940,6 @@ extern "C" int ps_moe_experts(const void* x, int64_t x_ld, const void* w1, const
   PS_REQUIRE(inner_x >= 0 && (inner_x == 0 || (top > 1 && w1x != nullptr && w2x != nullptr)),
              "ps_moe_experts: an expert for every token needs its matrices and its place behind the chosen ones");
   const int held = (inner_x > 0 ? top - 1 : top) * inner + inner_x;      // hidden columns of a token
-  PS_REQUIRE((size_t)width * 4 <= 64 * 1024 && (size_t)held * 4 <= 64 * 1024,
-             "ps_moe_experts: width %d or %d hidden columns of a token do not fit LDS", width, held);
   PS_REQUIRE(limit > 0.f && (inner_x == 0 || limit_x > 0.f), "ps_moe_experts: limits must be positive");
   PS_REQUIRE(dtype == PS_F32 || dtype == PS_BF16, "ps_moe_experts: unknown dtype %d", dtype);
   if (tokens == 0) return 0;
@@ -750,6 +947,37 @@ extern "C" int ps_moe_experts(const void* x, int64_t x_ld, const void* w1, const
   const bool wide1 = width % 8 == 0 && x_ld % 8 == 0, wide2 = inner % 8 == 0 && inner_x % 8 == 0;
   const int widest = inner > inner_x ? inner : inner_x;
   const GateForm form = {limit, slope, shift};
+  const int routed = inner_x > 0 ? top - 1 : top;
+  if (dtype == PS_BF16 && wide1 && wide2 && routed <= 64) {
+    const int group = MOE_GROUP * routed <= 64 ? MOE_GROUP : 64 / routed;
+    const int groups = (tokens + group - 1) / group;
+    const int most = tokens < group ? tokens : group;       // tokens of the fullest group
+    PS_REQUIRE(groups <= 65535, "ps_moe_experts: %d groups of tokens are too many", groups);
+    const ExtraExpert<bf16_t> extra = {(const bf16_t*)w1x, (const bf16_t*)w2x, inner_x, {limit_x, slope, shift}};
+    const int block = gated ? 16 : 32;
+    const dim3 grid1((widest + block - 1) / block, most * routed + (inner_x > 0 ? 1 : 0), groups);
+    if (gated)
+      hipLaunchKernelGGL(moe_hidden_group_kernel<true>, grid1, dim3(256), 0, s, (const bf16_t*)x, x_ld,
+                         (const bf16_t*)w1, ids, (bf16_t*)hidden, tokens, group, width, inner, routed, form, extra);
+    else
+      hipLaunchKernelGGL(moe_hidden_group_kernel<false>, grid1, dim3(256), 0, s, (const bf16_t*)x, x_ld,
+                         (const bf16_t*)w1, ids, (bf16_t*)hidden, tokens, group, width, inner, routed, form, extra);
+    // shares of the pieces until a block comes to every compute unit, no share without a piece
+    const int tiles = (width + 15) / 16;
+    const int pieces = most * routed * ((inner + MOE_PIECE - 1) / MOE_PIECE) + (inner_x + MOE_PIECE - 1) / MOE_PIECE;
+    int shares = ps_compute_units() / (tiles * groups);
+    const int useful = (pieces + MOE_DOWN_WAVES - 1) / MOE_DOWN_WAVES;
+    if (shares > useful) shares = useful;
+    if (shares > 8) shares = 8;
+    if (shares < 1) shares = 1;
+    hipLaunchKernelGGL(moe_down_group_kernel, dim3(tiles, shares, groups), dim3(64 * MOE_DOWN_WAVES), 0, s,
+                       (const bf16_t*)hidden, (const bf16_t*)w2, ids, weights, y, tokens, group, width,
+                       inner, routed, extra);
+    PS_CHECK_LAUNCH("ps_moe_experts");
+    return 0;
+  }
+  PS_REQUIRE((size_t)width * 4 <= 64 * 1024 && (size_t)held * 4 <= 64 * 1024,
+             "ps_moe_experts: width %d or %d hidden columns of a token do not fit LDS", width, held);
   // hidden columns / output columns per wave: four, or two while that still leaves the chip
   // short of blocks (a handful of decoded tokens)
   const bool few = (int64_t)tokens * ((width + 15) / 16) < 4 * ps_compute_units();

@@ -8,7 +8,8 @@
 // One pass over the stream's rows, every piece optional:
 //   h <- h + factor * column_scale * y + rows + bias;   zero <- 0 (may be y);
 //   normed <- h / sqrt(mean(h^2) + eps) * gamma;   normed2 <- the same * gamma2
-// (column_scale: a float per column, null for ones).  A block per token.
+// (column_scale: a float per column, null for ones).  A block of 256 threads per token.
+#define STREAM_HELD 8      // numbers of a row that a thread may hold
 template <typename T>
 __global__ __launch_bounds__(256) void stream_step_kernel(
     float* __restrict__ h, const float* y, float factor, const float* __restrict__ column_scale,
@@ -18,6 +19,45 @@ __global__ __launch_bounds__(256) void stream_step_kernel(
   const int64_t t = blockIdx.x;
   float* row = h + t * width;
   float sum = 0.f;
+  if (width <= 256 * STREAM_HELD) {
+    // rows that a block holds in registers, with the scales asked for beside them: one trip to
+    // memory and no second reading of the row
+    float held[STREAM_HELD], scale[STREAM_HELD], scale2[STREAM_HELD];
+#pragma unroll
+    for (int i = 0; i < STREAM_HELD; ++i) {
+      const int d = threadIdx.x + 256 * i;
+      held[i] = scale[i] = scale2[i] = 0.f;
+      if (d < width) {
+        float v = row[d];
+        if (gamma != nullptr) scale[i] = gamma[d];
+        if (gamma2 != nullptr) scale2[i] = gamma2[d];
+        if (y != nullptr) v = fmaf(column_scale ? factor * column_scale[d] : factor, y[t * width + d], v);
+        if (rows != nullptr) v += rows[t * width + d];
+        if (bias != nullptr) v += bias[d];
+        held[i] = v;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < STREAM_HELD; ++i) {
+      const int d = threadIdx.x + 256 * i;
+      if (d < width) {
+        if (y != nullptr || rows != nullptr || bias != nullptr) row[d] = held[i];
+        if (zero != nullptr) zero[t * width + d] = 0.f;
+      }
+      sum = fmaf(held[i], held[i], sum);
+    }
+    if (gamma == nullptr) return;
+    const float inv = 1.0f / sqrtf(block_sum(sum, scratch) / (float)width + eps);
+#pragma unroll
+    for (int i = 0; i < STREAM_HELD; ++i) {
+      const int d = threadIdx.x + 256 * i;
+      if (d < width) {
+        normed[t * width + d] = from_float<T>(held[i] * inv * scale[i]);
+        if (gamma2 != nullptr) normed2[t * width + d] = from_float<T>(held[i] * inv * scale2[i]);
+      }
+    }
+    return;
+  }
   for (int d = threadIdx.x; d < width; d += blockDim.x) {
     float v = row[d];
     if (y != nullptr) v = fmaf(column_scale ? factor * column_scale[d] : factor, y[t * width + d], v);

@@ -195,9 +195,10 @@ class MixtureOfExperts(FeedForward):
                 raise ValueError("a gate for the shared expert goes with the gated form")
             else:
                 self.shared = DenseFeedForward(width, dtype, shared_inner, "relu2", bias=False)
-        # whether the shared expert may ride along in the row kernels (they keep a token's hidden
-        # rows of all its experts in LDS)
-        self.shared_rides = bool(shared_inner) and (top * inner + shared_inner) * 4 <= 64 * 1024
+        # whether the shared expert may ride along in the row kernels (at inner widths that are no
+        # multiples of 8 they keep a token's hidden rows of all its experts in LDS)
+        self.shared_rides = bool(shared_inner) and (
+            (inner % 8 == 0 and shared_inner % 8 == 0) or (top * inner + shared_inner) * 4 <= 64 * 1024)
 
     def parameters(self):
         params = {
