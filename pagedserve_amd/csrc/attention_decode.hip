@@ -244,7 +244,7 @@ extern "C" int ps_attention_decode_partial(const void* q, int64_t q_stride, cons
                                            const int* tables, int table_width, int count,
                                            int heads, int kv_heads, int head_dim, int page_size,
                                            int num_pages, float scale, int window, int splits,
-                                           int waves, const float* sink, float softcap, int dtype,
+                                           int waves, const float* sink, float softcap, const float* logistic, float logistic_norm, int dtype,
                                            void* stream) {
   if (check_decode_sizes("ps_attention_decode_partial", count, heads, kv_heads, head_dim,
                          page_size, num_pages, table_width, splits, waves, dtype))
@@ -257,10 +257,10 @@ extern "C" int ps_attention_decode_partial(const void* q, int64_t q_stride, cons
   if (dtype == PS_F32)
     return launch_decode<float>(q, q_stride, k_pool, v_pool, nullptr, 0, partial, tok_list,
                                 tok_item, tok_pos, tables, table_width, count, heads, kv_heads,
-                                head_dim, page_size, num_pages, scale, window, splits, waves, AttnExtras{sink, nullptr, 0, softcap}, s);
+                                head_dim, page_size, num_pages, scale, window, splits, waves, AttnExtras{sink, nullptr, 0, softcap, logistic, logistic_norm}, s);
   return launch_decode<bf16_t>(q, q_stride, k_pool, v_pool, nullptr, 0, partial, tok_list,
                                tok_item, tok_pos, tables, table_width, count, heads, kv_heads,
-                               head_dim, page_size, num_pages, scale, window, splits, waves, AttnExtras{sink, nullptr, 0, softcap}, s);
+                               head_dim, page_size, num_pages, scale, window, splits, waves, AttnExtras{sink, nullptr, 0, softcap, logistic, logistic_norm}, s);
 }
 
 extern "C" int ps_attention_decode(const void* q, int64_t q_stride, const void* k_pool,
@@ -270,7 +270,7 @@ extern "C" int ps_attention_decode(const void* q, int64_t q_stride, const void* 
                                    int table_width, int count, int heads, int kv_heads,
                                    int head_dim, int page_size, int num_pages, float scale,
                                    int window, int splits, int waves, const float* sink,
-                                   const float* gate, int64_t gate_ld, float softcap, int dtype,
+                                   const float* gate, int64_t gate_ld, float softcap, const float* logistic, float logistic_norm, int dtype,
                                    void* stream) {
   if (check_decode_sizes("ps_attention_decode", count, heads, kv_heads, head_dim, page_size,
                          num_pages, table_width, splits, waves, dtype))
@@ -287,8 +287,8 @@ extern "C" int ps_attention_decode(const void* q, int64_t q_stride, const void* 
   if (dtype == PS_F32)
     return launch_decode<float>(q, q_stride, k_pool, v_pool, out, out_stride, partial, tok_list,
                                 tok_item, tok_pos, tables, table_width, count, heads, kv_heads,
-                                head_dim, page_size, num_pages, scale, window, splits, waves, AttnExtras{sink, gate, gate_ld, softcap}, s);
+                                head_dim, page_size, num_pages, scale, window, splits, waves, AttnExtras{sink, gate, gate_ld, softcap, logistic, logistic_norm}, s);
   return launch_decode<bf16_t>(q, q_stride, k_pool, v_pool, out, out_stride, partial, tok_list,
                                tok_item, tok_pos, tables, table_width, count, heads, kv_heads,
-                               head_dim, page_size, num_pages, scale, window, splits, waves, AttnExtras{sink, gate, gate_ld, softcap}, s);
+                               head_dim, page_size, num_pages, scale, window, splits, waves, AttnExtras{sink, gate, gate_ld, softcap, logistic, logistic_norm}, s);
 }

@@ -103,6 +103,12 @@ __device__ __forceinline__ void attention_decode_block(
     m = extra.sink[head] * 1.4426950408889634f;
     l = 1.f;
   }
+  const bool logistic = extra.logistic != nullptr;
+  const float shift = logistic ? extra.logistic[head] * 1.4426950408889634f : 0.f;
+  if (logistic) {
+    m = 0.f;
+    if (split == 0 && wave == 0 && group == 0) l = extra.logistic_norm;
+  }
   float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
 
   for (int base = range_begin + wave * KEYS_PER_WAVE; base < range_end;
@@ -163,7 +169,16 @@ __device__ __forceinline__ void attention_decode_block(
       s[u] = valid[u] ? score : -INFINITY;
       m_new = fmaxf(m_new, s[u]);
     }
-    if (m_new != -INFINITY) {
+    if (logistic) {
+#pragma unroll
+      for (int u = 0; u < AD_UNROLL; ++u) {
+        const float p = valid[u] ? logistic_weight_as<T>(s[u] + shift) : 0.f;
+        float vf[8];
+        vr[u].widen(vf);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[i] = valid[u] ? fmaf(p, vf[i], acc[i]) : acc[i];
+      }
+    } else if (m_new != -INFINITY) {
       const float correction = (m == -INFINITY) ? 0.f : exp2_fast<T>(m - m_new);
       l *= correction;
 #pragma unroll

@@ -54,6 +54,8 @@ struct AdsArgs {
   int window, splits;
   float softcap_log2;
   int page_shift, pieces_shift;     // log2 of the page size and of head_dim / 8, or -1
+  const float* logistic;            // (common.h: AttnExtras)
+  float logistic_norm;
 };
 
 // dynamic LDS: keys [64][D + 8] bf16 | values the same (absent when they are the keys) |
@@ -104,8 +106,8 @@ __global__ __launch_bounds__(256) void attention_decode_shared_kernel(const AdsA
   }
   for (int i = tid; i < ADS_HEADS * ADS_PROW / 2; i += 256) reinterpret_cast<uint32_t*>(s_p)[i] = 0u;
   if (tid < ADS_HEADS) {
-    s_m[tid] = -INFINITY;
-    s_l[tid] = 0.f;
+    s_m[tid] = a.logistic ? 0.f : -INFINITY;
+    s_l[tid] = a.logistic && split == 0 ? a.logistic_norm : 0.f;
     s_f[tid] = 1.f;
   }
   // O^T: tile j of the wave covers dimensions 16 (wave + 4 j) ..; element i of a lane: dimension
@@ -174,6 +176,11 @@ __global__ __launch_bounds__(256) void attention_decode_shared_kernel(const AdsA
       float s = s_s[h * ADS_KEYS + lane];
       if (a.softcap_log2 > 0.f) s = capped_score_fast(s, a.softcap_log2);
       if (!visible) s = -INFINITY;
+      if (a.logistic != nullptr) {
+        const float p = visible ? logistic_weight_fast(s + a.logistic[head0 + h] * 1.4426950408889634f) : 0.f;
+        s_p[h * ADS_PROW + lane] = float_to_bf16(p);
+        continue;
+      }
       const float before = s_m[h];
       const float m_new = fmaxf(before, wave_max(s));          // (a tile has at least one visible key)
       const float p = visible ? __builtin_amdgcn_exp2f(s - m_new) : 0.f;
@@ -260,7 +267,8 @@ extern "C" int ps_attention_decode_shared(const void* q, int64_t q_stride, const
                                           int table_width, int count, int heads, int kv_heads,
                                           int head_dim, int page_size, int num_pages, float scale,
                                           int window, int splits, const float* gate, int64_t gate_ld,
-                                          float softcap, void* stream) {
+                                          float softcap, const float* logistic, float logistic_norm,
+                                          void* stream) {
   PS_REQUIRE(count >= 0 && heads > 0 && kv_heads > 0 && page_size > 0 && num_pages > 0 && table_width > 0,
              "ps_attention_decode_shared: bad sizes");
   PS_REQUIRE(heads % kv_heads == 0, "ps_attention_decode_shared: heads (%d) must be a multiple of kv_heads (%d)",
@@ -290,7 +298,8 @@ extern "C" int ps_attention_decode_shared(const void* q, int64_t q_stride, const
   const AdsArgs a = {(const bf16_t*)q, q_stride, (const bf16_t*)k_pool, (const bf16_t*)v_pool, partial,
                      tok_list, tok_item, tok_pos, tables, table_width, heads, kv_heads, head_dim,
                      page_size, num_pages, scale * 1.4426950408889634f, window, splits,
-                     softcap * 1.4426950408889634f, ads_shift(page_size), ads_shift(head_dim / 8)};
+                     softcap * 1.4426950408889634f, ads_shift(page_size), ads_shift(head_dim / 8),
+                     logistic, logistic_norm};
   hipLaunchKernelGGL(attention_decode_shared_kernel, dim3(count, kv_heads * parts, splits), dim3(256), lds, s, a);
   PS_CHECK_LAUNCH("ps_attention_decode_shared");
   if (out == nullptr) return 0;      // the records are all that is asked for: the caller merges them

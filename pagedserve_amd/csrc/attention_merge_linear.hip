@@ -136,7 +136,7 @@ __global__ __launch_bounds__(64 * GROUP) void attention_merge_linear_kernel(
           value[st][h][e] = fmaf(__shfl_xor(value[st][h][e], offset, 64), weight, value[st][h][e] * keep);
     total_m = new_m;
   }
-  const float inverse = (merges && total_l > 0.f) ? 1.f / total_l : 0.f;
+  const float inverse = (merges && total_l != 0.f) ? 1.f / total_l : 0.f;
 
   f32x4_t acc[TILES];
 #pragma unroll

@@ -202,6 +202,12 @@ __device__ __forceinline__ void attention_prefill_block(
     m = extra.sink[head] * 1.4426950408889634f;
     l = 1.f;
   }
+  const bool logistic = extra.logistic != nullptr;
+  const float shift = logistic ? extra.logistic[head] * 1.4426950408889634f : 0.f;
+  if (logistic) {
+    m = 0.f;
+    if (wave_k == 0) l = extra.logistic_norm;
+  }
   f32x16 acc[NDB32];
 #pragma unroll
   for (int db = 0; db < NDB32; ++db)
@@ -334,39 +340,54 @@ __device__ __forceinline__ void attention_prefill_block(
 #pragma unroll
           for (int e = 0; e < 16; ++e) tile_max = fmaxf(tile_max, s[r][e]);
       }
-      tile_max = halves_max(tile_max) * scale_log2;   // scale > 0
-      const float m_new = fmaxf(m, tile_max);
-      // A query that has seen nothing yet (m_new = -inf) takes 0 as its reference: its scores
-      // are all -inf and their exponentials 0.  Other lanes of the wave may differ, so the
-      // products below run in any case.
-      const float reference = (m_new == -INFINITY) ? 0.f : m_new;
-      float tile_sum = 0.f;
       u32x4 p[2 * KR];      // per 16 keys
+      if (logistic) {
+        // weights of their own: nothing is summed and nothing rescaled (a masked score is -inf and
+        // weighs 0)
 #pragma unroll
-      for (int r = 0; r < KR; ++r) {
-        uint32_t words[8];
+        for (int r = 0; r < KR; ++r) {
+          uint32_t words[8];
 #pragma unroll
-        for (int e = 0; e < 16; e += 2) {
-          const float p0 = __builtin_amdgcn_exp2f(fmaf(s[r][e], scale_log2, -reference));
-          const float p1 = __builtin_amdgcn_exp2f(fmaf(s[r][e + 1], scale_log2, -reference));
-          tile_sum += p0 + p1;
-          words[e >> 1] = pack2_bf16(p0, p1);
+          for (int e = 0; e < 16; e += 2)
+            words[e >> 1] = pack2_bf16(logistic_weight_fast(fmaf(s[r][e], scale_log2, shift)),
+                                       logistic_weight_fast(fmaf(s[r][e + 1], scale_log2, shift)));
+          p[2 * r] = u32x4{words[0], words[1], words[2], words[3]};
+          p[2 * r + 1] = u32x4{words[4], words[5], words[6], words[7]};
         }
-        p[2 * r] = u32x4{words[0], words[1], words[2], words[3]};
-        p[2 * r + 1] = u32x4{words[4], words[5], words[6], words[7]};
-      }
-      tile_sum = halves_sum(tile_sum);
-      // the running maximum rarely moves after the first tiles: rescale only where it did
-      if (__builtin_amdgcn_readfirstlane(__any(m_new != m) ? 1 : 0)) {
-        const float correction = (m == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(m - reference);
-        l *= correction;
+      } else {
+        tile_max = halves_max(tile_max) * scale_log2;   // scale > 0
+        const float m_new = fmaxf(m, tile_max);
+        // A query that has seen nothing yet (m_new = -inf) takes 0 as its reference: its scores
+        // are all -inf and their exponentials 0.  Other lanes of the wave may differ, so the
+        // products below run in any case.
+        const float reference = (m_new == -INFINITY) ? 0.f : m_new;
+        float tile_sum = 0.f;
 #pragma unroll
-        for (int db = 0; db < NDB32; ++db)
+        for (int r = 0; r < KR; ++r) {
+          uint32_t words[8];
 #pragma unroll
-          for (int e = 0; e < 16; ++e) acc[db][e] *= correction;
-        m = m_new;
+          for (int e = 0; e < 16; e += 2) {
+            const float p0 = __builtin_amdgcn_exp2f(fmaf(s[r][e], scale_log2, -reference));
+            const float p1 = __builtin_amdgcn_exp2f(fmaf(s[r][e + 1], scale_log2, -reference));
+            tile_sum += p0 + p1;
+            words[e >> 1] = pack2_bf16(p0, p1);
+          }
+          p[2 * r] = u32x4{words[0], words[1], words[2], words[3]};
+          p[2 * r + 1] = u32x4{words[4], words[5], words[6], words[7]};
+        }
+        tile_sum = halves_sum(tile_sum);
+        // the running maximum rarely moves after the first tiles: rescale only where it did
+        if (__builtin_amdgcn_readfirstlane(__any(m_new != m) ? 1 : 0)) {
+          const float correction = (m == -INFINITY) ? 0.f : __builtin_amdgcn_exp2f(m - reference);
+          l *= correction;
+#pragma unroll
+          for (int db = 0; db < NDB32; ++db)
+#pragma unroll
+            for (int e = 0; e < 16; ++e) acc[db][e] *= correction;
+          m = m_new;
+        }
+        l += tile_sum;
       }
-      l += tile_sum;
 
       // O^T += V^T P^T, 16 keys per instruction: slots 0..3 are keys base + half*4 + 0..3,
       // slots 4..7 keys base + 8 + half*4 + 0..3, in both operands
@@ -474,7 +495,7 @@ __device__ __forceinline__ void attention_prefill_block(
   }
 
   // element e of an accumulator: head dimension db*32 + (e/4)*8 + half*4 + e%4 of query `sub`
-  if (q_valid && l > 0.f) {
+  if (q_valid && l != 0.f) {
     const float inv = gate_factor(extra, tok0 + qi, head) / l;
     bf16_t* dst = out + (int64_t)(tok0 + qi) * out_stride + (int64_t)head * HD;
 #pragma unroll

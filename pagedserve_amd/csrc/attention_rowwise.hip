@@ -44,6 +44,12 @@ __global__ __launch_bounds__(64) void attention_rowwise_kernel(
   // a sink is a score without a key or a value: it only takes part in the denominator
   float running_max = extra.sink ? extra.sink[head] : -INFINITY;
   float running_sum = extra.sink ? 1.f : 0.f;
+  const bool logistic = extra.logistic != nullptr;
+  const float shift = logistic ? extra.logistic[head] : 0.f;
+  if (logistic) {
+    running_max = 0.f;
+    running_sum = extra.logistic_norm;
+  }
   float acc[AR_MAX_DIMS] = {0.f, 0.f, 0.f, 0.f};
 
   for (int k0 = first_key; k0 < end_key; k0 += 64) {
@@ -63,13 +69,18 @@ __global__ __launch_bounds__(64) void attention_rowwise_kernel(
         if (extra.softcap > 0.f) score = capped_score(score, extra.softcap);
       }
     }
-    const float chunk_max = wave_max(score);
-    const float new_max = fmaxf(running_max, chunk_max);
-    // new_max is -inf only if no key has been visible so far; then nothing accumulates.
-    const float correction = (new_max == -INFINITY) ? 1.f : expf(running_max - new_max);
-    const float p = (score == -INFINITY) ? 0.f : expf(score - new_max);
-    running_sum = running_sum * correction + wave_sum(p);
-    running_max = new_max;
+    float correction = 1.f, p;
+    if (logistic) {
+      p = (score == -INFINITY) ? 0.f : 1.0f / (1.0f + expf(-(score + shift)));
+    } else {
+      const float chunk_max = wave_max(score);
+      const float new_max = fmaxf(running_max, chunk_max);
+      // new_max is -inf only if no key has been visible so far; then nothing accumulates.
+      correction = (new_max == -INFINITY) ? 1.f : expf(running_max - new_max);
+      p = (score == -INFINITY) ? 0.f : expf(score - new_max);
+      running_sum = running_sum * correction + wave_sum(p);
+      running_max = new_max;
+    }
     __syncthreads();
     prob[lane] = p;
     key_base[lane] = base;
@@ -106,7 +117,7 @@ extern "C" int ps_attention_rowwise(const void* q, int64_t q_stride, const void*
                                     int kv_heads,
                                     int head_dim, int page_size, int num_pages, float scale,
                                     int window, const float* sink, const float* gate,
-                                    int64_t gate_ld, float softcap, int dtype, void* stream) {
+                                    int64_t gate_ld, float softcap, const float* logistic, float logistic_norm, int dtype, void* stream) {
   PS_REQUIRE(tokens >= 0 && heads > 0 && kv_heads > 0 && page_size > 0 && num_pages > 0 &&
                  table_width > 0,
              "ps_attention_rowwise: bad sizes");
@@ -118,7 +129,7 @@ extern "C" int ps_attention_rowwise(const void* q, int64_t q_stride, const void*
   PS_REQUIRE(dtype == PS_F32 || dtype == PS_BF16, "ps_attention_rowwise: unknown dtype %d", dtype);
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-  const AttnExtras extra = {sink, gate, gate_ld, softcap};
+  const AttnExtras extra = {sink, gate, gate_ld, softcap, logistic, logistic_norm};
   dim3 grid(tokens, heads);
   if (dtype == PS_F32)
     hipLaunchKernelGGL(attention_rowwise_kernel<float>, grid, dim3(64), 0, s, (const float*)q,

@@ -83,6 +83,7 @@ __global__ __launch_bounds__(256) void attention_tiled_f32_kernel(
     // (a sink is a score without key or value: it starts the denominator)
     run_max[i] = extra.sink ? extra.sink[head] : -INFINITY;
     run_sum[i] = extra.sink ? 1.f : 0.f;
+    if (extra.logistic != nullptr) run_sum[i] = extra.logistic_norm;
 #pragma unroll
     for (int v = 0; v < DV; ++v) acc[v][i] = make_float4(0.f, 0.f, 0.f, 0.f);
   }
@@ -153,6 +154,14 @@ __global__ __launch_bounds__(256) void attention_tiled_f32_kernel(
         s[i][j] = visible ? score : -INFINITY;
         tile_max = fmaxf(tile_max, s[i][j]);
       }
+      if (extra.logistic != nullptr) {
+        const float shift = extra.logistic[head];
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          s_p[(4 * ty + i) * AF_P_STRIDE + tx + 16 * j] =
+              s[i][j] == -INFINITY ? 0.f : 1.0f / (1.0f + expf(-(s[i][j] + shift)));
+        continue;
+      }
       // the 16 threads of a row are 16 neighbouring lanes of one wave
 #pragma unroll
       for (int mask = 8; mask >= 1; mask >>= 1) tile_max = fmaxf(tile_max, __shfl_xor(tile_max, mask, 16));
@@ -213,7 +222,7 @@ __global__ __launch_bounds__(256) void attention_tiled_f32_kernel(
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     if (q_pos[i] < 0) continue;
-    const float inverse = (run_sum[i] > 0.f ? 1.f / run_sum[i] : 0.f) *
+    const float inverse = (run_sum[i] != 0.f ? 1.f / run_sum[i] : 0.f) *
                           gate_factor(extra, tok0 + q0 + 4 * ty + i, head);
     float* row = out + (int64_t)(tok0 + q0 + 4 * ty + i) * out_stride + (int64_t)head * head_dim;
 #pragma unroll
@@ -240,7 +249,8 @@ extern "C" int ps_attention_tiled_f32(const void* q, int64_t q_stride, const voi
                                       int table_width, int heads, int kv_heads, int head_dim,
                                       int page_size, int num_pages, float scale, int window,
                                       const float* sink, const float* gate, int64_t gate_ld,
-                                      float softcap, void* stream) {
+                                      float softcap, const float* logistic, float logistic_norm,
+                                      void* stream) {
   PS_REQUIRE(tiles >= 0 && heads > 0 && kv_heads > 0 && page_size > 0 && num_pages > 0 &&
                  table_width > 0,
              "ps_attention_tiled_f32: bad sizes");
@@ -258,7 +268,7 @@ extern "C" int ps_attention_tiled_f32(const void* q, int64_t q_stride, const voi
   PS_REQUIRE(blocks < ((int64_t)1 << 31), "ps_attention_tiled_f32: too many blocks");
   if (blocks == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
-  const AttnExtras extra = {sink, gate, gate_ld, softcap};
+  const AttnExtras extra = {sink, gate, gate_ld, softcap, logistic, logistic_norm};
 #define PS_LAUNCH_AF(DV)                                                                          \
   hipLaunchKernelGGL(attention_tiled_f32_kernel<DV>, dim3((unsigned)blocks), dim3(256), 0, s,     \
                      (const float*)q, q_stride, (const float*)k_pool, (const float*)v_pool,       \

@@ -281,13 +281,32 @@ __host__ __device__ inline int first_visible_key(int pos, int window) {
 // What an attention kernel may be given beside its operands: a sink (one float per head whose
 // exponential joins the softmax's denominator; null: none), a gate (the output of token t
 // and head h is multiplied by sigmoid(gate[t * gate_ld + h]); null: none) and a cap on the
-// scaled scores (s <- cap * tanh(s / cap) before the softmax; 0: none).
+// scaled scores (s <- cap * tanh(s / cap) before the softmax; 0: none).  `logistic` (a float per
+// head; null: a softmax as ever) replaces the softmax: a visible key's weight is sigmoid(s +
+// logistic[head]) and the weighted values are divided by logistic_norm instead of by a sum over the
+// keys.  Such a state keeps a maximum of 0 everywhere and has logistic_norm as its sum in exactly one
+// place (the first range, wave or lane group), so that whatever merges softmax states merges these.
 struct AttnExtras {
   const float* sink;
   const float* gate;
   long long gate_ld;
   float softcap;
+  const float* logistic;
+  float logistic_norm;
 };
+
+// sigmoid(x / log2(e)) of a score kept in units of log 2: exact, and from the hardware's exponential
+// and reciprocal (for weights that are rounded to bfloat16)
+__device__ inline float logistic_weight(float s_log2) { return 1.0f / (1.0f + exp2f(-s_log2)); }
+__device__ inline float logistic_weight_fast(float s_log2) {
+  return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-s_log2));
+}
+template <typename T>
+__device__ inline float logistic_weight_as(float s_log2);
+template <>
+__device__ inline float logistic_weight_as<float>(float s) { return logistic_weight(s); }
+template <>
+__device__ inline float logistic_weight_as<bf16_t>(float s) { return logistic_weight_fast(s); }
 
 // c * tanh(s / c), with the score and the cap in the same units (a kernel that keeps scores
 // unscaled, or in units of log 2, hands over the cap divided or multiplied accordingly).

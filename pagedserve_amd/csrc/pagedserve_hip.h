@@ -122,13 +122,15 @@ int ps_kv_write(const void* k, const void* v, int64_t stride, void* k_pool, void
 // gate_ld apart: the output of token t and head h is multiplied by sigmoid(gate[t * gate_ld + h]);
 // the same in the attention kernels below (ps_attention_decode_partial leaves the gate to
 // whoever merges its records).  softcap: 0, or c > 0: a scaled score s enters the softmax as
-// c * tanh(s / c).
+// c * tanh(s / c).  logistic: null, or one float per head: no softmax then, a visible key's weight is
+// sigmoid(s + logistic[head]) and the weighted values are divided by logistic_norm (not with a sink).
 int ps_attention_rowwise(const void* q, int64_t q_stride, const void* k_pool, const void* v_pool,
                          void* out, int64_t out_stride, const int* tok_list, const int* tok_item,
                          const int* tok_pos, const int* tables, int table_width, int tokens,
                          int heads, int kv_heads, int head_dim, int page_size, int num_pages,
                          float scale, int window, const float* sink, const float* gate,
-                         int64_t gate_ld, float softcap, int dtype, void* stream);
+                         int64_t gate_ld, float softcap, const float* logistic,
+                         float logistic_norm, int dtype, void* stream);
 
 // The same result in true 32-bit for the items of several tokens (prompt portions), a block
 // of four waves per (tile of ps_attention_tiled_f32_tile() queries, head): float pools, float
@@ -142,7 +144,8 @@ int ps_attention_tiled_f32(const void* q, int64_t q_stride, const void* k_pool, 
                            int tiles, const int* cu_tokens, const int* kv_lens, const int* tables,
                            int table_width, int heads, int kv_heads, int head_dim, int page_size,
                            int num_pages, float scale, int window, const float* sink, const float* gate,
-                           int64_t gate_ld, float softcap, void* stream);
+                           int64_t gate_ld, float softcap, const float* logistic,
+                         float logistic_norm, void* stream);
 
 // The same result for single queries, with each token's keys cut into `splits` ranges that
 // run as separate blocks of `waves` (4 or 16) waves; `partial` is scratch of
@@ -156,7 +159,8 @@ int ps_attention_decode(const void* q, int64_t q_stride, const void* k_pool, con
                         const int* tables, int table_width, int count, int heads, int kv_heads,
                         int head_dim, int page_size, int num_pages, float scale, int window,
                         int splits, int waves, const float* sink, const float* gate, int64_t gate_ld,
-                        float softcap, int dtype, void* stream);
+                        float softcap, const float* logistic,
+                         float logistic_norm, int dtype, void* stream);
 
 // The same result for bfloat16 layers whose query heads share key/value heads in large groups
 // (one cached row that all heads read): a block takes a token's heads of one group (up to 16)
@@ -168,7 +172,8 @@ int ps_attention_decode_shared(const void* q, int64_t q_stride, const void* k_po
                                const int* tok_list, const int* tok_item, const int* tok_pos,
                                const int* tables, int table_width, int count, int heads, int kv_heads,
                                int head_dim, int page_size, int num_pages, float scale, int window,
-                               int splits, const float* gate, int64_t gate_ld, float softcap,
+                               int splits, const float* gate, int64_t gate_ld, float softcap, const float* logistic,
+                         float logistic_norm,
                                void* stream);
 
 // Only the records of ps_attention_decode: (unnormalised sum of values [head_dim], maximum in
@@ -180,7 +185,8 @@ int ps_attention_decode_partial(const void* q, int64_t q_stride, const void* k_p
                                 const int* tables, int table_width, int count, int heads,
                                 int kv_heads, int head_dim, int page_size, int num_pages,
                                 float scale, int window, int splits, int waves, const float* sink,
-                                float softcap, int dtype, void* stream);
+                                float softcap, const float* logistic,
+                         float logistic_norm, int dtype, void* stream);
 
 // The merge of those records inside the output projection, for up to 16 tokens and head sizes
 // that are multiples of 64 (bfloat16 weights in their packed copy, n output columns,
@@ -226,7 +232,8 @@ int ps_attention_prefill(const void* q, int64_t q_stride, const void* k_pool, co
                          int tiles, const int* cu_tokens, const int* kv_lens, const int* tables,
                          int table_width, int heads, int kv_heads, int head_dim, int page_size,
                          int num_pages, float scale, int window, int max_kv_len, int query_tile,
-                         const float* sink, const float* gate, int64_t gate_ld, float softcap,
+                         const float* sink, const float* gate, int64_t gate_ld, float softcap, const float* logistic,
+                         float logistic_norm,
                          int dtype, void* stream);
 
 // Both of the above in one launch, for a step that has items of one token (tok_list lists the
@@ -242,7 +249,8 @@ int ps_attention_mixed(const void* q, int64_t q_stride, const void* k_pool, cons
                        const int* tile_q0, int tiles, const int* cu_tokens, const int* kv_lens,
                        const int* tables, int table_width, int heads, int kv_heads, int head_dim,
                        int page_size, int num_pages, float scale, int window, const float* sink,
-                       const float* gate, int64_t gate_ld, float softcap, int dtype, void* stream);
+                       const float* gate, int64_t gate_ld, float softcap, const float* logistic,
+                         float logistic_norm, int dtype, void* stream);
 
 // The constants of that kernel that a caller builds its index arrays by: queries per tile (of
 // the two sizes), and the widest block table (entries per item) that it takes.
@@ -398,7 +406,8 @@ int ps_stream_step(float* h, const float* y, float factor, const float* column_s
                    int out_dtype, void* stream);
 // out[t, c] = unit(gu[t * ld + c], gu[t * ld + inner + c]) (* row_scale[t], unless null) with
 // unit(g, u) = g' sigmoid(slope g') (u' + shift), g' = min(g, limit), u' = clamp(u, -limit, limit):
-// silu(g) * u for an infinite limit, slope 1 and shift 0.  activation 1: gelu_tanh(g) * u.
+// silu(g) * u for an infinite limit, slope 1 and shift 0.  activation 1: gelu_tanh(g) * u; 2:
+// max(g, 0) * u.
 int ps_silu_gate(const float* gu, int64_t ld, void* out, int64_t out_ld, int tokens, int inner,
                  int activation, float limit, float slope, float shift, const float* row_scale,
                  int dtype, void* stream);
@@ -479,6 +488,59 @@ int ps_differential_merge(const float* partial, int64_t partial_floats, const in
                           const float* lambda, float factor, float eps, const float* gate,
                           int64_t gate_ld, void* out, int64_t out_ld, int heads, int head_dim,
                           int value_dim, int splits, int map_major, int dtype, void* stream);
+
+// ---- sublayers between two layer norms, a gate on their result -------------------------------
+// With LN(x) = (x - mean) / sqrt(mean((x - mean)^2) + eps) * scale + shift over the row, per token:
+//   y != null:       h += LN(sigmoid(gate + gate_bias) * y; gamma, beta), y <- 0   (gate rows gate_ld apart)
+//   gamma2 != null:  normed = LN(h; gamma2, beta2) in the engine's type
+// width up to 16384.
+int ps_gated_norm_step(float* h, float* y, const float* gate, int64_t gate_ld, const float* gate_bias,
+                       const float* gamma, const float* beta, const float* gamma2, const float* beta2,
+                       float eps, void* normed, int tokens, int width, int out_dtype, void* stream);
+
+// ---- recurrences whose state is a matrix per head (matrix_state.hip) --------------------------
+// A slot's state is a run of slot_stride floats: per head and value column the key_dim numbers of
+// S[:, column], then what else the mixer keeps (`history`: the last taps - 1 raw inputs of the
+// convolution, [taps - 1][channels], oldest first; `maxima`: a running maximum per head).
+//
+// What the recurrence is fed with.  out[t, c] = silu(bias[c] + sum_j w[c, j] u[t - taps + 1 + j, c]) of
+// the raw inputs u = proj[:, col ...] of the item, earlier ones from its slot; the first unit_heads
+// runs of `head` channels become unit vectors, x / sqrt(sum(x^2) + 1e-6), the first scale_heads of
+// them times q_scale.  rule 0: dt = softplus(proj[t, take_col + h] + z_bias[h]), take = dt, decay =
+// -exp(a_log[h]) dt; rule 1: take = sigmoid(proj[t, take_col + h]), decay[t, h * per_head + r] =
+// exp(-exp(a_log[h]) softplus(z[t, ..] + z_bias[..])).
+int ps_state_prepare(const float* proj, int64_t ld, int col, int channels, int taps, const float* w,
+                     const float* bias, const float* state, int64_t slot_stride, int64_t history,
+                     float* out, int unit_heads, int head, int scale_heads, float q_scale, int rule,
+                     int heads, int per_head, const float* z, int64_t z_ld, const float* z_bias,
+                     const float* a_log, int take_col, float* decay, float* take, const int* tok_item,
+                     const int* cu_tokens, const int* slots, int tokens, void* stream);
+// Exponential gates with a running maximum m (kept in the slot): i = cap tanh((proj[t, i_col + h] +
+// i_bias[h]) / cap), f = log sigmoid(cap tanh(..f..)), m_t = max(f + m, i); log_decay = f + m_(t-1) -
+// m_t, take = exp(i - m_t), floor_out = exp(-m_t), all [tokens, heads].
+int ps_memory_gates(const float* proj, int64_t ld, int i_col, int f_col, const float* i_bias,
+                    const float* f_bias, float cap, float* state, int64_t slot_stride, int64_t maxima,
+                    float* log_decay, float* take, float* floor_out, const int* cu_tokens,
+                    const int* slots, int items, int heads, void* stream);
+// The recurrence over the items of a step, token after token; head h reads key/query head h /
+// key_share.  rule 0: S = e^decay[t, h] S + take[t, h] k v^T; rule 1: S = diag(decay[t, h]) S, then S +=
+// take[t, h] k (v - S^T k)^T.  out[t, h] = S^T (q_scale q).  ones: one more column, whose value is one
+// for every token (the keys' own sum).  longest 1: no item brings more tokens (launch shape only).
+// raw: the convolution's raw inputs, whose last ones are kept (channels 0: none).
+int ps_state_scan(const float* q, int64_t q_ld, const float* k, int64_t k_ld, const float* v,
+                  int64_t v_ld, const float* decay, const float* take, float* state,
+                  int64_t slot_stride, float* out, const int* cu_tokens, const int* slots, int items,
+                  int rule, int heads, int key_share, int key_dim, int value_dim, int ones,
+                  float q_scale, int longest, const float* raw, int64_t raw_ld, int channels, int taps,
+                  int64_t history, void* stream);
+// out[t, c] from the recurrence's o [tokens, heads, value_dim (+ 1)]: x = o (+ skip[h] u[t, c]); ones: x /
+// (max(|key sum|, floor_in[t, h]) + 1e-6); x *= silu(before[t, c]); x / rms over each of `groups` equal
+// runs of columns (eps inside the root) * weight[c % weight_count]; x *= sigmoid(behind[t, c]).
+int ps_state_output(const float* o, int heads, int value_dim, int ones, const float* floor_in,
+                    const float* skip, const float* u, int64_t u_ld, const float* before,
+                    int64_t before_ld, const float* weight, int weight_count, float eps, int groups,
+                    const float* behind, int64_t behind_ld, void* out, int64_t out_ld, int tokens,
+                    int dtype, void* stream);
 
 #ifdef __cplusplus
 }

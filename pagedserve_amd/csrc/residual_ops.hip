@@ -77,9 +77,9 @@ __global__ __launch_bounds__(256) void stream_step_kernel(
   }
 }
 
-// out[t, c] = unit(gu[t, c], gu[t, inner + c]) (common.h: GateForm), or (GELU) gelu_tanh(gu[t, c]) *
-// gu[t, inner + c]; times row_scale[t] where that is given
-template <typename T, bool GELU>
+// out[t, c] = unit(gu[t, c], gu[t, inner + c]) (common.h: GateForm), or act(gu[t, c]) * gu[t, inner + c]
+// with ACT 1: gelu_tanh, 2: relu; times row_scale[t] where that is given
+template <typename T, int ACT>
 __global__ __launch_bounds__(256) void silu_gate_kernel(const float* __restrict__ gu, int64_t ld,
                                                         T* __restrict__ out, int64_t out_ld,
                                                         int inner, const GateForm form,
@@ -89,7 +89,7 @@ __global__ __launch_bounds__(256) void silu_gate_kernel(const float* __restrict_
   if (c >= inner) return;
   const float g = gu[t * ld + c];
   const float u = gu[t * ld + inner + c];
-  float v = GELU ? gelu_tanh_f(g) * u : gated_unit(g, u, form);
+  float v = ACT == 1 ? gelu_tanh_f(g) * u : (ACT == 2 ? fmaxf(g, 0.f) * u : gated_unit(g, u, form));
   if (row_scale != nullptr) v *= row_scale[t];
   out[t * out_ld + c] = from_float<T>(v);
 }
@@ -159,17 +159,21 @@ extern "C" int ps_silu_gate(const float* gu, int64_t ld, void* out, int64_t out_
   if (tokens == 0) return 0;
   hipStream_t s = (hipStream_t)stream;
   const dim3 grid(tokens, (inner + 255) / 256);
-  PS_REQUIRE(activation == 0 || activation == 1, "ps_silu_gate: activation %d (0: silu, 1: gelu_tanh)", activation);
+  PS_REQUIRE(activation >= 0 && activation <= 2, "ps_silu_gate: activation %d (0: silu, 1: gelu_tanh, 2: relu)", activation);
   PS_REQUIRE(limit > 0.f, "ps_silu_gate: the limit must be positive");
   const GateForm form = {limit, slope, shift};
-  if (dtype == PS_F32 && activation)
-    hipLaunchKernelGGL((silu_gate_kernel<float, true>), grid, dim3(256), 0, s, gu, ld, (float*)out, out_ld, inner, form, row_scale);
-  else if (dtype == PS_F32)
-    hipLaunchKernelGGL((silu_gate_kernel<float, false>), grid, dim3(256), 0, s, gu, ld, (float*)out, out_ld, inner, form, row_scale);
-  else if (activation)
-    hipLaunchKernelGGL((silu_gate_kernel<bf16_t, true>), grid, dim3(256), 0, s, gu, ld, (bf16_t*)out, out_ld, inner, form, row_scale);
-  else
-    hipLaunchKernelGGL((silu_gate_kernel<bf16_t, false>), grid, dim3(256), 0, s, gu, ld, (bf16_t*)out, out_ld, inner, form, row_scale);
+#define PS_LAUNCH_SG(T, ACT) \
+  hipLaunchKernelGGL((silu_gate_kernel<T, ACT>), grid, dim3(256), 0, s, gu, ld, (T*)out, out_ld, inner, form, row_scale)
+#define PS_LAUNCH_SG_T(T)                          \
+  do {                                             \
+    if (activation == 1) PS_LAUNCH_SG(T, 1);       \
+    else if (activation == 2) PS_LAUNCH_SG(T, 2);  \
+    else PS_LAUNCH_SG(T, 0);                       \
+  } while (0)
+  if (dtype == PS_F32) PS_LAUNCH_SG_T(float);
+  else PS_LAUNCH_SG_T(bf16_t);
+#undef PS_LAUNCH_SG_T
+#undef PS_LAUNCH_SG
   PS_CHECK_LAUNCH("ps_silu_gate");
   return 0;
 }
@@ -190,5 +194,114 @@ extern "C" int ps_pair_norm_mix(float* a, float* b, const float* wa, const float
   hipLaunchKernelGGL(pair_norm_mix_kernel, dim3(tokens), dim3(256), 0, (hipStream_t)stream, a, b, wa,
                      wb, eps, share, y, width);
   PS_CHECK_LAUNCH("ps_pair_norm_mix");
+  return 0;
+}
+
+// Sublayers between two layer norms, with a gate on their result.  Per token, one pass:
+//   h <- h + LN(sigmoid(gate + gate_bias) * y; gamma, beta);   y <- 0
+//   normed <- LN(h; gamma2, beta2)
+// with LN(x) = (x - mean) / sqrt(mean((x - mean)^2) + eps) * gamma + beta; either half is optional.  A
+// block holds its row in registers, HELD numbers to a thread.
+template <typename T, int HELD>
+__global__ __launch_bounds__(1024) void gated_norm_step_kernel(
+    float* __restrict__ h, float* __restrict__ y, const float* __restrict__ gate, int64_t gate_ld,
+    const float* __restrict__ gate_bias, const float* __restrict__ gamma, const float* __restrict__ beta,
+    const float* __restrict__ gamma2, const float* __restrict__ beta2, float eps, T* __restrict__ normed,
+    int width) {
+  __shared__ float scratch[16];
+  const int64_t t = blockIdx.x;
+  float* row = h + t * width;
+  float x[HELD], v[HELD], scale[HELD], shift[HELD], scale2[HELD], shift2[HELD];
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < HELD; ++i) {
+    const int d = threadIdx.x + blockDim.x * i;
+    x[i] = v[i] = scale[i] = shift[i] = scale2[i] = shift2[i] = 0.f;
+    if (d < width) {
+      x[i] = row[d];
+      if (gamma2 != nullptr) {
+        scale2[i] = gamma2[d];
+        shift2[i] = beta2[d];
+      }
+      if (y != nullptr) {
+        scale[i] = gamma[d];
+        shift[i] = beta[d];
+        v[i] = y[t * width + d] / (1.0f + expf(-(gate[t * gate_ld + d] + gate_bias[d])));
+        y[t * width + d] = 0.f;
+      }
+    }
+    sum += v[i];
+  }
+  if (y != nullptr) {
+    const float mean = block_sum(sum, scratch) / (float)width;
+    float squares = 0.f;
+#pragma unroll
+    for (int i = 0; i < HELD; ++i) {
+      const int d = threadIdx.x + blockDim.x * i;
+      v[i] = d < width ? v[i] - mean : 0.f;
+      squares = fmaf(v[i], v[i], squares);
+    }
+    const float inv = 1.0f / sqrtf(block_sum(squares, scratch) / (float)width + eps);
+#pragma unroll
+    for (int i = 0; i < HELD; ++i) {
+      const int d = threadIdx.x + blockDim.x * i;
+      x[i] += fmaf(v[i] * inv, scale[i], shift[i]);
+      if (d < width) row[d] = x[i];
+    }
+  }
+  if (gamma2 == nullptr) return;
+  sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < HELD; ++i) sum += x[i];
+  const float mean = block_sum(sum, scratch) / (float)width;
+  float squares = 0.f;
+#pragma unroll
+  for (int i = 0; i < HELD; ++i) {
+    const int d = threadIdx.x + blockDim.x * i;
+    x[i] = d < width ? x[i] - mean : 0.f;
+    squares = fmaf(x[i], x[i], squares);
+  }
+  const float inv = 1.0f / sqrtf(block_sum(squares, scratch) / (float)width + eps);
+#pragma unroll
+  for (int i = 0; i < HELD; ++i) {
+    const int d = threadIdx.x + blockDim.x * i;
+    if (d < width) normed[t * width + d] = from_float<T>(fmaf(x[i] * inv, scale2[i], shift2[i]));
+  }
+}
+
+extern "C" int ps_gated_norm_step(float* h, float* y, const float* gate, int64_t gate_ld,
+                                  const float* gate_bias, const float* gamma, const float* beta,
+                                  const float* gamma2, const float* beta2, float eps, void* normed,
+                                  int tokens, int width, int out_dtype, void* stream) {
+  PS_REQUIRE(tokens >= 0 && width > 0 && width <= 16384 && eps > 0.f,
+             "ps_gated_norm_step: bad sizes (width %d, at most 16384)", width);
+  PS_REQUIRE(y == nullptr || (gate != nullptr && gate_bias != nullptr && gamma != nullptr && beta != nullptr && gate_ld >= width),
+             "ps_gated_norm_step: a result needs its gate and its norm");
+  PS_REQUIRE(gamma2 == nullptr || (beta2 != nullptr && normed != nullptr),
+             "ps_gated_norm_step: a second norm needs its shift and an output");
+  PS_REQUIRE(out_dtype == PS_F32 || out_dtype == PS_BF16, "ps_gated_norm_step: unknown dtype %d", out_dtype);
+  if (tokens == 0) return 0;
+  hipStream_t s = (hipStream_t)stream;
+  // few rows wait for their trips to memory: a thread per column as far as a block has them; many
+  // rows fill the chip with blocks of four waves
+  int threads = width >= 1024 ? 1024 : (width + 63) / 64 * 64;
+  if (tokens > 256 && threads > 256 && width <= 256 * 16) threads = 256;
+  const int held = (width + threads - 1) / threads;
+#define PS_LAUNCH_GNS(T, HELD)                                                                          \
+  hipLaunchKernelGGL((gated_norm_step_kernel<T, HELD>), dim3(tokens), dim3(threads), 0, s, h, y, gate,  \
+                     gate_ld, gate_bias, gamma, beta, gamma2, beta2, eps, (T*)normed, width)
+#define PS_LAUNCH_GNS_T(T)                       \
+  do {                                           \
+    if (held <= 1) PS_LAUNCH_GNS(T, 1);          \
+    else if (held <= 2) PS_LAUNCH_GNS(T, 2);     \
+    else if (held <= 4) PS_LAUNCH_GNS(T, 4);     \
+    else if (held <= 8) PS_LAUNCH_GNS(T, 8);     \
+    else PS_LAUNCH_GNS(T, 16);                   \
+  } while (0)
+  if (out_dtype == PS_F32) PS_LAUNCH_GNS_T(float);
+  else PS_LAUNCH_GNS_T(bf16_t);
+#undef PS_LAUNCH_GNS_T
+#undef PS_LAUNCH_GNS
+  PS_CHECK_LAUNCH("ps_gated_norm_step");
   return 0;
 }

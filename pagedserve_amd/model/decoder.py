@@ -232,7 +232,7 @@ class DecoderModel:
             # a block may leave its last write to the block that follows, if that one takes it
             if hasattr(block, "finish"):
                 follower = self.blocks[schedule[index + 1].block] if index + 1 < len(schedule) else None
-                if not getattr(follower, "takes_stream_write", False):
+                if getattr(follower, "takes_stream_write", False) != block.takes_stream_write:
                     block.finish(h, ctx)
         wanted = logit_rows.numel()
         if wanted == 0:

@@ -31,7 +31,7 @@ _SIGNATURES = {
                     c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p],
     "ps_attention_rowwise": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                              c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
-                             c_int, c_float, c_int, c_void_p, c_void_p, c_int64, c_float, c_int,
+                             c_int, c_float, c_int, c_void_p, c_void_p, c_int64, c_float, c_void_p, c_float, c_int,
                              c_void_p],
     "ps_hyper_step": [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_float, c_void_p,
                       c_void_p, c_int, c_int, c_int, c_int, c_void_p],
@@ -98,29 +98,43 @@ _SIGNATURES = {
     "ps_attention_decode": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                             c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
                             c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_void_p, c_void_p,
-                            c_int64, c_float, c_int, c_void_p],
+                            c_int64, c_float, c_void_p, c_float, c_int, c_void_p],
     "ps_attention_decode_shared": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                                    c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
                                    c_int, c_int, c_int, c_int, c_float, c_int, c_int, c_void_p, c_int64,
-                                   c_float, c_void_p],
+                                   c_float, c_void_p, c_float, c_void_p],
     "ps_attention_decode_partial": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                                     c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
-                                    c_int, c_int, c_float, c_int, c_int, c_int, c_void_p, c_float, c_int,
+                                    c_int, c_int, c_float, c_int, c_int, c_int, c_void_p, c_float, c_void_p, c_float, c_int,
                                     c_void_p],
     "ps_attention_merge_linear": [c_void_p, c_int64, c_void_p, c_int, c_int, c_int, c_int, c_void_p,
                                   c_void_p, c_void_p, c_int64, c_int, c_int, c_void_p],
     "ps_attention_tiled_f32": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                                c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
-                               c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_int64, c_float,
+                               c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p, c_int64, c_float, c_void_p, c_float,
                                c_void_p],
     "ps_attention_prefill": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p,
                              c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int,
                              c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_void_p, c_void_p, c_int64,
-                             c_float, c_int, c_void_p],
+                             c_float, c_void_p, c_float, c_int, c_void_p],
     "ps_attention_mixed": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_int,
                            c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
                            c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_void_p, c_void_p,
-                           c_int64, c_float, c_int, c_void_p],
+                           c_int64, c_float, c_void_p, c_float, c_int, c_void_p],
+    "ps_gated_norm_step": [c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
+                           c_void_p, c_float, c_void_p, c_int, c_int, c_int, c_void_p],
+    "ps_state_prepare": [c_void_p, c_int64, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int64, c_int64,
+                         c_void_p, c_int, c_int, c_int, c_float, c_int, c_int, c_int, c_void_p, c_int64,
+                         c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                         c_void_p],
+    "ps_memory_gates": [c_void_p, c_int64, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_int64, c_int64,
+                        c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
+    "ps_state_scan": [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p,
+                      c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
+                      c_float, c_int, c_void_p, c_int64, c_int, c_int, c_int64, c_void_p],
+    "ps_state_output": [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_int64,
+                        c_void_p, c_int, c_float, c_int, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int,
+                        c_void_p],
     "ps_sample": [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int, c_void_p],
 }
 
@@ -739,8 +753,26 @@ def _check_cap(softcap):
     return softcap
 
 
+def _check_logistic(logistic, heads):
+    """``logistic = (shift, norm)``: no softmax; a visible key weighs ``sigmoid(score + shift[head])``
+    and the weighted values are divided by ``norm``.  (address, norm), or (0, 1) for None."""
+    if logistic is None:
+        return 0, 1.0
+    shift, norm = logistic
+    _check(shift, "logistic shift", torch.float32, 1)
+    if shift.numel() != heads or not shift.is_contiguous():
+        raise KernelError(f"attention: logistic weights need one float per head ({heads})")
+    if float(norm) == 0.0 or float(norm) != float(norm):
+        raise KernelError(f"attention: the norm of logistic weights must not be {norm}")
+    return shift.data_ptr(), float(norm)
+
+
+def _logistic_key(logistic):
+    return (0, 1.0) if logistic is None else (logistic[0].data_ptr(), float(logistic[1]))
+
+
 def attention_rowwise(q, k_pool, v_pool, out, tok_item, tok_pos, tables, heads, scale, window=0,
-                      tok_list=None, sink=None, gate=None, softcap=0.0):
+                      tok_list=None, sink=None, gate=None, softcap=0.0, logistic=None):
     """out[t, h] = softmax(q[t, h] . K * scale) V over the cached keys of t's request, for the
     tokens in ``tok_list`` (all when it is None).  ``sink``: one float per head whose
     exponential joins the denominator (a score that has no key and no value)."""
@@ -750,7 +782,7 @@ def attention_rowwise(q, k_pool, v_pool, out, tok_item, tok_pos, tables, heads, 
     _call("ps_attention_rowwise", q.data_ptr(), q_stride, k_pool.data_ptr(), v_pool.data_ptr(),
           out.data_ptr(), out_stride, _ptr(tok_list), tok_item.data_ptr(), tok_pos.data_ptr(),
           tables.data_ptr(), tables.shape[1], count, heads, kv_heads, head_dim, page_size, pages,
-          float(scale), int(window), sink, *_check_gate(gate, q.shape[0], heads), _check_cap(softcap),
+          float(scale), int(window), sink, *_check_gate(gate, q.shape[0], heads), _check_cap(softcap), *_check_logistic(logistic, heads),
           dtype_code(q.dtype), _stream())
     return out
 
@@ -763,7 +795,7 @@ def decode_keys_per_block(head_dim: int, waves: int = 4) -> int:
 
 
 def attention_decode(q, k_pool, v_pool, out, tok_item, tok_pos, tables, heads, scale, splits,
-                     partial=None, window=0, tok_list=None, waves=4, sink=None, gate=None, softcap=0.0):
+                     partial=None, window=0, tok_list=None, waves=4, sink=None, gate=None, softcap=0.0, logistic=None):
     """The same result as ``attention_rowwise`` by the split-KV kernel; ``partial`` is float
     scratch of ``count * heads * splits * (head_dim + 2)`` values when ``splits > 1``.
     ``tok_item=None`` says that token t is item t (row t of ``tables``), as in a step of single
@@ -781,7 +813,7 @@ def attention_decode(q, k_pool, v_pool, out, tok_item, tok_pos, tables, heads, s
           _ptr(tok_list), _ptr(tok_item), tok_pos.data_ptr(), tables.data_ptr(),
           tables.shape[1], count, heads, kv_heads, head_dim, page_size, pages, float(scale),
           int(window), int(splits), int(waves), _check_sink(sink, heads),
-          *_check_gate(gate, q.shape[0], heads), _check_cap(softcap), dtype_code(q.dtype), _stream())
+          *_check_gate(gate, q.shape[0], heads), _check_cap(softcap), *_check_logistic(logistic, heads), dtype_code(q.dtype), _stream())
     return out
 
 
@@ -798,7 +830,7 @@ def shared_decode_supported(dtype, heads, kv_heads, head_dim, sink=None) -> bool
 
 
 def attention_decode_shared(q, k_pool, v_pool, out, tok_item, tok_pos, tables, heads, scale, splits, partial,
-                            window=0, tok_list=None, gate=None, softcap=0.0):
+                            window=0, tok_list=None, gate=None, softcap=0.0, logistic=None):
     """``attention_decode`` by blocks that load a tile of keys once for all heads of a group (up
     to 16) and work on the matrix cores; ``v_pool`` may be ``k_pool``.  ``partial``: float scratch of
     ``count * heads * splits * (head_dim + 2)`` values, also with one range."""
@@ -816,7 +848,7 @@ def attention_decode_shared(q, k_pool, v_pool, out, tok_item, tok_pos, tables, h
           _ptr(out), out_stride, partial.data_ptr(), partial.numel(), _ptr(tok_list), _ptr(tok_item),
           tok_pos.data_ptr(), tables.data_ptr(), tables.shape[1], count, heads, kv_heads, head_dim,
           page_size, pages, float(scale), int(window), int(splits), *_check_gate(gate, q.shape[0], heads),
-          _check_cap(softcap), _stream())
+          _check_cap(softcap), *_check_logistic(logistic, heads), _stream())
     return out
 
 
@@ -835,7 +867,7 @@ def merge_linear_supported(dtype, tokens, head_dim, packed) -> bool:
 
 
 def attention_decode_partial(q, k_pool, v_pool, partial, tok_item, tok_pos, tables, heads, scale, splits,
-                             window=0, tok_list=None, waves=4, sink=None, softcap=0.0):
+                             window=0, tok_list=None, waves=4, sink=None, softcap=0.0, logistic=None):
     """The per-range records of decode attention only (``partial``: float scratch of
     ``count * heads * splits * (head_dim + 2)`` values); ``attention_merge_linear`` merges them.
     ``tok_item=None``: token t is item t, as for ``attention_decode``."""
@@ -859,7 +891,7 @@ def attention_decode_partial(q, k_pool, v_pool, partial, tok_item, tok_pos, tabl
           partial.data_ptr(), partial.numel(), _ptr(tok_list), _ptr(tok_item), tok_pos.data_ptr(),
           tables.data_ptr(), tables.shape[1], count, heads, kv_heads, head_dim, page_size, pages,
           float(scale), int(window), int(splits), int(waves), _check_sink(sink, heads),
-          _check_cap(softcap), dtype_code(q.dtype), _stream())
+          _check_cap(softcap), *_check_logistic(logistic, heads), dtype_code(q.dtype), _stream())
     return count
 
 
@@ -965,7 +997,7 @@ def prefill_large_tile_pays(heads, head_dim, large_tiles, max_kv_len=0) -> bool:
 
 def attention_prefill(q, k_pool, v_pool, out, tile_item, tile_q0, cu_tokens, kv_lens, tables,
                       heads, scale, window=0, max_kv_len=0, query_tile=PREFILL_TILE, memo=None,
-                      shared=None, sink=None, gate=None, softcap=0.0):
+                      shared=None, sink=None, gate=None, softcap=0.0, logistic=None):
     """Attention of items with several tokens, ``query_tile`` (64, 32 or 128) queries per block,
     on the matrix cores.  Blocks start in the order of the tile list, which is cut for that size:
     the tiles that see the most keys belong first.
@@ -976,7 +1008,7 @@ def attention_prefill(q, k_pool, v_pool, out, tile_item, tile_q0, cu_tokens, kv_
         step_key = ("prefill", q.data_ptr(), q.shape[0], out.data_ptr(),
                     tile_item.data_ptr(), tile_item.numel(), tile_q0.data_ptr(), cu_tokens.data_ptr(),
                     cu_tokens.numel(), kv_lens.data_ptr(), tables.data_ptr(), tables.shape[1], heads, scale,
-                    window, max_kv_len, query_tile, _ptr(sink), _ptr(gate), softcap)
+                    window, max_kv_len, query_tile, _ptr(sink), _ptr(gate), softcap, *_logistic_key(logistic))
         key = step_key + (k_pool.data_ptr(), v_pool.data_ptr())
         kept = memo.get(key) or _sibling_call(memo, shared, key, step_key, k_pool, v_pool)
         if kept is not None:
@@ -1007,7 +1039,7 @@ def attention_prefill(q, k_pool, v_pool, out, tile_item, tile_q0, cu_tokens, kv_
                 cu_tokens.data_ptr(), kv_lens.data_ptr(), tables.data_ptr(), tables.shape[1], heads,
                 kv_heads, head_dim, page_size, pages, float(scale), int(window), int(max_kv_len),
                 int(query_tile), _check_sink(sink, heads), *_check_gate(gate, q.shape[0], heads),
-                _check_cap(softcap), dtype_code(q.dtype)),
+                _check_cap(softcap), *_check_logistic(logistic, heads), dtype_code(q.dtype)),
                shared, step_key, (kv_heads, head_dim, page_size, pages, q.dtype))
     return out
 
@@ -1022,7 +1054,7 @@ _TILED_F32_CHECKED = False
 
 
 def attention_tiled_f32(q, k_pool, v_pool, out, tile_item, tile_q0, cu_tokens, kv_lens, tables, heads,
-                        scale, window=0, sink=None, gate=None, softcap=0.0):
+                        scale, window=0, sink=None, gate=None, softcap=0.0, logistic=None):
     """Attention of items with several tokens in true 32-bit, ``PREFILL_TILE`` queries per
     block: keys and values pass through LDS once per tile of queries instead of once per query
     (``attention_rowwise``), scores and sums are plain float arithmetic.  The tile list is the
@@ -1058,7 +1090,7 @@ def attention_tiled_f32(q, k_pool, v_pool, out, tile_item, tile_q0, cu_tokens, k
           out.data_ptr(), out_stride, tile_item.data_ptr(), tile_q0.data_ptr(), tiles,
           cu_tokens.data_ptr(), kv_lens.data_ptr(), tables.data_ptr(), tables.shape[1], heads,
           kv_heads, head_dim, page_size, pages, float(scale), int(window), _check_sink(sink, heads),
-          *_check_gate(gate, q.shape[0], heads), _check_cap(softcap), _stream())
+          *_check_gate(gate, q.shape[0], heads), _check_cap(softcap), *_check_logistic(logistic, heads), _stream())
     return out
 
 
@@ -1110,7 +1142,7 @@ def _sibling_call(memo, shared, key, step_key, k_pool, v_pool):
 
 def attention_mixed(q, k_pool, v_pool, out, tok_list, tok_item, positions, tile_item, tile_q0,
                     cu_tokens, kv_lens, tables, heads, scale, window=0, memo=None, shared=None,
-                    sink=None, gate=None, softcap=0.0):
+                    sink=None, gate=None, softcap=0.0, logistic=None):
     """The attention of a step that mixes decoded tokens with prompt portions, in one launch:
     the tokens listed in ``tok_list`` (the step's one-token items) as ``attention_decode`` with
     one range of keys computes them, the tiles of 64 queries listed in ``tile_item`` /
@@ -1126,7 +1158,7 @@ def attention_mixed(q, k_pool, v_pool, out, tok_list, tok_item, positions, tile_
                     tok_list.data_ptr(), tok_list.numel(), tok_item.data_ptr(), positions.data_ptr(),
                     tile_item.data_ptr(), tile_item.numel(), tile_q0.data_ptr(), cu_tokens.data_ptr(),
                     cu_tokens.numel(), kv_lens.data_ptr(), tables.data_ptr(), tables.shape[1], heads, scale, window,
-                    _ptr(sink), _ptr(gate), softcap)
+                    _ptr(sink), _ptr(gate), softcap, *_logistic_key(logistic))
         key = step_key + (k_pool.data_ptr(), v_pool.data_ptr())
         kept = memo.get(key) or _sibling_call(memo, shared, key, step_key, k_pool, v_pool)
         if kept is not None:
@@ -1160,7 +1192,7 @@ def attention_mixed(q, k_pool, v_pool, out, tok_list, tok_item, positions, tile_
                 positions.data_ptr(), tile_item.data_ptr(), tile_q0.data_ptr(), tiles,
                 cu_tokens.data_ptr(), kv_lens.data_ptr(), tables.data_ptr(), tables.shape[1], heads,
                 kv_heads, head_dim, page_size, pages, float(scale), int(window),
-                _check_sink(sink, heads), *_check_gate(gate, q.shape[0], heads), _check_cap(softcap),
+                _check_sink(sink, heads), *_check_gate(gate, q.shape[0], heads), _check_cap(softcap), *_check_logistic(logistic, heads),
                 dtype_code(q.dtype)),
                shared, step_key, (kv_heads, head_dim, page_size, pages, q.dtype))
     return out
@@ -1752,7 +1784,7 @@ def stream_step(h, tokens, width, add=None, bias=None, norm=None, zero=None, row
           _stream())
 
 
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "relu": 2}
 
 # constants of the gated unit ``g' sigmoid(slope g') (u' + shift)`` with ``g' = min(g, limit)`` and
 # ``u' = clamp(u, -limit, limit)`` (csrc/common.h: GateForm); these are ``silu(g) * u``
@@ -1769,8 +1801,8 @@ def _gate_form(form):
 
 def silu_gate(gu, out, activation="silu", form=PLAIN_GATE, row_scale=None):
     """``out[t, c] = act(gu[t, c]) * gu[t, inner + c]`` for float ``gu`` of ``2 * inner`` columns;
-    ``act``: ``silu`` (with the unit's other constants as ``form = (limit, slope, shift)``) or
-    ``gelu_tanh``.  ``row_scale``: a float per row that multiplies it."""
+    ``act``: ``silu`` (with the unit's other constants as ``form = (limit, slope, shift)``),
+    ``gelu_tanh`` or ``relu``.  ``row_scale``: a float per row that multiplies it."""
     if row_scale is not None:
         _float_vector(row_scale, "row_scale", gu.shape[0])
     if activation not in GATE_ACTIVATIONS:
@@ -1936,6 +1968,169 @@ def moe_experts(x, w1, w2, ids, weights, hidden, y, gated=True, extra=None, form
           weights.data_ptr(), hidden.data_ptr(), y.data_ptr(), tokens, width, inner, top,
           1 if gated else 0, *_gate_form(form), _ptr(w1x), _ptr(w2x), inner_x, float(extra_limit),
           dtype_code(x.dtype), _stream())
+
+
+def gated_norm_step(h, tokens, width, eps, add=None, norm=None):
+    """One pass over the float stream ``h`` with layer norms (scale and shift): ``add = (y, gate, gate_bias,
+    gamma, beta)``: ``h += layer_norm(sigmoid(gate + gate_bias) * y) * gamma + beta`` and ``y`` is cleared
+    (``gate``: float columns of a wider buffer); ``norm = (gamma, beta, normed)``: ``normed`` gets the layer norm
+    of the new ``h`` in the engine dtype."""
+    _float_rows(h, "h", tokens, width)
+    y = gate = gate_bias = gamma = beta = gamma2 = beta2 = normed = None
+    gate_ld, code = 0, F32
+    if add is not None:
+        y, gate, gate_bias, gamma, beta = add
+        _float_rows(y, "y", tokens, width)
+        gate_ld = _float_columns(gate, "gate", tokens, width)
+        for name, vector in (("gate_bias", gate_bias), ("gamma", gamma), ("beta", beta)):
+            _float_vector(vector, name, width)
+    if norm is not None:
+        gamma2, beta2, normed = norm
+        _float_vector(gamma2, "gamma2", width)
+        _float_vector(beta2, "beta2", width)
+        _check(normed, "normed", ndim=2)
+        if normed.shape[0] < tokens or normed.shape[1] != width or not normed.is_contiguous():
+            raise KernelError("gated_norm_step: normed must be contiguous [>= tokens, width]")
+        code = dtype_code(normed.dtype)
+    _call("ps_gated_norm_step", h.data_ptr(), _ptr(y), _ptr(gate), gate_ld, _ptr(gate_bias), _ptr(gamma), _ptr(beta),
+          _ptr(gamma2), _ptr(beta2), float(eps), _ptr(normed), tokens, width, code, _stream())
+
+
+def _float_columns(tensor, name, rows, columns):
+    """Row stride of float columns of a (possibly wider) buffer."""
+    _check(tensor, name, torch.float32, 2)
+    if tensor.shape[0] < rows or tensor.shape[1] != columns:
+        raise KernelError(f"{name} must be float [>= {rows}, {columns}], got {tuple(tensor.shape)}")
+    return _rows(tensor, name)
+
+
+def _slot_rows(state, needed, what):
+    """Row stride of a state that is one run of floats per slot."""
+    _check(state, "state", torch.float32, 2)
+    if state.shape[1] < needed or not state.is_contiguous():
+        raise KernelError(f"{what}: a slot of {state.shape[1]} floats cannot hold {needed}")
+    return state.shape[1]
+
+
+STATE_RULES = {"decayed": 0, "delta": 1}
+
+
+def state_prepare(proj, col, weight, bias, state, history, out, rule, decay, take, a_log, z_bias, take_col,
+                  tok_item, cu_tokens, slots, z=None, per_head=1, unit_heads=0, head=0, scale_heads=0,
+                  q_scale=1.0):
+    """What a matrix-state recurrence is fed with (``csrc/pagedserve_hip.h: ps_state_prepare``): the short
+    convolution of ``weight [channels, taps]`` with silu and unit norms into ``out`` (float), decays and weights.
+    ``history``: where a slot of ``state`` (float ``[slots, n]``) keeps the last inputs."""
+    _check(proj, "proj", torch.float32, 2)
+    _check(weight, "weight", torch.float32, 2)
+    tokens = proj.shape[0]
+    channels, taps = weight.shape
+    heads = a_log.numel()
+    if not weight.is_contiguous() or col + channels > proj.shape[1] or take_col + heads > proj.shape[1]:
+        raise KernelError("state_prepare: the projection's rows are too short for its columns")
+    if bias is not None:
+        _float_vector(bias, "bias", channels)
+    stride = _slot_rows(state, history + (taps - 1) * channels, "state_prepare")
+    _float_rows(out, "out", tokens, channels)
+    _float_vector(a_log, "a_log", heads)
+    _float_vector(z_bias, "z_bias", heads * per_head)
+    _float_rows(take, "take", tokens, heads)
+    _float_rows(decay, "decay", tokens, heads * per_head)
+    z_ld = 0
+    if z is not None:
+        z_ld = _float_columns(z, "z", tokens, heads * per_head)
+    if unit_heads and (unit_heads * head > channels or not 0 < head <= 256):
+        raise KernelError("state_prepare: the unit heads do not fit the channels")
+    _check(tok_item, "tok_item", torch.int32, 1)
+    if tok_item.numel() < tokens:
+        raise KernelError("state_prepare: tok_item is shorter than the step")
+    _step_items(cu_tokens, slots, "state_prepare")
+    _call("ps_state_prepare", proj.data_ptr(), _rows(proj, "proj"), int(col), channels, taps, weight.data_ptr(),
+          _ptr(bias), state.data_ptr(), stride, int(history), out.data_ptr(), int(unit_heads), int(head),
+          int(scale_heads), float(q_scale), STATE_RULES[rule], heads, int(per_head), _ptr(z), z_ld,
+          z_bias.data_ptr(), a_log.data_ptr(), int(take_col), decay.data_ptr(), take.data_ptr(),
+          tok_item.data_ptr(), cu_tokens.data_ptr(), slots.data_ptr(), tokens, _stream())
+
+
+def memory_gates(proj, i_col, f_col, i_bias, f_bias, cap, state, maxima, log_decay, take, floor, cu_tokens, slots):
+    """Exponential gates with a running maximum that the slot keeps from float ``maxima`` on
+    (``csrc/pagedserve_hip.h: ps_memory_gates``)."""
+    _check(proj, "proj", torch.float32, 2)
+    tokens = proj.shape[0]
+    heads = i_bias.numel()
+    if max(i_col, f_col) + heads > proj.shape[1]:
+        raise KernelError("memory_gates: the projection's rows are too short for its columns")
+    _float_vector(i_bias, "i_bias", heads)
+    _float_vector(f_bias, "f_bias", heads)
+    stride = _slot_rows(state, maxima + heads, "memory_gates")
+    for name, rows in (("log_decay", log_decay), ("take", take), ("floor", floor)):
+        _float_rows(rows, name, tokens, heads)
+    items = _step_items(cu_tokens, slots, "memory_gates")
+    _call("ps_memory_gates", proj.data_ptr(), _rows(proj, "proj"), int(i_col), int(f_col), i_bias.data_ptr(),
+          f_bias.data_ptr(), float(cap), state.data_ptr(), stride, int(maxima), log_decay.data_ptr(),
+          take.data_ptr(), floor.data_ptr(), cu_tokens.data_ptr(), slots.data_ptr(), items, heads, _stream())
+
+
+def state_scan(q, k, v, decay, take, state, out, cu_tokens, slots, rule, heads, key_heads, key_dim, value_dim,
+               ones=False, q_scale=1.0, longest=0, raw=None, taps=1, history=0):
+    """The recurrence over the step's items (``csrc/pagedserve_hip.h: ps_state_scan``).  ``q``, ``k``, ``v``: float columns
+    of (possibly wider) buffers; ``state``: float ``[slots, n]`` whose slots begin with the heads' matrices;
+    ``raw``: the raw input columns of the short convolution that the slot keeps (from ``history`` on)."""
+    tokens = q.shape[0]
+    q_ld = _float_columns(q, "q", tokens, key_heads * key_dim)
+    k_ld = _float_columns(k, "k", tokens, key_heads * key_dim)
+    v_ld = _float_columns(v, "v", tokens, heads * value_dim)
+    columns = value_dim + (1 if ones else 0)
+    _float_rows(decay, "decay", tokens, heads * (key_dim if rule == "delta" else 1))
+    _float_rows(take, "take", tokens, heads)
+    _float_rows(out, "out", tokens, heads * columns)
+    needed = heads * columns * key_dim
+    channels, raw_ld = 0, 0
+    if raw is not None:
+        channels = raw.shape[1]
+        raw_ld = _float_columns(raw, "raw", tokens, channels)
+        if history < needed:
+            raise KernelError("state_scan: the kept inputs overlap the state")
+        needed = history + (taps - 1) * channels
+    stride = _slot_rows(state, needed, "state_scan")
+    if heads % key_heads:
+        raise KernelError(f"state_scan: {heads} heads do not share {key_heads} key heads evenly")
+    items = _step_items(cu_tokens, slots, "state_scan")
+    _call("ps_state_scan", q.data_ptr(), q_ld, k.data_ptr(), k_ld, v.data_ptr(), v_ld, decay.data_ptr(),
+          take.data_ptr(), state.data_ptr(), stride, out.data_ptr(), cu_tokens.data_ptr(), slots.data_ptr(), items,
+          STATE_RULES[rule], heads, heads // key_heads, key_dim, value_dim, 1 if ones else 0, float(q_scale),
+          int(longest), _ptr(raw), raw_ld, channels, int(taps), int(history), _stream())
+
+
+def state_output(o, heads, value_dim, weight, eps, groups, out, floor=None, skip=None, u=None, before=None,
+                 behind=None):
+    """Norm and gates of a recurrence's output (``csrc/pagedserve_hip.h: ps_state_output``): ``floor``: the output has a
+    key sum per head and is divided by it; ``skip``, ``u``: ``skip[h] * u`` is added; ``before``: float columns whose silu
+    multiplies ahead of the norm over ``groups`` equal runs of columns; ``behind``: columns whose sigmoid multiplies
+    behind it.  ``weight``: a float per column, or per column of a head."""
+    columns = heads * value_dim
+    ones = floor is not None
+    tokens = out.shape[0]
+    _float_rows(o, "o", tokens, heads * (value_dim + (1 if ones else 0)))
+    _check(out, "out", ndim=2)
+    if out.shape[1] != columns or columns % groups:
+        raise KernelError(f"state_output: out must hold {columns} columns in {groups} equal groups")
+    _check(weight, "weight", torch.float32, 1)
+    if weight.numel() not in (columns, value_dim) or not weight.is_contiguous():
+        raise KernelError("state_output: a weight per column, or per column of a head")
+    u_ld = before_ld = behind_ld = 0
+    if ones:
+        _float_rows(floor, "floor", tokens, heads)
+    if skip is not None:
+        _float_vector(skip, "skip", heads)
+        u_ld = _float_columns(u, "u", tokens, columns)
+    if before is not None:
+        before_ld = _float_columns(before, "before", tokens, columns)
+    if behind is not None:
+        behind_ld = _float_columns(behind, "behind", tokens, columns)
+    _call("ps_state_output", o.data_ptr(), heads, value_dim, 1 if ones else 0, _ptr(floor), _ptr(skip), _ptr(u), u_ld,
+          _ptr(before), before_ld, weight.data_ptr(), weight.numel(), float(eps), int(groups), _ptr(behind), behind_ld,
+          out.data_ptr(), _rows(out, "out"), tokens, dtype_code(out.dtype), _stream())
 
 
 def gla_output(o, weight, eps, gate, out, heads, value_dim):

@@ -56,10 +56,13 @@ class Attention(Mixer):
     * ``values_from_keys``: there is no value projection; the values are the keys as projected,
       before rotation and norm (the packed product is ``[q | k]``).
     * ``score_cap``: ``c > 0``: a scaled score ``s`` enters the softmax as ``c tanh(s / c)``.
+    * ``logistic``: no softmax; a visible key weighs ``sigmoid(score + shift)`` with a learned ``shift`` per
+      head (``logistic.shift``), and the weights are not normalised.  ``out_scale`` multiplies the result (with
+      ``logistic`` only: the kernels divide by a constant where a softmax divides by its sum).
     * ``pad_heads``: heads are cached with their size rounded up to a multiple of this (zeros
       behind), so that a head size which the tiled kernels do not take still runs on them.
 
-    ``rotary_layout="halves"``, ``rotary_scaling``, ``rotary_bands``, ``head_norm`` and ``values_from_keys`` go
+    ``rotary_layout="halves"``, ``rotary_scaling``, ``rotary_bands``, ``head_norm``, ``values_from_keys`` and ``logistic`` go
     through the launch that treats every head on its own (``kernels.attention_prepare_heads``);
     that one does not norm over the whole projection or mix values.
     """
@@ -79,6 +82,7 @@ class Attention(Mixer):
     VALUE_MIXES = ("none", "source", "mix")
 
     chunk = 0      # (mixers that are built on this one and set no chunk of their own)
+    logistic = None
 
     @property
     def span(self) -> int:
@@ -91,7 +95,8 @@ class Attention(Mixer):
                  sink: bool = False, value_mix: str = "none", head_gate: bool = False,
                  out_bias=None, rotary_layout: str = "neighbours", rotary_scaling=None,
                  head_norm=False, values_from_keys: bool = False, score_cap: float = 0.0,
-                 pad_heads: int = 0, chunk: int = 0, rotary_bands=None):
+                 pad_heads: int = 0, chunk: int = 0, rotary_bands=None, logistic: bool = False,
+                 out_scale: float = 1.0):
         if heads % kv_heads != 0:
             raise ValueError(f"heads ({heads}) must be a multiple of kv_heads ({kv_heads})")
         if not 0 < head_dim <= 256:
@@ -140,8 +145,14 @@ class Attention(Mixer):
             raise ValueError("a score cap must be positive (0: none)")
         if self.values_from_keys and self.value_dim != self.key_dim:
             raise ValueError("values that are the keys have the keys' head size")
+        self.is_logistic = bool(logistic)
+        self.out_scale = float(out_scale)
+        if self.is_logistic and self.has_sink:
+            raise ValueError("a sink belongs to a softmax")
+        if self.out_scale != 1.0 and not self.is_logistic:
+            raise ValueError("a factor on the result goes with logistic weights")
         # the launch that treats every head on its own
-        self.head_wise = (self.head_norm or self.values_from_keys or self.rotary_scaling is not None
+        self.head_wise = (self.is_logistic or self.head_norm or self.values_from_keys or self.rotary_scaling is not None
                           or self.rotary_bands is not None or (self.rotary_halves and self.rotary_dims > 0))
         if self.head_wise and (self.qk_norm or value_mix != "none"):
             raise ValueError("a norm over the whole projection and mixed values do not go with "
@@ -198,23 +209,66 @@ class Attention(Mixer):
             params["sink"] = ParamSpec((self.heads,), VECTOR)
         if self.value_mix == "mix":
             params["value_mix.weight"] = ParamSpec((), VECTOR)
+        if self.is_logistic:
+            params["logistic.shift"] = ParamSpec((self.heads,), VECTOR)
         return params
+
+    # ---- as one of several mixers between two products of the caller (``parts/joined.py``)
+    PRODUCTS = ("qkv.weight", "out.weight", "qkv.bias", "out.bias")
+
+    @property
+    def core_rows(self):
+        return self._projection_columns()[4]
+
+    @property
+    def core_columns(self):
+        return self.q_cols
+
+    @property
+    def stored_columns(self):
+        return self.heads * self.value_dim
+
+    def core_parameters(self):
+        if self.bias or self.out_has_bias or not self.head_wise:
+            raise ValueError("attention between products of the caller has no biases and treats its heads one by one")
+        return {name: spec for name, spec in self.parameters().items() if name not in self.PRODUCTS}
+
+    def core(self, proj, col, out, ctx, cache):
+        tables = ctx.tables[cache.group]
+        q, gates = self._prepare_heads(proj, col, ctx, cache, tables)
+        self._attend(q, out, gates, None, ctx, cache, tables)
+
+    def pad_out(self, weight):
+        """The output matrix for the context's heads, which may be cached wider than the values: zero columns there."""
+        if self.head_dim == self.value_dim:
+            return weight
+        padded = weight.new_zeros((self.width, self.heads, self.head_dim))
+        padded[:, :, :self.value_dim] = weight.reshape(self.width, self.heads, self.value_dim)
+        return padded.view(self.width, self.q_cols)
 
     def bind(self, tensors):
         self.qkv_weight = tensors["qkv.weight"]
-        self.out_weight = tensors["out.weight"]
+        self.out_weight = self.pad_out(tensors["out.weight"])
         self.qkv_bias = tensors.get("qkv.bias")
         self.out_bias = tensors.get("out.bias")
+        self.bind_core(tensors, self.out_weight.device)
+        # copies in the layout that the products of few rows (decode steps) read fastest
+        self.qkv_packed = kernels.pack_decode_weight(self.qkv_weight)
+        self.out_packed = kernels.pack_decode_weight(self.out_weight)
+        self._memo_qkv.clear()
+        self._memo_out.clear()
+
+    def bind_core(self, tensors, device):
+        """Everything but the two products' matrices and biases."""
         self.q_gamma = tensors.get("q_norm.gamma")
         self.k_gamma = tensors.get("k_norm.gamma")
         self.sink = tensors.get("sink")
         self.mix_weight = tensors["value_mix.weight"].reshape(1) if self.value_mix == "mix" else None
-        if self.head_dim != self.value_dim:
-            # heads are cached wider than the values: the context has zero columns there, and
-            # the output projection gets zero columns to match
-            padded = self.out_weight.new_zeros((self.width, self.heads, self.head_dim))
-            padded[:, :, :self.value_dim] = self.out_weight.view(self.width, self.heads, self.value_dim)
-            self.out_weight = padded.view(self.width, self.q_cols)
+        self.logistic = None
+        if self.is_logistic:
+            # (the kernels divide the weighted values by this number)
+            norm = 1.0 / self.out_scale if self.out_scale else float("inf")
+            self.logistic = (tensors["logistic.shift"], norm)
         self.freqs = None
         self.rotary_magnitude = 1.0
         if self.rotary_dims:
@@ -224,12 +278,7 @@ class Attention(Mixer):
             else:
                 freqs, self.rotary_magnitude = rotary_frequencies(self.rotary_dims, self.rotary_base,
                                                                   self.rotary_scaling)
-            self.freqs = freqs.to(torch.float32).to(self.out_weight.device)
-        # copies in the layout that the products of few rows (decode steps) read fastest
-        self.qkv_packed = kernels.pack_decode_weight(self.qkv_weight)
-        self.out_packed = kernels.pack_decode_weight(self.out_weight)
-        self._memo_qkv.clear()
-        self._memo_out.clear()
+            self.freqs = freqs.to(torch.float32).to(device)
         self._memo_attention.clear()
 
     def cache_spec(self):
@@ -245,19 +294,13 @@ class Attention(Mixer):
         proj = ctx.workspace.first_rows("attn_proj", total, torch.float32, tokens)
         kernels.linear(x, self.qkv_weight, self.qkv_bias, proj, packed=self.qkv_packed,
                        memo=site_memo(self._memo_qkv, ctx.workspace), shared=ctx.shared_calls)
+        if self.head_wise:
+            return self._prepare_heads(proj, 0, ctx, cache, tables)
         q = ctx.workspace.first_rows("attn_q", self.q_cols, self.dtype, tokens)
         v_first = None
         if self.value_mix != "none":
             v_first = ctx.workspace.first_rows("values_source", self.kv_heads * self.value_dim,
                                                self.dtype, tokens)
-        if self.head_wise:
-            kernels.attention_prepare_heads(
-                proj, (q_col, k_col, v_col), q, cache.k_pool, cache.v_pool, ctx.tok_item, ctx.positions,
-                tables, self.heads, self.key_dim, self.value_dim, freqs=self.freqs,
-                rot_dims=self.rotary_dims, halves=self.rotary_halves, magnitude=self.rotary_magnitude,
-                head_norm=self.head_norm, eps=self.norm_eps, norm_first=self.norm_before,
-                q_gamma=self.q_gamma, k_gamma=self.k_gamma)
-            return q, (proj[:, gate_col:gate_col + self.heads] if self.head_gate else None)
         kernels.attention_prepare(
             proj, (q_col, k_col, v_col), q, cache.k_pool, cache.v_pool, ctx.tok_item, ctx.positions,
             tables, self.heads, self.key_dim, self.value_dim, q_gamma=self.q_gamma,
@@ -266,7 +309,22 @@ class Attention(Mixer):
             v_mode=self.VALUE_MIXES.index(self.value_mix))
         return q, (proj[:, gate_col:gate_col + self.heads] if self.head_gate else None)
 
+    def _prepare_heads(self, proj, col, ctx, cache, tables):
+        """Rotation, norms and cache write of the heads whose float columns begin at ``col`` of ``proj``; returns the
+        queries and the gates' columns."""
+        q_col, k_col, v_col, gate_col, _ = (col + at for at in self._projection_columns())
+        q = ctx.workspace.first_rows("attn_q", self.q_cols, self.dtype, ctx.tokens)
+        kernels.attention_prepare_heads(
+            proj, (q_col, k_col, v_col), q, cache.k_pool, cache.v_pool, ctx.tok_item, ctx.positions,
+            tables, self.heads, self.key_dim, self.value_dim, freqs=self.freqs,
+            rot_dims=self.rotary_dims, halves=self.rotary_halves, magnitude=self.rotary_magnitude,
+            head_norm=self.head_norm, eps=self.norm_eps, norm_first=self.norm_before,
+            q_gamma=self.q_gamma, k_gamma=self.k_gamma)
+        return q, (proj[:, gate_col:gate_col + self.heads] if self.head_gate else None)
+
     def _project_out(self, context, residual, ctx):
+        if residual is None:
+            return      # (the caller multiplies)
         kernels.linear(context, self.out_weight, self.out_bias, residual, epilogue="residual",
                        packed=self.out_packed, memo=site_memo(self._memo_out, ctx.workspace),
                        shared=ctx.shared_calls)
@@ -316,7 +374,7 @@ class Attention(Mixer):
             # too, goes to the kernel that takes all sizes
             singles = 0
         merged_splits = 0
-        if gates is None and singles == tokens and kernels.merge_linear_supported(
+        if residual is not None and gates is None and singles == tokens and kernels.merge_linear_supported(
                 self.dtype, tokens, self.head_dim, self.out_packed):
             merged_splits = self._merged_splits(singles, ctx.max_kv_len)
         if merged_splits:
@@ -326,7 +384,7 @@ class Attention(Mixer):
             partial = self._range_records(ctx)
             kernels.attention_decode_partial(q, cache.k_pool, cache.v_pool, partial, ctx.tok_item,
                                              ctx.positions, tables, self.heads, self.scale, splits,
-                                             window=self.span, waves=4, sink=sink, softcap=self.score_cap)
+                                             window=self.span, waves=4, sink=sink, softcap=self.score_cap, logistic=self.logistic)
             kernels.attention_merge_linear(partial, singles, self.heads, self.head_dim, splits,
                                            self.out_weight, self.out_packed, self.out_bias, residual)
             return
@@ -338,7 +396,7 @@ class Attention(Mixer):
                                     ctx.tok_item, ctx.positions, tile_item, tile_q0, ctx.cu_tokens,
                                     ctx.kv_lens, tables, self.heads, self.scale, self.span,
                                     memo=site_memo(self._memo_attention, ctx.workspace),
-                                    shared=ctx.shared_calls, sink=sink, gate=gates, softcap=self.score_cap)
+                                    shared=ctx.shared_calls, sink=sink, gate=gates, softcap=self.score_cap, logistic=self.logistic)
             return self._project_out(context, residual, ctx)
         if singles and kernels.shared_decode_supported(self.dtype, self.heads, self.kv_heads, self.head_dim, sink):
             # many heads to a key/value head: blocks that load a tile of keys once for all of them
@@ -348,7 +406,7 @@ class Attention(Mixer):
                                             self._shared_splits(singles, ctx.max_kv_len),
                                             self._range_records(ctx), window=self.span,
                                             tok_list=None if singles == tokens else ctx.single_tokens,
-                                            gate=gates, softcap=self.score_cap)
+                                            gate=gates, softcap=self.score_cap, logistic=self.logistic)
         elif singles:
             # one-token items: keys of a request are cut into ranges so that few requests
             # still fill the chip
@@ -369,7 +427,7 @@ class Attention(Mixer):
                                      ctx.positions, tables, self.heads, self.scale, splits,
                                      partial=partial, window=self.span, waves=waves,
                                      tok_list=None if singles == tokens else ctx.single_tokens,
-                                     sink=sink, gate=gates, softcap=self.score_cap)
+                                     sink=sink, gate=gates, softcap=self.score_cap, logistic=self.logistic)
         whole = singles == 0
         if tiled:
             size = kernels.PREFILL_TILE
@@ -387,7 +445,7 @@ class Attention(Mixer):
                                       self.heads, self.scale, self.span,
                                       max_kv_len=ctx.max_kv_len, query_tile=size,
                                       memo=site_memo(self._memo_attention, ctx.workspace),
-                                      shared=ctx.shared_calls, sink=sink, gate=gates, softcap=self.score_cap)
+                                      shared=ctx.shared_calls, sink=sink, gate=gates, softcap=self.score_cap, logistic=self.logistic)
         elif singles < tokens and kernels.tiled_f32_supported(self.dtype, self.head_dim):
             # 32-bit: tiles of queries too, on plain float arithmetic.  The tiles hold the items
             # of several tokens; one-token items that the split-KV kernel did not take (a head
@@ -396,16 +454,16 @@ class Attention(Mixer):
             if tile_item.numel():
                 kernels.attention_tiled_f32(q, cache.k_pool, cache.v_pool, context, tile_item, tile_q0,
                                             ctx.cu_tokens, ctx.kv_lens, tables, self.heads, self.scale,
-                                            self.span, sink=sink, gate=gates, softcap=self.score_cap)
+                                            self.span, sink=sink, gate=gates, softcap=self.score_cap, logistic=self.logistic)
             if not singles and ctx.single_tokens is not None and ctx.single_tokens.numel():
                 kernels.attention_rowwise(q, cache.k_pool, cache.v_pool, context, ctx.tok_item,
                                           ctx.positions, tables, self.heads, self.scale, self.span,
                                           tok_list=None if ctx.single_tokens.numel() == tokens
-                                          else ctx.single_tokens, sink=sink, gate=gates, softcap=self.score_cap)
+                                          else ctx.single_tokens, sink=sink, gate=gates, softcap=self.score_cap, logistic=self.logistic)
         elif singles < tokens:
             kernels.attention_rowwise(q, cache.k_pool, cache.v_pool, context, ctx.tok_item,
                                       ctx.positions, tables, self.heads, self.scale, self.span,
-                                      tok_list=None if whole else ctx.portion_tokens, sink=sink, gate=gates, softcap=self.score_cap)
+                                      tok_list=None if whole else ctx.portion_tokens, sink=sink, gate=gates, softcap=self.score_cap, logistic=self.logistic)
         self._project_out(context, residual, ctx)
 
     def _one_launch(self, singles: int, ctx, tables) -> bool:

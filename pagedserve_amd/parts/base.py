@@ -31,7 +31,8 @@ from typing import Dict, List, Optional
 
 import torch
 
-from ..weights.loader import ParamSpec
+from ..ops import kernels
+from ..weights.loader import MATRIX, ParamSpec
 
 
 @dataclass(frozen=True)
@@ -147,6 +148,71 @@ class Mixer(Part):
 
     def forward(self, x, residual, ctx, cache: CacheView):
         raise NotImplementedError
+
+
+class CoreMixer(Mixer):
+    """A mixer that works between two products: a packed product of the layer's input in float, the mixer's own
+    work (``core``) on its columns, and an output product of what that leaves.  Kinds give ``core_rows`` (rows
+    of the packed product) and ``core_columns`` (inputs of the output product) to the constructor, and implement
+    ``core_parameters``, ``bind_core`` and ``core(proj, col, out, ctx, cache)``: read the float columns ``col ..
+    col + core_rows - 1`` of ``proj``, write ``out [T, core_columns]`` in the engine dtype.  A mixer made of several
+    runs the two products for all of them.
+
+    ``ride``: that many more rows of the packed product belong to the caller (the arrangement's gate on the
+    result, for instance): ``forward`` returns their float columns."""
+
+    graph_safe = True
+
+    accepts_pending_norm = True
+
+    def __init__(self, width: int, dtype, core_rows: int, core_columns: int, ride: int = 0):
+        self.width = width
+        self.dtype = dtype
+        self.core_rows = core_rows
+        self.core_columns = self.stored_columns = core_columns
+        self.ride = int(ride)
+        self._memo_in, self._memo_out = {}, {}
+
+    def core_parameters(self):
+        return {}
+
+    def bind_core(self, tensors, device):
+        raise NotImplementedError
+
+    def core(self, proj, col, out, ctx, cache):
+        raise NotImplementedError
+
+    def pad_out(self, weight):
+        """The output matrix for ``core_columns`` from the stored one of ``stored_columns``."""
+        return weight
+
+    def parameters(self):
+        return {
+            "in.weight": ParamSpec((self.core_rows + self.ride, self.width), MATRIX),
+            "out.weight": ParamSpec((self.width, self.stored_columns), MATRIX),
+            **self.core_parameters(),
+        }
+
+    def bind(self, tensors):
+        self.in_weight = tensors["in.weight"]
+        self.out_weight = self.pad_out(tensors["out.weight"])
+        self.bind_core({name: tensors[name] for name in self.core_parameters()}, self.in_weight.device)
+        self.in_packed = kernels.pack_decode_weight(self.in_weight)
+        self.out_packed = kernels.pack_decode_weight(self.out_weight)
+        self._memo_in.clear()
+        self._memo_out.clear()
+
+    def forward(self, x, residual, ctx, cache):
+        tokens, workspace = ctx.tokens, ctx.workspace
+        proj, _, ridden = workspace.column_views("core_proj", self.core_rows + self.ride, torch.float32, tokens,
+                                                 (self.core_rows, self.ride))
+        kernels.linear(x, self.in_weight, None, proj, packed=self.in_packed,
+                       memo=site_memo(self._memo_in, workspace), shared=ctx.shared_calls)
+        out = workspace.first_rows("core_out", self.core_columns, self.dtype, tokens)
+        self.core(proj, 0, out, ctx, cache)
+        kernels.linear(out, self.out_weight, None, residual, epilogue="residual", packed=self.out_packed,
+                       memo=site_memo(self._memo_out, workspace), shared=ctx.shared_calls)
+        return ridden if self.ride else None
 
 
 class FeedForward(Part):

@@ -312,3 +312,75 @@ class ParallelScaledMixerBlock(ParallelScaledBlock):
     """The same with a mixer only."""
 
     roles = {"norm1": "norm", "mixer": "mixer"}
+
+
+_GATED_ADD = "gated_add"      # key of ``ctx.extra``: a sublayer's result with its gate and norm, not added yet
+
+
+@register_arrangement("gated_between_norms")
+class GatedBetweenNormsBlock:
+    """``h += post1(sigmoid(G1 u + b1) * mixer(u))`` with ``u = norm1(h)``, then the same with ``norm2``, ``feed_forward``, ``gate2``
+    and ``post2``: a norm on either side of every sublayer and a gate on its result ahead of the second one,
+    all norms layer norms with a shift.  The gates' rows ride along in the sublayers' packed products
+    (``parts/connection.py: ridden_gate``).  A sublayer adds into a float row ``y`` per token; one launch
+    gates and norms it, adds it to the stream, norms for the next sublayer and clears ``y``
+    (``kernels.gated_norm_step``).  A block's last sum is left to the next block's first launch, or to
+    ``finish``."""
+
+    roles = {"norm1": "norm", "mixer": "mixer", "gate1": "connection", "post1": "norm",
+             "norm2": "norm", "feed_forward": "feed_forward", "gate2": "connection", "post2": "norm"}
+    takes_stream_write = "gated_between_norms"
+
+    def __init__(self, width, dtype, parts):
+        self.width = width
+        self.dtype = dtype
+        self._parts = dict(parts)
+        self.mixer = parts["mixer"]
+        self.sublayers = [(parts["norm1"], self.mixer, parts["gate1"], parts["post1"])]
+        if "feed_forward" in parts:
+            self.sublayers.append((parts["norm2"], parts["feed_forward"], parts["gate2"], parts["post2"]))
+        self.eps = parts["norm1"].eps
+        for norm, part, _, post in self.sublayers:
+            if any(getattr(one, "eps", None) != self.eps or "beta" not in one.parameters() for one in (norm, post)):
+                raise ValueError("a gated block between norms needs layer norms with a shift and of one eps")
+            if getattr(part, "ride", 0) != width:
+                raise ValueError("the sublayers of a gated block between norms carry the gate's rows")
+
+    @property
+    def graph_safe(self):
+        return all(getattr(part, "graph_safe", False) for part in self._parts.values())
+
+    def parts(self):
+        return dict(self._parts)
+
+    def forward(self, h, ctx, cache):
+        tokens = ctx.tokens
+        normed = ctx.workspace.first_rows("normed", self.width, self.dtype, tokens)
+        # (made cleared; every launch that folds it into the stream clears it again)
+        ctx.workspace.rows("sublayer_sum", self.width, torch.float32, cleared=True)
+        y = ctx.workspace.first_rows("sublayer_sum", self.width, torch.float32, tokens)
+        if ctx.extra is None:
+            ctx.extra = {}
+        add = ctx.extra.pop(_GATED_ADD, None)
+        for norm, part, gate, post in self.sublayers:
+            kernels.gated_norm_step(h, tokens, self.width, self.eps, add=add, norm=(norm.gamma, norm.beta, normed))
+            if part is self.mixer:
+                ridden = part.forward(normed, y, ctx, cache)
+            else:
+                ridden = part.forward(normed, y, ctx)
+            add = (y, ridden, gate.bias, post.gamma, post.beta)
+        ctx.extra[_GATED_ADD] = add
+        return h
+
+    def finish(self, h, ctx):
+        """Fold in what the block left (no block follows that would)."""
+        add = ctx.extra.pop(_GATED_ADD, None) if ctx.extra else None
+        if add is not None:
+            kernels.gated_norm_step(h, ctx.tokens, self.width, self.eps, add=add)
+
+
+@register_arrangement("gated_between_norms_mixer")
+class GatedBetweenNormsMixerBlock(GatedBetweenNormsBlock):
+    """The same with a mixer only."""
+
+    roles = {"norm1": "norm", "mixer": "mixer", "gate1": "connection", "post1": "norm"}

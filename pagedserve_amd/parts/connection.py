@@ -60,3 +60,22 @@ class ColumnScale(Part):
 
     def bind(self, tensors):
         self.weight = tensors["weight"]
+
+
+@register_connection("ridden_gate")
+class RiddenGate(Part):
+    """A gate ``sigmoid(W u + bias)`` per column on what a sublayer adds to the stream, ``u`` being the sublayer's own
+    input: the rows of ``W`` ride along in the sublayer's packed product (``ride``), which leaves the connection
+    the bias, ``bias [width]``, 32-bit."""
+
+    graph_safe = True
+
+    def __init__(self, width: int, dtype):
+        self.width = width
+        self.dtype = dtype
+
+    def parameters(self):
+        return {"bias": ParamSpec((self.width,), VECTOR)}
+
+    def bind(self, tensors):
+        self.bias = tensors["bias"]

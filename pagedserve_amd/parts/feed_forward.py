@@ -68,15 +68,17 @@ class GatedFeedForward(FeedForward):
     """``residual += W_down (act(W_gate x) * (W_up x))``, no biases; ``activation``: ``silu`` (with
     other constants of the gated unit as ``form = (limit, slope, shift)``: ``g' sigmoid(slope g') (u' +
     shift)`` of ``g' = min(W_gate x, limit)`` and ``u' = clamp(W_up x, -limit, limit)``) or
-    ``gelu_tanh``.  One packed product gives ``[gate | up]`` in float; the activation and the
+    ``gelu_tanh`` or ``relu``.  One packed product gives ``[gate | up]`` in float; the activation and the
     product of the halves are 32-bit.  ``forward(row_scale=...)``: a float per token that
-    multiplies its result."""
+    multiplies its result.  ``ride``: that many more rows of the packed product belong to the caller;
+    ``forward`` returns their float columns."""
 
     graph_safe = True
 
     accepts_pending_norm = True
 
-    def __init__(self, width: int, dtype, inner: int, activation: str = "silu", form=kernels.PLAIN_GATE):
+    def __init__(self, width: int, dtype, inner: int, activation: str = "silu", form=kernels.PLAIN_GATE,
+                 ride: int = 0):
         if activation not in kernels.GATE_ACTIVATIONS:
             raise ValueError(f"unknown gate activation {activation!r}; known: "
                              f"{', '.join(kernels.GATE_ACTIVATIONS)}")
@@ -85,11 +87,12 @@ class GatedFeedForward(FeedForward):
         self.inner = inner
         self.activation = activation
         self.form = tuple(float(value) for value in form)
+        self.ride = int(ride)
         self._memo_up, self._memo_down = {}, {}
 
     def parameters(self):
         return {
-            "gate_up.weight": ParamSpec((2 * self.inner, self.width), MATRIX),
+            "gate_up.weight": ParamSpec((2 * self.inner + self.ride, self.width), MATRIX),
             "down.weight": ParamSpec((self.width, self.inner), MATRIX),
         }
 
@@ -103,14 +106,16 @@ class GatedFeedForward(FeedForward):
 
     def forward(self, x, residual, ctx, row_scale=None):
         tokens = ctx.tokens
-        both = ctx.workspace.first_rows("ffn_gate_up", 2 * self.inner, torch.float32, tokens)
-        kernels.linear(x, self.gate_up_weight, None, both, packed=self.gate_up_packed,
+        whole, both, ridden = ctx.workspace.column_views("ffn_gate_up", 2 * self.inner + self.ride, torch.float32,
+                                                         tokens, (2 * self.inner, self.ride))
+        kernels.linear(x, self.gate_up_weight, None, whole, packed=self.gate_up_packed,
                        memo=site_memo(self._memo_up, ctx.workspace), shared=ctx.shared_calls)
         hidden = ctx.workspace.first_rows("ffn", self.inner, self.dtype, tokens)
         kernels.silu_gate(both, hidden, self.activation, form=self.form, row_scale=row_scale)
         kernels.linear(hidden, self.down_weight, None, residual, epilogue="residual",
                        packed=self.down_packed, memo=site_memo(self._memo_down, ctx.workspace),
                        shared=ctx.shared_calls)
+        return ridden if self.ride else None
 
 
 @register_feed_forward("moe")
