@@ -35,6 +35,7 @@ One JSON line is printed:
     python bench.py --design rezelix [--sizes small,medium,small_wide_heads]     Rezelix beside Zetunex at equal size
     python bench.py --design kozapel [--sizes small,medium,small_narrow_maps]    Kozapel beside Kosesun at equal size
     python bench.py --design malalix [--sizes small,medium,small_passed_twice,small_wide_heads]  Malalix beside Zetunex at equal size
+    python bench.py --design fadosun [--sizes small,medium,small_wide_heads]     Fadosun beside Zetunex at equal size
 
 ``--kernels`` times every kernel of a decode step (1, 8 and 64 requests over 1,024 keys), of
 the prefill step (2 x 1,024 tokens) and of a mixed step (32 decoded tokens beside a portion of
@@ -672,9 +673,41 @@ MALALIX_SIZES = {
     "small_wide_heads": (malalix_shape(768, 12, 6, 2, 128, 64, 3072, 50257, experts=16, top=4),
                          zetunex_shape(768, 12, 6, 2, 128, 3072, 50257, experts=16, top=4)),
 }
+
+
+def fadosun_shape(width, layers, heads, kv_heads, dim, ff, vocab, states=128, rank=None):
+    """A Fadosun configuration of a real model's layer sizes: in turn a delta-rule layer (four taps, low-rank
+    decays and gates), logistic attention with grouped heads (half of every head rotated) joined with a state
+    space twice the width (heads of 64, ``states`` states, one group), a matrix memory, and such a pair again;
+    every layer has a gated feed-forward."""
+    listed = []
+    for index in range(layers):
+        kind = ("channel_delta", "parallel", "mlstm", "parallel")[index % 4]
+        if kind == "channel_delta":
+            mixer = {"heads": heads, "kv_heads": heads, "dim": dim, "vdim": dim, "conv": 4,
+                     "decay_rank": rank or dim, "gate_rank": rank or dim}
+        elif kind == "mlstm":
+            mixer = {"heads": heads, "dim": dim, "vdim": dim, "gate_cap": 15.0}
+        else:
+            left = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+                    "rot": {"dims": dim // 2, "base": 500000.0}}
+            right = {"heads": 2 * width // 64, "vdim": 64, "state": states, "groups": 1, "conv": 4, "norm_groups": 1}
+            mixer = {"left": left, "right": right, "left_scale": 0.75, "right_scale": 1.25}
+        listed.append({"type": kind, "mixer": mixer, "mlp": {"kind": "dense", "ff": ff}})
+    return {"architecture": "Fadosun", "vocab": vocab, "width": width, "layers": listed, "norm": {"eps": 1e-6}}
+
+
+# name -> (Fadosun configuration, the Zetunex configuration of equal width, depth, heads and inner
+# width, with dense feed-forwards)
+FADOSUN_SIZES = {
+    "small": (fadosun_shape(768, 12, 12, 4, 64, 3072, 50257), _dense_zetunex(768, 12, 12, 4, 64, 3072, 50257)),
+    "medium": (fadosun_shape(1024, 24, 16, 4, 64, 4096, 50257), _dense_zetunex(1024, 24, 16, 4, 64, 4096, 50257)),
+    # heads of 128
+    "small_wide_heads": (fadosun_shape(768, 12, 6, 2, 128, 3072, 50257), _dense_zetunex(768, 12, 6, 2, 128, 3072, 50257)),
+}
 DESIGNS = {"kosesun": (("kosesun", "gpt2"), DESIGN_SIZES), "zetunex": (("zetunex", "kosesun"), ZETUNEX_SIZES),
            "rezelix": (("rezelix", "zetunex"), REZELIX_SIZES), "kozapel": (("kozapel", "kosesun"), KOZAPEL_SIZES),
-           "malalix": (("malalix", "zetunex"), MALALIX_SIZES)}
+           "malalix": (("malalix", "zetunex"), MALALIX_SIZES), "fadosun": (("fadosun", "zetunex"), FADOSUN_SIZES)}
 
 
 def design_comparison(args):

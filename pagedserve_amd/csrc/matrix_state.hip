@@ -24,15 +24,14 @@ __device__ inline float ms_sigmoid(float v) { return 1.0f / (1.0f + expf(-v)); }
 __device__ inline float ms_softplus(float v) { return fmaxf(v, 0.f) + log1pf(expf(-fabsf(v))); }
 
 // ---- short convolutions and what goes with them ------------------------------------------------
-// A wave per unit of a token.  Units of the convolution: the first `unit_heads` runs of `head`
+// A wave per unit of TT tokens.  Units of the convolution: the first `unit_heads` runs of `head`
 // channels each, whose activated values are made unit vectors (the first `scale_heads` of them are
-// also multiplied by q_scale), then runs of 256 of the other channels.  Then units of 256 decays.
-#define MS_UNIT 256
+// also multiplied by q_scale), then runs of 64 NR of the other channels.  Then units of 64 NR decays.
 struct PrepareArgs {
   const float* proj;
   int64_t ld;
   int col, channels, taps;
-  const float* w;          // [channels, taps], the last column is the current token's
+  const float* w;          // [taps, channels], the last row is the current token's
   const float* bias;       // [channels] or null
   const float* state;
   int64_t slot_stride;
@@ -52,73 +51,131 @@ struct PrepareArgs {
   const int* tok_item;
   const int* cu_tokens;
   const int* slots;
-  int conv_units, decay_units;
+  int conv_units, decay_units, tokens;
 };
 
+template <int NR, int TT>
 __global__ __launch_bounds__(256) void state_prepare_kernel(const PrepareArgs p) {
-  const int t = blockIdx.x;
+  const int t0 = blockIdx.x * TT;
+  const int many = p.tokens - t0 < TT ? p.tokens - t0 : TT;
   const int lane = threadIdx.x & 63;
-  const int unit = blockIdx.y * 4 + (threadIdx.x >> 6);
+  const int unit = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   if (unit >= p.conv_units + p.decay_units) return;
-  const float* row = p.proj + (int64_t)t * p.ld;
   if (unit >= p.conv_units) {
-    const int first = (unit - p.conv_units) * MS_UNIT;
+    const int first = (unit - p.conv_units) * 64 * NR;
     const int count = p.rule == PS_STATE_DELTA ? p.heads * p.per_head : p.heads;
+    for (int tt = 0; tt < many; ++tt) {
+      const int64_t t = t0 + tt;
+      const float* row = p.proj + t * p.ld;
 #pragma unroll
-    for (int j = 0; j < MS_UNIT / 64; ++j) {
-      const int c = first + j * 64 + lane;
-      if (c < p.heads) {
-        const float raw = row[p.take_col + c];
-        if (p.rule == PS_STATE_DELTA) {
-          p.take[(int64_t)t * p.heads + c] = ms_sigmoid(raw);
-        } else {
-          const float dt = ms_softplus(raw + p.z_bias[c]);
-          p.take[(int64_t)t * p.heads + c] = dt;
-          p.decay[(int64_t)t * p.heads + c] = -expf(p.a_log[c]) * dt;
+      for (int j = 0; j < NR; ++j) {
+        const int c = first + j * 64 + lane;
+        if (c < p.heads) {
+          const float raw = row[p.take_col + c];
+          if (p.rule == PS_STATE_DELTA) {
+            p.take[t * p.heads + c] = ms_sigmoid(raw);
+          } else {
+            const float dt = ms_softplus(raw + p.z_bias[c]);
+            p.take[t * p.heads + c] = dt;
+            p.decay[t * p.heads + c] = -expf(p.a_log[c]) * dt;
+          }
         }
-      }
-      if (p.rule == PS_STATE_DELTA && c < count) {
-        const float step = ms_softplus(p.z[(int64_t)t * p.z_ld + c] + p.z_bias[c]);
-        p.decay[(int64_t)t * count + c] = expf(-expf(p.a_log[c / p.per_head]) * step);
+        if (p.rule == PS_STATE_DELTA && c < count) {
+          const float step = ms_softplus(p.z[t * p.z_ld + c] + p.z_bias[c]);
+          p.decay[t * count + c] = expf(-expf(p.a_log[c / p.per_head]) * step);
+        }
       }
     }
     return;
   }
   const bool normed = unit < p.unit_heads;
-  const int c0 = normed ? unit * p.head : p.unit_heads * p.head + (unit - p.unit_heads) * MS_UNIT;
-  const int most = normed ? p.head : MS_UNIT;
+  const int c0 = normed ? unit * p.head : p.unit_heads * p.head + (unit - p.unit_heads) * 64 * NR;
+  const int most = normed ? p.head : 64 * NR;
   const int count = p.channels - c0 < most ? p.channels - c0 : most;
-  const int item = p.tok_item[t];
+  const int item = p.tok_item[t0];
   const int first = p.cu_tokens[item];
-  const float* kept = p.state + p.slots[item] * p.slot_stride + p.history;
-  float value[4], squares = 0.f;
+  float value[TT][NR];
+  // every load below is unconditional, from the last channel where a lane has none
+  if (TT > 1 && many == TT && p.taps <= 4 && t0 - first >= p.taps - 1 && t0 + TT <= p.cu_tokens[item + 1]) {
+    // all inputs are of this step and this item: each is loaded once for the tokens that see it
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int d = j * 64 + lane;
-    value[j] = 0.f;
-    if (d < count) {
-      const int c = c0 + d;
-      float sum = p.bias ? p.bias[c] : 0.f;
-      for (int tap = 0; tap < p.taps; ++tap) {
-        const int back = p.taps - 1 - tap;          // the input `back` tokens before this one
-        const int local = (t - first) - back;       // its place among the item's tokens of this step
-        const float u = local >= 0 ? row[p.col + c - (int64_t)back * p.ld]
-                                   : kept[(int64_t)(p.taps - 1 + local) * p.channels + c];
-        sum = fmaf(p.w[(int64_t)c * p.taps + tap], u, sum);
+    for (int j = 0; j < NR; ++j) {
+      const int c = c0 + (j * 64 + lane < count ? j * 64 + lane : count - 1);
+      float x[TT + 3], w[4];
+#pragma unroll
+      for (int i = 0; i < TT + 3; ++i) {
+        const int t = t0 - 3 + i > 0 ? t0 - 3 + i : 0;
+        x[i] = p.proj[(int64_t)t * p.ld + p.col + c];
       }
-      value[j] = ms_silu(sum);
+#pragma unroll
+      for (int back = 0; back < 4; ++back)
+        w[back] = back < p.taps ? p.w[(int64_t)(p.taps - 1 - back) * p.channels + c] : 0.f;
+      const float start = p.bias ? p.bias[c] : 0.f;
+#pragma unroll
+      for (int tt = 0; tt < TT; ++tt) {
+        float sum = start;
+#pragma unroll
+        for (int back = 3; back >= 0; --back) sum = back < p.taps ? fmaf(w[back], x[tt + 3 - back], sum) : sum;
+        value[tt][j] = ms_silu(sum);
+      }
     }
-    squares = fmaf(value[j], value[j], squares);
-  }
-  float factor = 1.f;
-  if (normed) {
-    factor = 1.0f / sqrtf(wave_sum(squares) + 1e-6f);
-    if (unit < p.scale_heads) factor *= p.q_scale;
+  } else {
+#pragma unroll
+    for (int tt = 0; tt < TT; ++tt) {
+      const int t = tt < many ? t0 + tt : t0;
+      const int it = TT > 1 ? p.tok_item[t] : item;
+      const int begin = TT > 1 ? p.cu_tokens[it] : first;
+      const float* kept = p.state + p.slots[it] * p.slot_stride + p.history;
+      const float* row = p.proj + (int64_t)t * p.ld + p.col;
+      float sum[NR];
+#pragma unroll
+      for (int j = 0; j < NR; ++j)
+        sum[j] = p.bias ? p.bias[c0 + (j * 64 + lane < count ? j * 64 + lane : count - 1)] : 0.f;
+      for (int tap0 = 0; tap0 < p.taps; tap0 += 4) {
+        float x[4][NR], w[4][NR];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int tap = tap0 + i < p.taps ? tap0 + i : p.taps - 1;
+          const int back = p.taps - 1 - tap;          // the input `back` tokens before this one
+          const int local = (t - begin) - back;       // its place among the item's tokens of this step
+          const float* from = local >= 0 ? row - (int64_t)back * p.ld
+                                         : kept + (int64_t)(p.taps - 1 + local) * p.channels;
+#pragma unroll
+          for (int j = 0; j < NR; ++j) {
+            const int c = c0 + (j * 64 + lane < count ? j * 64 + lane : count - 1);
+            x[i][j] = from[c];
+            w[i][j] = p.w[(int64_t)tap * p.channels + c];
+          }
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+#pragma unroll
+          for (int j = 0; j < NR; ++j)
+            if (tap0 + i < p.taps) sum[j] = fmaf(w[i][j], x[i][j], sum[j]);
+      }
+#pragma unroll
+      for (int j = 0; j < NR; ++j) value[tt][j] = ms_silu(sum[j]);
+    }
   }
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const int d = j * 64 + lane;
-    if (d < count) p.out[(int64_t)t * p.channels + c0 + d] = value[j] * factor;
+  for (int tt = 0; tt < TT; ++tt) {
+    if (tt >= many) break;
+    float factor = 1.f;
+    if (normed) {
+      float squares = 0.f;
+#pragma unroll
+      for (int j = 0; j < NR; ++j) {
+        const float v = j * 64 + lane < count ? value[tt][j] : 0.f;
+        squares = fmaf(v, v, squares);
+      }
+      factor = 1.0f / sqrtf(wave_sum(squares) + 1e-6f);
+      if (unit < p.scale_heads) factor *= p.q_scale;
+    }
+#pragma unroll
+    for (int j = 0; j < NR; ++j) {
+      const int d = j * 64 + lane;
+      if (d < count) p.out[(int64_t)(t0 + tt) * p.channels + c0 + d] = value[tt][j] * factor;
+    }
   }
 }
 
@@ -133,21 +190,37 @@ extern "C" int ps_state_prepare(const float* proj, int64_t ld, int col, int chan
   PS_REQUIRE(tokens >= 0 && channels > 0 && taps >= 1 && taps <= 64 && heads > 0 && per_head > 0,
              "ps_state_prepare: bad sizes");
   PS_REQUIRE(unit_heads >= 0 && (int64_t)unit_heads * head <= channels && scale_heads <= unit_heads &&
-                 (unit_heads == 0 || (head > 0 && head <= MS_UNIT)),
-             "ps_state_prepare: %d heads of %d do not fit %d channels (heads of up to %d)", unit_heads, head,
-             channels, MS_UNIT);
+                 (unit_heads == 0 || (head > 0 && head <= 256)),
+             "ps_state_prepare: %d heads of %d do not fit %d channels (heads of up to 256)", unit_heads, head,
+             channels);
   PS_REQUIRE(rule == PS_STATE_DECAYED || (rule == PS_STATE_DELTA && z != nullptr),
              "ps_state_prepare: rule %d", rule);
   if (tokens == 0) return 0;
   PrepareArgs p = {proj, ld, col, channels, taps, w, bias, state, slot_stride, history, out, unit_heads,
                    head, scale_heads, q_scale, rule, heads, per_head, z, z_ld, z_bias, a_log, take_col,
-                   decay, take, tok_item, cu_tokens, slots, 0, 0};
-  p.conv_units = unit_heads + (channels - unit_heads * head + MS_UNIT - 1) / MS_UNIT;
+                   decay, take, tok_item, cu_tokens, slots, 0, 0, tokens};
+  // few tokens: as many waves as there are runs of 64 channels; many: several tokens to a wave, which
+  // share their inputs
+  const bool few = tokens <= 64;
+  const int nr = unit_heads > 0 ? (head <= 64 ? 1 : (head <= 128 ? 2 : 4)) : (few ? 1 : 2);
+  p.conv_units = unit_heads + (channels - unit_heads * head + 64 * nr - 1) / (64 * nr);
   const int decays = rule == PS_STATE_DELTA ? heads * per_head : heads;
-  p.decay_units = (decays + MS_UNIT - 1) / MS_UNIT;
+  p.decay_units = (decays + 64 * nr - 1) / (64 * nr);
   const int units = p.conv_units + p.decay_units;
   PS_REQUIRE((units + 3) / 4 <= 65535, "ps_state_prepare: too many channels");
-  hipLaunchKernelGGL(state_prepare_kernel, dim3(tokens, (units + 3) / 4), dim3(256), 0, (hipStream_t)stream, p);
+#define PS_LAUNCH_PREP(NR, TT)                                                                          \
+  hipLaunchKernelGGL((state_prepare_kernel<NR, TT>), dim3((tokens + TT - 1) / TT, (units + 3) / 4),     \
+                     dim3(256), 0, (hipStream_t)stream, p)
+#define PS_LAUNCH_PREP_T(NR)              \
+  do {                                    \
+    if (few) PS_LAUNCH_PREP(NR, 1);       \
+    else PS_LAUNCH_PREP(NR, 8);           \
+  } while (0)
+  if (nr == 1) PS_LAUNCH_PREP_T(1);
+  else if (nr == 2) PS_LAUNCH_PREP_T(2);
+  else PS_LAUNCH_PREP_T(4);
+#undef PS_LAUNCH_PREP_T
+#undef PS_LAUNCH_PREP
   PS_CHECK_LAUNCH("ps_state_prepare");
   return 0;
 }
@@ -223,22 +296,53 @@ extern "C" int ps_memory_gates(const float* proj, int64_t ld, int i_col, int f_c
 // A block of four waves owns 4 COLS columns of one head's state for one item.  Within a wave, lane =
 // column * GROUPS + row group; a lane keeps RPL neighbouring key rows of its column in registers, and
 // the sums over the row groups run over neighbouring lanes.  Keys, queries, decays and values of
-// MS_CHUNK tokens wait in LDS for all four waves; the next chunk's loads travel while this one is
-// worked on.
+// CHUNK tokens wait in LDS for all four waves; the next chunk's loads travel while this one is
+// worked on.  The chain from token to token is what bounds a long portion, and one wave has a SIMD to
+// itself, so nothing may stand between two tokens: a chunk's tokens are one straight run of
+// instructions (places behind the item's last token decay by one and add nothing), and the lanes'
+// shares of the outputs stay in registers until they are summed for GROUPS tokens at once.
+
+// values[i] of every lane of an aligned group of N = the share of token i; returns the sum over the
+// group's lanes of token (lane % N).  Every step halves the tokens a lane still cares for.
+template <int N>
+__device__ inline float sum_transposed(float (&values)[N], int lane) {
+  float v[N];
+#pragma unroll
+  for (int i = 0; i < N; ++i) v[i] = values[i];
+  // a lane keeps the tokens whose bit is its own and takes its partner's share of them (the partner: the
+  // mirrored lane of 16 or 8, then the lane with that bit turned)
+  auto halve = [&](auto exchange, const int half) {
+    const bool upper = (lane & half) != 0;
+#pragma unroll
+    for (int i = 0; i < N / 2; ++i) {
+      if (i < half) {
+        const float keep = upper ? v[i + half] : v[i];
+        const float give = upper ? v[i] : v[i + half];
+        v[i] = keep + exchange(give);
+      }
+    }
+  };
+  if constexpr (N >= 16) halve([](float x) { return lane_exchange<0x140>(x); }, 8);
+  if constexpr (N >= 8) halve([](float x) { return lane_exchange<0x141>(x); }, 4);
+  if constexpr (N >= 4) halve([](float x) { return lane_exchange<0x4E>(x); }, 2);
+  halve([](float x) { return lane_exchange<0xB1>(x); }, 1);
+  return v[0];
+}
 
 template <int RPL, int GROUPS, int CHUNK, bool DELTA>
-__global__ __launch_bounds__(256) void state_walk_kernel(const StateStep p) {
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) void state_walk_kernel(const StateStep p) {
   constexpr int COLS = 64 / GROUPS;                // columns of a wave
   constexpr int BLOCK_COLS = 4 * COLS;
   constexpr int ROWS = GROUPS * RPL;               // key rows with padding up to the lanes' share
   constexpr int PAD = RPL < 4 ? 4 : RPL + 4;       // row groups start in different banks
   constexpr int PER = (CHUNK * ROWS + 255) / 256;  // values of a chunk per thread and array
   constexpr int PER_V = (CHUNK * BLOCK_COLS + 255) / 256;
+  constexpr int RUN = CHUNK < GROUPS ? CHUNK : GROUPS;   // tokens whose outputs are summed together
+  static_assert(CHUNK == 1 || CHUNK % GROUPS == 0, "whole runs of tokens, or one token");
   __shared__ __attribute__((aligned(16))) float s_q[CHUNK][GROUPS * PAD];
   __shared__ __attribute__((aligned(16))) float s_k[CHUNK][GROUPS * PAD];
   __shared__ __attribute__((aligned(16))) float s_a[DELTA ? CHUNK : 1][GROUPS * PAD];
   __shared__ float s_v[CHUNK][BLOCK_COLS];
-  __shared__ float s_o[CHUNK][BLOCK_COLS];
   __shared__ float s_d[CHUNK], s_w[CHUNK];
   const int item = blockIdx.x, head = blockIdx.y;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -258,6 +362,87 @@ __global__ __launch_bounds__(256) void state_walk_kernel(const StateStep p) {
   const float* v_base = p.v + head * p.value_dim;
   const float* a_base = DELTA ? p.decay + (int64_t)head * p.key_dim : nullptr;
   const int64_t a_ld = (int64_t)p.heads * p.key_dim;
+  // a chunk on its way from memory; two of them travel at a time (a chunk's work is shorter than a trip)
+  struct Coming {
+    float q[PER], k[PER], a[DELTA ? PER : 1], v[PER_V], d, w;
+  };
+  Coming even, odd;
+  // A thread's places within a chunk are the same in every chunk: their distances from the chunk's first
+  // row are worked out once, and a chunk's loads are a scalar address and such a distance each.
+  int place_tt[PER], place_at[PER], off_q[PER], off_k[PER], off_a[DELTA ? PER : 1], col_q[PER];
+  bool place_row[PER];
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int idx = tid + j * 256;
+    const int tt = idx / ROWS;
+    const int r = idx - tt * ROWS;
+    place_tt[j] = tt;
+    place_at[j] = tt * (GROUPS * PAD) + (r / RPL) * PAD + (r % RPL);
+    place_row[j] = r < p.key_dim;
+    col_q[j] = r < p.key_dim ? r : 0;
+    off_q[j] = tt * (int)p.q_ld + col_q[j];
+    off_k[j] = tt * (int)p.k_ld + col_q[j];
+    if (DELTA) off_a[j] = tt * (int)a_ld + col_q[j];
+  }
+  int v_tt[PER_V], v_at[PER_V], off_v[PER_V];
+  float v_factor[PER_V], v_add[PER_V];
+#pragma unroll
+  for (int j = 0; j < PER_V; ++j) {
+    const int idx = tid + j * 256;
+    v_tt[j] = idx / BLOCK_COLS;
+    const int c = col0 + (idx - v_tt[j] * BLOCK_COLS);
+    v_at[j] = c < p.value_dim ? c : 0;
+    off_v[j] = v_tt[j] * (int)p.v_ld + v_at[j];
+    // (the column behind the values sums the keys alone: its value is one)
+    v_factor[j] = c < p.value_dim ? 1.f : 0.f;
+    v_add[j] = p.ones && c == p.value_dim ? 1.f : 0.f;
+  }
+  // every load is unconditional (from the chunk's first row where the item has no such token); what lies
+  // outside is masked when stored
+  auto fetch = [&](Coming& in, const int base) {
+    if (base >= t1) return;
+    const int count = (t1 - base) < CHUNK ? (t1 - base) : CHUNK;
+    const float* q_row = q_base + (int64_t)base * p.q_ld;
+    const float* k_row = k_base + (int64_t)base * p.k_ld;
+    const float* a_row = DELTA ? a_base + (int64_t)base * a_ld : nullptr;
+    const float* v_row = v_base + (int64_t)base * p.v_ld;
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const bool there = place_tt[j] < count;
+      in.q[j] = q_row[there ? off_q[j] : col_q[j]];
+      in.k[j] = k_row[there ? off_k[j] : col_q[j]];
+      if (DELTA) in.a[j] = a_row[there ? off_a[j] : col_q[j]];
+    }
+#pragma unroll
+    for (int j = 0; j < PER_V; ++j) in.v[j] = v_row[v_tt[j] < count ? off_v[j] : v_at[j]];
+    if (tid < CHUNK) {
+      const int64_t at = (int64_t)(base + (tid < count ? tid : 0)) * p.heads + head;
+      in.w = p.take[at];
+      if (!DELTA) in.d = p.decay[at];
+    }
+  };
+  auto stash = [&](const Coming& in, const int base) {
+    const int count = (t1 - base) < CHUNK ? (t1 - base) : CHUNK;
+#pragma unroll
+    for (int j = 0; j < PER; ++j) {
+      const bool valid = place_tt[j] < count && place_row[j];
+      if (CHUNK * ROWS % 256 == 0 || place_tt[j] < CHUNK) {
+        (&s_q[0][0])[place_at[j]] = valid ? in.q[j] * p.q_scale : 0.f;
+        (&s_k[0][0])[place_at[j]] = valid ? in.k[j] : 0.f;
+        if (DELTA) (&s_a[0][0])[place_at[j]] = valid ? in.a[j] : 1.f;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < PER_V; ++j)
+      if (CHUNK * BLOCK_COLS % 256 == 0 || v_tt[j] < CHUNK)
+        (&s_v[0][0])[tid + j * 256] = v_tt[j] < count ? fmaf(in.v[j], v_factor[j], v_add[j]) : 0.f;
+    if (tid < CHUNK) {
+      s_w[tid] = tid < count ? in.w : 0.f;
+      s_d[tid] = DELTA || tid >= count ? 1.f : expf(in.d);
+    }
+  };
+  fetch(even, t0);
+  fetch(odd, t0 + CHUNK);
   float S[RPL];
   const int rows_mine = p.key_dim - group * RPL;   // key rows from the lane's first on
   const bool whole = RPL % 4 == 0 && p.key_dim % 4 == 0 && p.aligned;
@@ -267,128 +452,94 @@ __global__ __launch_bounds__(256) void state_walk_kernel(const StateStep p) {
       float4 four = make_float4(0.f, 0.f, 0.f, 0.f);
       if (i < rows_mine && has_col) four = *reinterpret_cast<const float4*>(s_ptr + i);
       S[i] = four.x;
-      if (RPL >= 4) {
-        S[(i + 1) % RPL] = four.y;
-        S[(i + 2) % RPL] = four.z;
-        S[(i + 3) % RPL] = four.w;
-      }
+      S[(i + 1) % RPL] = four.y;
+      S[(i + 2) % RPL] = four.z;
+      S[(i + 3) % RPL] = four.w;
     }
   } else {
 #pragma unroll
     for (int i = 0; i < RPL; ++i) S[i] = (i < rows_mine && has_col) ? s_ptr[i] : 0.f;
   }
-  float rq[PER], rk[PER], ra[DELTA ? PER : 1], rv[PER_V], rd = 0.f, rw = 0.f;
-  // every load is unconditional from a clamped address; what lies outside is masked when stored
-  auto fetch = [&](const int base) {
-    const int count = (t1 - base) < CHUNK ? (t1 - base) : CHUNK;
-#pragma unroll
-    for (int j = 0; j < PER; ++j) {
-      const int idx = tid + j * 256;
-      const int tt = idx / ROWS;
-      const int r = idx - tt * ROWS;
-      const int64_t t = base + (tt < count ? tt : 0);
-      const int c = r < p.key_dim ? r : 0;
-      rq[j] = q_base[t * p.q_ld + c];
-      rk[j] = k_base[t * p.k_ld + c];
-      if (DELTA) ra[j] = a_base[t * a_ld + c];
-    }
-#pragma unroll
-    for (int j = 0; j < PER_V; ++j) {
-      const int idx = tid + j * 256;
-      const int tt = idx / BLOCK_COLS;
-      const int c = col0 + (idx - tt * BLOCK_COLS);
-      const int64_t t = base + (tt < count ? tt : 0);
-      rv[j] = v_base[t * p.v_ld + (c < p.value_dim ? c : 0)];
-    }
-    if (tid < CHUNK) {
-      const int64_t at = (int64_t)(base + (tid < count ? tid : 0)) * p.heads + head;
-      rw = p.take[at];
-      if (!DELTA) rd = p.decay[at];
-    }
-  };
-  auto stash = [&](const int base) {
-    const int count = (t1 - base) < CHUNK ? (t1 - base) : CHUNK;
-#pragma unroll
-    for (int j = 0; j < PER; ++j) {
-      const int idx = tid + j * 256;
-      const int tt = idx / ROWS;
-      const int r = idx - tt * ROWS;
-      const bool valid = tt < count && r < p.key_dim;
-      const int at = (r / RPL) * PAD + (r % RPL);
-      if (CHUNK * ROWS % 256 == 0 || tt < CHUNK) {
-        s_q[tt][at] = valid ? rq[j] * p.q_scale : 0.f;
-        s_k[tt][at] = valid ? rk[j] : 0.f;
-        if (DELTA) s_a[tt][at] = valid ? ra[j] : 0.f;
-      }
-    }
-#pragma unroll
-    for (int j = 0; j < PER_V; ++j) {
-      const int idx = tid + j * 256;
-      const int tt = idx / BLOCK_COLS;
-      if (CHUNK * BLOCK_COLS % 256 == 0 || tt < CHUNK) {
-        const int c = col0 + (idx - tt * BLOCK_COLS);
-        // (the column behind the values sums the keys alone: its value is one)
-        const float v = c < p.value_dim ? rv[j] : (p.ones && c == p.value_dim ? 1.f : 0.f);
-        s_v[tt][idx - tt * BLOCK_COLS] = tt < count ? v : 0.f;
-      }
-    }
-    if (tid < CHUNK) {
-      s_w[tid] = rw;
-      s_d[tid] = DELTA ? 0.f : expf(rd);
-    }
-  };
-  fetch(t0);
-  for (int base = t0; base < t1; base += CHUNK) {
-    const int count = (t1 - base) < CHUNK ? (t1 - base) : CHUNK;
+  const int out_ld = p.heads * columns;
+  auto work = [&](Coming& in, const int base) {
     __syncthreads();      // the chunk before has been read
-    stash(base);
+    stash(in, base);
     __syncthreads();
-    if (base + CHUNK < t1) fetch(base + CHUNK);   // in flight during the work below
-    auto token = [&](const int tt) {
-      const float* kr = &s_k[tt][group * PAD];
-      const float* qr = &s_q[tt][group * PAD];
-      float v = s_v[tt][mine];
-      const float w = s_w[tt];
+    fetch(in, base + 2 * CHUNK);
+    // what a token's step reads from LDS, into registers
+    struct Operands {
+      float q[RPL], k[RPL], a[DELTA ? RPL : 1], v, w, d;
+    };
+    auto load = [&](const int tt, Operands& in) {
+#pragma unroll
+      for (int i = 0; i < RPL; i += 4) {
+        *reinterpret_cast<float4*>(&in.k[i]) = *reinterpret_cast<const float4*>(&s_k[tt][group * PAD + i]);
+        if (DELTA)
+          *reinterpret_cast<float4*>(&in.a[i % (DELTA ? RPL : 1)]) = *reinterpret_cast<const float4*>(&s_a[tt][group * PAD + i]);
+        *reinterpret_cast<float4*>(&in.q[i]) = *reinterpret_cast<const float4*>(&s_q[tt][group * PAD + i]);
+      }
+      in.v = s_v[tt][mine];
+      in.w = s_w[tt];
+      in.d = DELTA ? 1.f : s_d[tt];
+    };
+    // the lane's share of a token's output
+    auto token = [&](const Operands& in) -> float {
+      float v = in.v;
       if (DELTA) {
-        const float* ar = &s_a[tt][group * PAD];
         float dot0 = 0.f, dot1 = 0.f;
 #pragma unroll
         for (int i = 0; i < RPL; ++i) {
-          S[i] *= ar[i];
-          if (i & 1) dot1 = fmaf(S[i], kr[i], dot1);
-          else dot0 = fmaf(S[i], kr[i], dot0);
+          S[i] *= in.a[i % (DELTA ? RPL : 1)];
+          if (i & 1) dot1 = fmaf(S[i], in.k[i], dot1);
+          else dot0 = fmaf(S[i], in.k[i], dot0);
         }
-        v = w * (v - lanes_sum<GROUPS>(dot0 + dot1));
+        v = in.w * (v - lanes_sum<GROUPS>(dot0 + dot1));
       } else {
-        const float d = s_d[tt];
-        v *= w;
+        v *= in.w;
 #pragma unroll
-        for (int i = 0; i < RPL; ++i) S[i] *= d;
+        for (int i = 0; i < RPL; ++i) S[i] *= in.d;
       }
       float o0 = 0.f, o1 = 0.f;
 #pragma unroll
       for (int i = 0; i < RPL; ++i) {
-        S[i] = fmaf(kr[i], v, S[i]);
-        if (i & 1) o1 = fmaf(S[i], qr[i], o1);
-        else o0 = fmaf(S[i], qr[i], o0);
+        S[i] = fmaf(in.k[i], v, S[i]);
+        if (i & 1) o1 = fmaf(S[i], in.q[i], o1);
+        else o0 = fmaf(S[i], in.q[i], o0);
       }
-      const float o = lanes_sum<GROUPS>(o0 + o1);
-      if (group == 0) s_o[tt][mine] = o;
+      return o0 + o1;
     };
-    if (count == CHUNK) {
-      // a whole chunk: unrolled, so that the reads of the next tokens run ahead of the chain
-#pragma unroll
-      for (int tt = 0; tt < CHUNK; ++tt) token(tt);
+    if constexpr (CHUNK == 1) {
+      Operands in;
+      load(0, in);
+      const float o = lanes_sum<GROUPS>(token(in));
+      if (group == 0 && has_col) p.out[((int64_t)base * p.heads + head) * columns + col] = o;
     } else {
-      for (int tt = 0; tt < count; ++tt) token(tt);
+      // the reads of the next tokens are on their way while a token is worked on: the barriers keep the
+      // compiler from moving them down to where they are used
+      constexpr int AHEAD = RPL > 8 ? 1 : 2;
+      Operands in[AHEAD + 1];
+#pragma unroll
+      for (int i = 0; i < AHEAD; ++i) load(i, in[i]);
+#pragma unroll
+      for (int run = 0; run < CHUNK; run += RUN) {
+        float shares[GROUPS];
+#pragma unroll
+        for (int i = 0; i < GROUPS; ++i) {
+          const int tt = run + i;
+          if (tt + AHEAD < CHUNK) load(tt + AHEAD, in[(tt + AHEAD) % (AHEAD + 1)]);
+          __builtin_amdgcn_sched_barrier(0);
+          shares[i] = token(in[tt % (AHEAD + 1)]);
+          __builtin_amdgcn_sched_barrier(0);
+        }
+        const float o = sum_transposed<GROUPS>(shares, lane);
+        if (base + run + group < t1 && has_col)
+          (p.out + (int64_t)(base + run) * out_ld + head * columns)[group * out_ld + col] = o;
+      }
     }
-    __syncthreads();
-    for (int idx = tid; idx < count * BLOCK_COLS; idx += 256) {
-      const int tt = idx / BLOCK_COLS;
-      const int c = idx - tt * BLOCK_COLS;
-      if (col0 + c < columns)
-        p.out[((int64_t)(base + tt) * p.heads + head) * columns + col0 + c] = s_o[tt][c];
-    }
+  };
+  for (int base = t0; base < t1; base += 2 * CHUNK) {
+    work(even, base);
+    if (base + CHUNK < t1) work(odd, base + CHUNK);
   }
   if (has_col) {
     if (whole) {
@@ -432,18 +583,18 @@ extern "C" int ps_state_scan(const float* q, int64_t q_ld, const float* k, int64
 #define PS_LAUNCH_WALK(RPL, GROUPS, CHUNK)                  \
   do {                                                      \
     if (rule == PS_STATE_DELTA) {                           \
-      if (brief) PS_LAUNCH_WALK_D(RPL, GROUPS, 2, true);    \
+      if (brief) PS_LAUNCH_WALK_D(RPL, GROUPS, 1, true);    \
       else PS_LAUNCH_WALK_D(RPL, GROUPS, CHUNK, true);      \
     } else {                                                \
-      if (brief) PS_LAUNCH_WALK_D(RPL, GROUPS, 2, false);   \
+      if (brief) PS_LAUNCH_WALK_D(RPL, GROUPS, 1, false);   \
       else PS_LAUNCH_WALK_D(RPL, GROUPS, CHUNK, false);     \
     }                                                       \
   } while (0)
-  if (key_dim <= 16) PS_LAUNCH_WALK(4, 4, 32);
-  else if (key_dim <= 32) PS_LAUNCH_WALK(4, 8, 32);
-  else if (key_dim <= 64) PS_LAUNCH_WALK(4, 16, 32);
+  if (key_dim <= 16) PS_LAUNCH_WALK(4, 4, 16);
+  else if (key_dim <= 32) PS_LAUNCH_WALK(4, 8, 16);
+  else if (key_dim <= 64) PS_LAUNCH_WALK(4, 16, 16);
   else if (key_dim <= 128) PS_LAUNCH_WALK(8, 16, 16);
-  else PS_LAUNCH_WALK(16, 16, 8);
+  else PS_LAUNCH_WALK(16, 16, 16);
 #undef PS_LAUNCH_WALK
 #undef PS_LAUNCH_WALK_D
   PS_CHECK_LAUNCH("ps_state_scan");
@@ -475,18 +626,9 @@ struct OutputArgs {
   int tokens;
 };
 
-__device__ inline float state_output_value(const OutputArgs& p, int64_t t, int c) {
-  const int h = c / p.value_dim;
-  const int64_t head_row = (t * p.heads + h) * (p.value_dim + p.ones);
-  float x = p.o[head_row + (c - h * p.value_dim)];
-  if (p.skip != nullptr) x = fmaf(p.skip[h], p.u[t * p.u_ld + c], x);
-  if (p.ones) x /= fmaxf(fabsf(p.o[head_row + p.value_dim]), p.floor[t * p.heads + h]) + 1e-6f;
-  if (p.before != nullptr) x *= ms_silu(p.before[t * p.before_ld + c]);
-  return x;
-}
-
-#define MS_HELD 8
-template <typename T, int LANES>
+// A thread's share of its group: HELD columns, every load of which leaves before any is used (from the
+// group's last column where a thread has none).
+template <typename T, int LANES, int HELD>
 __global__ __launch_bounds__(256) void state_output_kernel(const OutputArgs p, T* __restrict__ out) {
   __shared__ float scratch[16];
   const int groups = p.heads * p.value_dim / p.group;
@@ -495,29 +637,49 @@ __global__ __launch_bounds__(256) void state_output_kernel(const OutputArgs p, T
   if (index >= (int64_t)p.tokens * groups) return;     // (whole waves, or the whole block)
   const int64_t t = index / groups;
   const int c0 = (int)(index - t * groups) * p.group;
-  float held[MS_HELD], squares = 0.f;
+  const float per_head = 1.0f / (float)p.value_dim;
+  const bool shared_weight = p.weight_count == p.value_dim;
+  float x[HELD], u[HELD], skip[HELD], sum[HELD], floor_of[HELD], before[HELD], behind[HELD], weight[HELD];
 #pragma unroll
-  for (int j = 0; j < MS_HELD; ++j) {
+  for (int j = 0; j < HELD; ++j) {
     const int d = lane + LANES * j;
-    held[j] = d < p.group ? state_output_value(p, t, c0 + d) : 0.f;
-    squares = fmaf(held[j], held[j], squares);
+    const int c = c0 + (d < p.group ? d : p.group - 1);
+    const int h = (int)(((float)c + 0.5f) * per_head);   // c / value_dim (columns are far fewer than 2^20)
+    const int64_t row = (t * p.heads + h) * (p.value_dim + p.ones);
+    x[j] = p.o[row + (c - h * p.value_dim)];
+    weight[j] = p.weight[shared_weight ? c - h * p.value_dim : c];
+    u[j] = skip[j] = before[j] = behind[j] = 0.f;
+    sum[j] = floor_of[j] = 1.f;
+    if (p.skip != nullptr) {
+      u[j] = p.u[t * p.u_ld + c];
+      skip[j] = p.skip[h];
+    }
+    if (p.ones) {
+      sum[j] = p.o[row + p.value_dim];
+      floor_of[j] = p.floor[t * p.heads + h];
+    }
+    if (p.before != nullptr) before[j] = p.before[t * p.before_ld + c];
+    if (p.behind != nullptr) behind[j] = p.behind[t * p.behind_ld + c];
   }
-  for (int d = lane + LANES * MS_HELD; d < p.group; d += LANES) {
-    const float x = state_output_value(p, t, c0 + d);
-    squares = fmaf(x, x, squares);
+  float squares = 0.f;
+#pragma unroll
+  for (int j = 0; j < HELD; ++j) {
+    x[j] = fmaf(skip[j], u[j], x[j]);
+    if (p.ones) x[j] /= fmaxf(fabsf(sum[j]), floor_of[j]) + 1e-6f;
+    if (p.before != nullptr) x[j] *= ms_silu(before[j]);
+    if (lane + LANES * j < p.group) squares = fmaf(x[j], x[j], squares);
   }
   const float total = LANES == 64 ? wave_sum(squares) : block_sum(squares, scratch);
   const float inv = 1.0f / sqrtf(total / (float)p.group + p.eps);
-  auto store = [&](const int d, float x) {
-    const int c = c0 + d;
-    x *= inv * p.weight[c % p.weight_count];
-    if (p.behind != nullptr) x *= ms_sigmoid(p.behind[t * p.behind_ld + c]);
-    out[t * p.out_ld + c] = from_float<T>(x);
-  };
 #pragma unroll
-  for (int j = 0; j < MS_HELD; ++j)
-    if (lane + LANES * j < p.group) store(lane + LANES * j, held[j]);
-  for (int d = lane + LANES * MS_HELD; d < p.group; d += LANES) store(d, state_output_value(p, t, c0 + d));
+  for (int j = 0; j < HELD; ++j) {
+    const int d = lane + LANES * j;
+    if (d < p.group) {
+      float v = x[j] * (inv * weight[j]);
+      if (p.behind != nullptr) v *= ms_sigmoid(behind[j]);
+      out[t * p.out_ld + c0 + d] = from_float<T>(v);
+    }
+  }
 }
 
 extern "C" int ps_state_output(const float* o, int heads, int value_dim, int ones, const float* floor_in,
@@ -537,18 +699,26 @@ extern "C" int ps_state_output(const float* o, int heads, int value_dim, int one
   const OutputArgs p = {o, heads, value_dim, ones ? 1 : 0, floor_in, skip, u, u_ld, before, before_ld, weight,
                         weight_count, eps, columns / groups, behind, behind_ld, out_ld, tokens};
   const int64_t units = (int64_t)tokens * groups;
-  const bool narrow = p.group <= 64 * MS_HELD;
+  const bool narrow = p.group <= 256;
+  const int held = (p.group + (narrow ? 63 : 255)) / (narrow ? 64 : 256);
+  PS_REQUIRE(held <= 32, "ps_state_output: groups of %d columns, at most 8192", p.group);
   const int64_t blocks = narrow ? (units + 3) / 4 : units;
   PS_REQUIRE(blocks < ((int64_t)1 << 31), "ps_state_output: too many blocks");
-#define PS_LAUNCH_SO(T)                                                                                   \
-  do {                                                                                                    \
-    if (narrow)                                                                                           \
-      hipLaunchKernelGGL((state_output_kernel<T, 64>), dim3((unsigned)blocks), dim3(256), 0, s, p, (T*)out); \
-    else                                                                                                  \
-      hipLaunchKernelGGL((state_output_kernel<T, 256>), dim3((unsigned)blocks), dim3(256), 0, s, p, (T*)out); \
+#define PS_LAUNCH_SO(T, LANES, HELD) \
+  hipLaunchKernelGGL((state_output_kernel<T, LANES, HELD>), dim3((unsigned)blocks), dim3(256), 0, s, p, (T*)out)
+#define PS_LAUNCH_SO_T(T)                               \
+  do {                                                  \
+    if (narrow && held == 1) PS_LAUNCH_SO(T, 64, 1);    \
+    else if (narrow && held == 2) PS_LAUNCH_SO(T, 64, 2); \
+    else if (narrow) PS_LAUNCH_SO(T, 64, 4);            \
+    else if (held <= 2) PS_LAUNCH_SO(T, 256, 2);        \
+    else if (held <= 4) PS_LAUNCH_SO(T, 256, 4);        \
+    else if (held <= 8) PS_LAUNCH_SO(T, 256, 8);        \
+    else PS_LAUNCH_SO(T, 256, 32);                      \
   } while (0)
-  if (dtype == PS_F32) PS_LAUNCH_SO(float);
-  else PS_LAUNCH_SO(bf16_t);
+  if (dtype == PS_F32) PS_LAUNCH_SO_T(float);
+  else PS_LAUNCH_SO_T(bf16_t);
+#undef PS_LAUNCH_SO_T
 #undef PS_LAUNCH_SO
   PS_CHECK_LAUNCH("ps_state_output");
   return 0;

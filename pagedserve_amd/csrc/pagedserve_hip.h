@@ -503,7 +503,7 @@ int ps_gated_norm_step(float* h, float* y, const float* gate, int64_t gate_ld, c
 // S[:, column], then what else the mixer keeps (`history`: the last taps - 1 raw inputs of the
 // convolution, [taps - 1][channels], oldest first; `maxima`: a running maximum per head).
 //
-// What the recurrence is fed with.  out[t, c] = silu(bias[c] + sum_j w[c, j] u[t - taps + 1 + j, c]) of
+// What the recurrence is fed with.  out[t, c] = silu(bias[c] + sum_j w[j, c] u[t - taps + 1 + j, c]) of
 // the raw inputs u = proj[:, col ...] of the item, earlier ones from its slot; the first unit_heads
 // runs of `head` channels become unit vectors, x / sqrt(sum(x^2) + 1e-6), the first scale_heads of
 // them times q_scale.  rule 0: dt = softplus(proj[t, take_col + h] + z_bias[h]), take = dt, decay =

@@ -2019,12 +2019,12 @@ def state_prepare(proj, col, weight, bias, state, history, out, rule, decay, tak
                   tok_item, cu_tokens, slots, z=None, per_head=1, unit_heads=0, head=0, scale_heads=0,
                   q_scale=1.0):
     """What a matrix-state recurrence is fed with (``csrc/pagedserve_hip.h: ps_state_prepare``): the short
-    convolution of ``weight [channels, taps]`` with silu and unit norms into ``out`` (float), decays and weights.
+    convolution of ``weight [taps, channels]`` (the last row is the current token's) with silu and unit norms into ``out`` (float), decays and weights.
     ``history``: where a slot of ``state`` (float ``[slots, n]``) keeps the last inputs."""
     _check(proj, "proj", torch.float32, 2)
     _check(weight, "weight", torch.float32, 2)
     tokens = proj.shape[0]
-    channels, taps = weight.shape
+    taps, channels = weight.shape
     heads = a_log.numel()
     if not weight.is_contiguous() or col + channels > proj.shape[1] or take_col + heads > proj.shape[1]:
         raise KernelError("state_prepare: the projection's rows are too short for its columns")

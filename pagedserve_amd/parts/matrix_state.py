@@ -66,7 +66,7 @@ class ChannelDelta(CoreMixer):
         }
 
     def bind_core(self, tensors, device):
-        self.conv_weight = tensors["conv.weight"]
+        self.conv_weight = tensors["conv.weight"].t().contiguous()
         self.decay_weight = tensors["decay.weight"].unsqueeze(0)
         self.decay_bias = tensors["decay.bias"]
         self.decay_log = tensors["decay.log"]
@@ -206,7 +206,7 @@ class HeadStateSpace(CoreMixer):
         }
 
     def bind_core(self, tensors, device):
-        self.conv_weight = tensors["conv.weight"]
+        self.conv_weight = tensors["conv.weight"].t().contiguous()
         self.conv_bias = tensors["conv.bias"]
         self.step_bias = tensors["step.bias"]
         self.decay_log = tensors["decay.log"]
