@@ -26,7 +26,8 @@ struct StateStep {
   int key_dim, value_dim;
   int ones;                  // one more column whose value is one for every token
   float q_scale;
-  int aligned;               // slots start at multiples of 16 bytes
+  int aligned;               // slots (records, in chunks) start at multiples of 16 bytes
+  int vectors;               // so do every head's queries, keys and values
   // the short convolution's raw inputs, kept for the next step (channels 0: none)
   const float* raw;
   int64_t raw_ld;

@@ -574,7 +574,7 @@ extern "C" int ps_state_scan(const float* q, int64_t q_ld, const float* k, int64
   hipStream_t s = (hipStream_t)stream;
   const int aligned = slot_stride % 4 == 0 && (uintptr_t)state % 16 == 0;
   const StateStep p = {q, q_ld, k, k_ld, v, v_ld, decay, take, state, slot_stride, out, cu_tokens, slots,
-                       heads, key_share, key_dim, value_dim, ones, q_scale, aligned, raw, raw_ld, channels, taps,
+                       heads, key_share, key_dim, value_dim, ones, q_scale, aligned, 0, raw, raw_ld, channels, taps,
                        history};
   const bool brief = longest == 1;
 #define PS_LAUNCH_WALK_D(RPL, GROUPS, CHUNK, DELTA)                                               \

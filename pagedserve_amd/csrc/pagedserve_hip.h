@@ -533,6 +533,19 @@ int ps_state_scan(const float* q, int64_t q_ld, const float* k, int64_t k_ld, co
                   int rule, int heads, int key_share, int key_dim, int value_dim, int ones,
                   float q_scale, int longest, const float* raw, int64_t raw_ld, int channels, int taps,
                   int64_t history, void* stream);
+// Rule 0 for steps with long portions, on the matrix cores: the items in pieces of
+// ps_state_chunk_tokens() tokens (piece_cu, item_first: ps_scan_pieces with that size) that run side by
+// side.  Queries, keys and values enter the products as bfloat16, everything else is float or two
+// bfloat16 parts of it.  records: scratch of pieces * heads * columns * key_dim floats (columns: value_dim,
+// one more with `ones`), totals: of pieces * heads.
+int ps_state_chunk_tokens(void);
+int ps_state_chunks(const float* q, int64_t q_ld, const float* k, int64_t k_ld, const float* v,
+                    int64_t v_ld, const float* decay, const float* take, float* state,
+                    int64_t slot_stride, float* out, const int* cu_tokens, const int* slots, int items,
+                    int heads, int key_share, int key_dim, int value_dim, int ones, float q_scale,
+                    const float* raw, int64_t raw_ld, int channels, int taps, int64_t history,
+                    const int* piece_cu, const int* item_first, int pieces, float* records,
+                    int64_t records_floats, float* totals, void* stream);
 // out[t, c] from the recurrence's o [tokens, heads, value_dim (+ 1)]: x = o (+ skip[h] u[t, c]); ones: x /
 // (max(|key sum|, floor_in[t, h]) + 1e-6); x *= silu(before[t, c]); x / rms over each of `groups` equal
 // runs of columns (eps inside the root) * weight[c % weight_count]; x *= sigmoid(behind[t, c]).

@@ -132,6 +132,10 @@ _SIGNATURES = {
     "ps_state_scan": [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p,
                       c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                       c_float, c_int, c_void_p, c_int64, c_int, c_int, c_int64, c_void_p],
+    "ps_state_chunks": [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p,
+                        c_int64, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float,
+                        c_void_p, c_int64, c_int, c_int, c_int64, c_void_p, c_void_p, c_int, c_void_p, c_int64,
+                        c_void_p, c_void_p],
     "ps_state_output": [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_int64,
                         c_void_p, c_int, c_float, c_int, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int,
                         c_void_p],
@@ -2013,6 +2017,23 @@ def _slot_rows(state, needed, what):
 
 
 STATE_RULES = {"decayed": 0, "delta": 1}
+STATE_CHUNK = 64            # tokens of a piece of the decayed rule on the matrix cores (csrc/matrix_state_chunks.hip)
+_STATE_CHUNK_CHECKED = False
+
+
+def _check_state_chunk():
+    global _STATE_CHUNK_CHECKED
+    if not _STATE_CHUNK_CHECKED:
+        lib = load_library()
+        lib.ps_state_chunk_tokens.restype = c_int
+        if lib.ps_state_chunk_tokens() != STATE_CHUNK:
+            raise KernelError("the library's pieces of a recurrence are not this module's; rebuild the library")
+        _STATE_CHUNK_CHECKED = True
+
+
+def state_chunk_floats(pieces, heads, key_dim, value_dim, ones=False):
+    """Floats of the two scratch buffers (records, totals) of ``state_scan(chunks=...)``."""
+    return pieces * heads * (value_dim + (1 if ones else 0)) * key_dim, pieces * heads
 
 
 def state_prepare(proj, col, weight, bias, state, history, out, rule, decay, take, a_log, z_bias, take_col,
@@ -2072,10 +2093,13 @@ def memory_gates(proj, i_col, f_col, i_bias, f_bias, cap, state, maxima, log_dec
 
 
 def state_scan(q, k, v, decay, take, state, out, cu_tokens, slots, rule, heads, key_heads, key_dim, value_dim,
-               ones=False, q_scale=1.0, longest=0, raw=None, taps=1, history=0):
+               ones=False, q_scale=1.0, longest=0, raw=None, taps=1, history=0, chunks=None):
     """The recurrence over the step's items (``csrc/pagedserve_hip.h: ps_state_scan``).  ``q``, ``k``, ``v``: float columns
     of (possibly wider) buffers; ``state``: float ``[slots, n]`` whose slots begin with the heads' matrices;
-    ``raw``: the raw input columns of the short convolution that the slot keeps (from ``history`` on)."""
+    ``raw``: the raw input columns of the short convolution that the slot keeps (from ``history`` on).
+    ``chunks = (piece_cu, item_first, pieces, records, totals)``: the decayed rule in pieces of ``STATE_CHUNK`` tokens on
+    the matrix cores, for steps with long portions (``ps_state_chunks``; ``scan_pieces`` gives the index arrays,
+    ``state_chunk_floats`` the sizes of the two scratch buffers)."""
     tokens = q.shape[0]
     q_ld = _float_columns(q, "q", tokens, key_heads * key_dim)
     k_ld = _float_columns(k, "k", tokens, key_heads * key_dim)
@@ -2096,6 +2120,27 @@ def state_scan(q, k, v, decay, take, state, out, cu_tokens, slots, rule, heads, 
     if heads % key_heads:
         raise KernelError(f"state_scan: {heads} heads do not share {key_heads} key heads evenly")
     items = _step_items(cu_tokens, slots, "state_scan")
+    if chunks is not None:
+        if rule != "decayed":
+            raise KernelError("state_scan: only the decayed rule runs in chunks")
+        piece_cu, item_first, pieces, records, totals = chunks
+        _check_state_chunk()
+        for name, index, least in (("piece_cu", piece_cu, pieces + 1), ("item_first", item_first, items + 1)):
+            _check(index, name, torch.int32, 1)
+            if index.numel() < least:
+                raise KernelError(f"state_scan: {name} needs {least} entries")
+        if pieces < tokens // STATE_CHUNK + items:
+            raise KernelError(f"state_scan: {tokens} tokens of {items} items may have more than {pieces} pieces")
+        _check(records, "records", torch.float32, 1)
+        _check(totals, "totals", torch.float32, 1)
+        if totals.numel() < pieces * heads:
+            raise KernelError("state_scan: the scratch for the pieces' sums is too small")
+        _call("ps_state_chunks", q.data_ptr(), q_ld, k.data_ptr(), k_ld, v.data_ptr(), v_ld, decay.data_ptr(),
+              take.data_ptr(), state.data_ptr(), stride, out.data_ptr(), cu_tokens.data_ptr(), slots.data_ptr(), items,
+              heads, heads // key_heads, key_dim, value_dim, 1 if ones else 0, float(q_scale), _ptr(raw), raw_ld,
+              channels, int(taps), int(history), piece_cu.data_ptr(), item_first.data_ptr(), int(pieces),
+              records.data_ptr(), records.numel(), totals.data_ptr(), _stream())
+        return
     _call("ps_state_scan", q.data_ptr(), q_ld, k.data_ptr(), k_ld, v.data_ptr(), v_ld, decay.data_ptr(),
           take.data_ptr(), state.data_ptr(), stride, out.data_ptr(), cu_tokens.data_ptr(), slots.data_ptr(), items,
           STATE_RULES[rule], heads, heads // key_heads, key_dim, value_dim, 1 if ones else 0, float(q_scale),

@@ -14,6 +14,31 @@ def _slot_floats(*pieces):
     return -(-sum(pieces) // 4) * 4
 
 
+# tokens beyond one per item from which a bfloat16 step runs a decayed recurrence in chunks
+CHUNKS_FROM = 128
+
+
+def _chunks(ctx, state, dtype, heads, key_dim, value_dim, ones=False):
+    """What ``kernels.state_scan`` needs to run this step in chunks, or None where it walks token by token."""
+    items = ctx.slots.numel()
+    if dtype != torch.bfloat16 or ctx.tokens - items < CHUNKS_FROM:
+        return None
+    workspace, slots, size = ctx.workspace, state.shape[0], kernels.STATE_CHUNK
+    # (the scratch is asked for at its largest, so that it never moves under recorded launches)
+    most = workspace.max_rows // size + slots
+    index = ctx.shared_calls.get("state_pieces")
+    if index is None:
+        # once per step, for all layers
+        index = (workspace.flat("state_piece_cu", most + 1, torch.int32),
+                 workspace.flat("state_item_first", slots + 1, torch.int32), ctx.tokens // size + items)
+        kernels.scan_pieces(ctx.cu_tokens, items, size, index[2], index[0], index[1])
+        ctx.shared_calls["state_pieces"] = index
+    records, totals = kernels.state_chunk_floats(most, heads, key_dim, value_dim, ones)
+    name = f"{heads}x{key_dim}x{value_dim}{'+1' if ones else ''}"
+    return index + (workspace.flat("state_records_" + name, records, torch.float32),
+                    workspace.flat("state_totals_" + name, totals, torch.float32))
+
+
 def _check_key_dim(dim):
     if not 0 < dim <= 256:
         raise ValueError(f"key head size {dim} must lie in 1..256")
@@ -158,7 +183,8 @@ class MatrixMemory(CoreMixer):
         o = workspace.first_rows("memory_out", heads * (dv + 1), torch.float32, tokens)
         kernels.state_scan(proj[:, col:k_col], proj[:, k_col:v_col], proj[:, v_col:gate_col], decay, take, cache.state,
                            o, ctx.cu_tokens, ctx.slots, "decayed", heads, heads, dk, dv, ones=True,
-                           q_scale=dk ** -0.5, longest=1 if ctx.decode_only else 0)
+                           q_scale=dk ** -0.5, longest=1 if ctx.decode_only else 0,
+                           chunks=_chunks(ctx, cache.state, self.dtype, heads, dk, dv, ones=True))
         kernels.state_output(o, heads, dv, self.norm_gamma, self.norm_eps, heads, out, floor=floor,
                              behind=proj[:, gate_col:i_col])
 
@@ -232,6 +258,7 @@ class HeadStateSpace(CoreMixer):
         o = workspace.first_rows("space_out", inner, torch.float32, tokens)
         kernels.state_scan(c, b, x, decay, take, cache.state, o, ctx.cu_tokens, ctx.slots, "decayed", heads,
                            self.groups, states, dv, longest=1 if ctx.decode_only else 0,
-                           raw=proj[:, x_col:step_col], taps=self.taps, history=self.history)
+                           raw=proj[:, x_col:step_col], taps=self.taps, history=self.history,
+                           chunks=_chunks(ctx, cache.state, self.dtype, heads, states, dv))
         kernels.state_output(o, heads, dv, self.norm_gamma, self.norm_eps, self.norm_groups, out, skip=self.skip,
                              u=x, before=proj[:, col:x_col])
