@@ -6,6 +6,9 @@ Notation: ``x`` the stream ``[T, d]``, ``N`` a layer norm with scale and shift. 
 N1(x)`` and adds ``N1b(sigmoid(R u + r) * F(u))``; a layer is a mixer, then a feed-forward or none.
 Matrices are stored ``[out, in]`` and applied as ``W u``.  Every recurrence takes the state it starts from
 and returns the one it leaves, so that a sequence may be cut.
+
+``forward(..., half=True)`` rounds to bfloat16 what a 16-bit engine may keep in 16 bits (inputs of matrix
+products, queries, keys and values): how far that moves the logits says what to expect of such an engine.
 """
 
 import math
@@ -13,6 +16,12 @@ import math
 import torch
 
 F64 = torch.float64
+_HALF = [False]
+
+
+def kept(x):
+    """``x``, or rounded to bfloat16 in a run that keeps 16 bits."""
+    return x.to(torch.bfloat16).to(F64) if _HALF[0] else x
 
 
 # ------------------------------------------------------------------ norms and small functions
@@ -78,19 +87,19 @@ def channel_delta(u, w, p, mixer, eps):
     heads, groups, dk, dv = mixer["heads"], mixer["kv_heads"], mixer["dim"], mixer["vdim"]
 
     def short(name, shape):
-        return silu(causal_conv(u @ w[p + name].T, w[p + name + ".conv"])).view(tokens, *shape)
+        return kept(silu(causal_conv(kept(u @ w[p + name].T), w[p + name + ".conv"]))).view(tokens, *shape)
 
     q = unit(short("q", (groups, dk))) * dk ** -0.5
     k = unit(short("k", (groups, dk)))
     v = short("v", (heads, dv))
     spread = torch.arange(heads) // (heads // groups)
     beta = torch.sigmoid(u @ w[p + "b"].T)
-    z = (u @ w[p + "a1"].T) @ w[p + "a2"].T + w[p + "dt_bias"]
+    z = kept(u @ w[p + "a1"].T) @ w[p + "a2"].T + w[p + "dt_bias"]
     g = torch.exp(-torch.exp(w[p + "A_log"])[:, None] * softplus(z).view(tokens, heads, dk))
     o, _ = delta_recurrence(q[:, spread], k[:, spread], v, beta, g)
     o = rms(o, eps) * w[p + "norm"]
-    gate = torch.sigmoid((u @ w[p + "g1"].T) @ w[p + "g2"].T)
-    return (o.reshape(tokens, heads * dv) * gate) @ w[p + "o"].T
+    gate = torch.sigmoid(kept(u @ w[p + "g1"].T) @ w[p + "g2"].T)
+    return kept(o.reshape(tokens, heads * dv) * gate) @ w[p + "o"].T
 
 
 # ------------------------------------------------------------------ attention without a softmax
@@ -126,11 +135,11 @@ def attention_half(u, w, p, left):
     tokens = u.shape[0]
     heads, groups, dk, dv = left["heads"], left["kv_heads"], left["dim"], left["vdim"]
     positions = torch.arange(tokens)
-    q = rotate_halves((u @ w[p + "q"].T).view(tokens, heads, dk), positions, left.get("rot"))
-    k = rotate_halves((u @ w[p + "k"].T).view(tokens, groups, dk), positions, left.get("rot"))
-    v = (u @ w[p + "v"].T).view(tokens, groups, dv)
+    q = kept(rotate_halves((u @ w[p + "q"].T).view(tokens, heads, dk), positions, left.get("rot")))
+    k = kept(rotate_halves((u @ w[p + "k"].T).view(tokens, groups, dk), positions, left.get("rot")))
+    v = kept(u @ w[p + "v"].T).view(tokens, groups, dv)
     o = logistic_attention(q, k, v, left["scale"], w[p + "pb"])
-    return o.reshape(tokens, heads * dv) @ w[p + "o"].T
+    return kept(o.reshape(tokens, heads * dv)) @ w[p + "o"].T
 
 
 # ------------------------------------------------------------------ state space with a decay per head
@@ -156,9 +165,9 @@ def state_space_half(u, w, p, right, eps):
     tokens = u.shape[0]
     heads, dv, states, groups = right["heads"], right["vdim"], right["state"], right["groups"]
     inner = heads * dv
-    both = u @ w[p + "in"].T
+    both = kept(u @ w[p + "in"].T)
     z, raw, dt = both[:, :inner], both[:, inner:2 * inner + 2 * groups * states], both[:, 2 * inner + 2 * groups * states:]
-    act = silu(causal_conv(raw, w[p + "conv"], w[p + "conv.b"]))
+    act = kept(silu(causal_conv(raw, w[p + "conv"], w[p + "conv.b"])))
     x = act[:, :inner].view(tokens, heads, dv)
     b = act[:, inner:inner + groups * states].view(tokens, groups, states)
     c = act[:, inner + groups * states:].view(tokens, groups, states)
@@ -166,7 +175,7 @@ def state_space_half(u, w, p, right, eps):
     dt = softplus(dt + w[p + "dt_bias"])
     y, _ = state_space_recurrence(x, dt, -torch.exp(w[p + "A_log"]), b[:, spread], c[:, spread], w[p + "D"])
     y = grouped_gated_norm(y.reshape(tokens, inner), z, w[p + "norm"], right["norm_groups"], eps)
-    return y @ w[p + "o"].T
+    return kept(y) @ w[p + "o"].T
 
 
 def parallel(u, w, p, mixer, eps):
@@ -206,18 +215,18 @@ def memory_gates(u, w, p, cap):
 def matrix_memory(u, w, p, mixer, eps):
     tokens = u.shape[0]
     heads, dk, dv = mixer["heads"], mixer["dim"], mixer["vdim"]
-    q = (u @ w[p + "q"].T).view(tokens, heads, dk) * dk ** -0.5
-    k = (u @ w[p + "k"].T).view(tokens, heads, dk)
-    v = (u @ w[p + "v"].T).view(tokens, heads, dv)
+    q = kept(u @ w[p + "q"].T).view(tokens, heads, dk) * dk ** -0.5
+    k = kept(u @ w[p + "k"].T).view(tokens, heads, dk)
+    v = kept(u @ w[p + "v"].T).view(tokens, heads, dv)
     i, f = memory_gates(u, w, p, mixer["gate_cap"])
     o, _ = matrix_memory_recurrence(q, k, v, i, f)
     o = rms(o, eps).reshape(tokens, heads * dv) * w[p + "norm"]
-    return (o * torch.sigmoid(u @ w[p + "g"].T)) @ w[p + "o"].T
+    return kept(o * torch.sigmoid(u @ w[p + "g"].T)) @ w[p + "o"].T
 
 
 # ------------------------------------------------------------------ the model
 def feed_forward(u, w, p):
-    return (torch.relu(u @ w[p + "gate"].T) * (u @ w[p + "up"].T)) @ w[p + "down"].T
+    return kept(torch.relu(u @ w[p + "gate"].T) * (u @ w[p + "up"].T)) @ w[p + "down"].T
 
 
 MIXERS = {"channel_delta": channel_delta, "parallel": parallel, "mlstm": matrix_memory}
@@ -226,13 +235,21 @@ MIXERS = {"channel_delta": channel_delta, "parallel": parallel, "mlstm": matrix_
 def gated_sublayer(x, w, p, number, eps, run):
     """``x + N_b(sigmoid(R u + r) * run(u))`` with ``u = N(x)``; ``number``: 1 the mixer's, 2 the feed-forward's."""
     a, b, r = f"{p}norm{number}", f"{p}norm{number}b", f"{p}rg{number}"
-    u = layer_norm(x, w[a], w[a + ".b"], eps)
+    u = kept(layer_norm(x, w[a], w[a + ".b"], eps))
     y = torch.sigmoid(u @ w[r].T + w[r + ".b"]) * run(u)
     return x + layer_norm(y, w[b], w[b + ".b"], eps)
 
 
-def forward(raw, tensors, tokens):
+def forward(raw, tensors, tokens, half=False):
     """(logits ``[T, vocab]``, the stream after every layer) of one sequence from its start."""
+    _HALF[0] = half
+    try:
+        return _forward(raw, tensors, tokens)
+    finally:
+        _HALF[0] = False
+
+
+def _forward(raw, tensors, tokens):
     w = {name: tensor.to(F64) for name, tensor in tensors.items()}
     eps = raw["norm"]["eps"]
     x = w["embed"][torch.tensor(list(tokens))]
@@ -243,7 +260,7 @@ def forward(raw, tensors, tokens):
         if layer.get("mlp") is not None:
             x = gated_sublayer(x, w, p, 2, eps, lambda u: feed_forward(u, w, p + "mlp."))
         after.append(x)
-    return layer_norm(x, w["final.norm"], w["final.norm.b"], eps) @ w["head"].T, after
+    return kept(layer_norm(x, w["final.norm"], w["final.norm.b"], eps)) @ w["head"].T, after
 
 
 def greedy_generate(raw, tensors, prompt, count):
@@ -251,3 +268,78 @@ def greedy_generate(raw, tensors, prompt, count):
     for _ in range(count):
         tokens.append(int(forward(raw, tensors, tokens)[0][-1].argmax()))
     return tokens[len(prompt):]
+
+
+# ------------------------------------------------------------------ random checkpoints
+def random_checkpoint(raw, seed, ranks=(6, 5)):
+    """Checkpoint tensors (float32) of a random model of the raw configuration: matrices N(0, 1/in), scales
+    around one, shifts and biases that matter, decays between fast and slow.  ``ranks``: inner widths of the
+    low-rank decay and gate of a delta layer where the configuration names none."""
+    g = torch.Generator().manual_seed(seed)
+
+    def normal(*shape, std=1.0):
+        return torch.randn(shape, generator=g) * std
+
+    def uniform(count, low, high):
+        return torch.rand(count, generator=g) * (high - low) + low
+
+    def matrix(rows, columns, gain=1.0):
+        return normal(rows, columns, std=gain / math.sqrt(columns))
+
+    d = raw["width"]
+    w = {"embed": normal(raw["vocab"], d), "head": matrix(raw["vocab"], d)}
+
+    def norm(name):
+        w[name], w[name + ".b"] = 1 + normal(d, std=0.2), normal(d, std=0.2)
+
+    norm("final.norm")
+    for i, layer in enumerate(raw["layers"]):
+        p, mixer = f"l{i}.", layer["mixer"]
+        m = p + "mix."
+        for number in (1, 2) if layer.get("mlp") is not None else (1,):
+            norm(f"{p}norm{number}")
+            norm(f"{p}norm{number}b")
+            w[f"{p}rg{number}"], w[f"{p}rg{number}.b"] = matrix(d, d), normal(d, std=0.5)
+        if layer["type"] == "channel_delta":
+            heads, groups, dk, dv = mixer["heads"], mixer["kv_heads"], mixer["dim"], mixer["vdim"]
+            for name, rows in (("q", groups * dk), ("k", groups * dk), ("v", heads * dv)):
+                w[m + name] = matrix(rows, d)
+                w[m + name + ".conv"] = normal(rows, mixer["conv"], std=1 / math.sqrt(mixer["conv"]))
+            a, b = mixer.get("decay_rank", ranks[0]), mixer.get("gate_rank", ranks[1])
+            w[m + "b"] = matrix(heads, d)
+            w[m + "A_log"] = uniform(heads, -2.0, 1.0)
+            w[m + "norm"] = 1 + normal(dv, std=0.2)
+            w[m + "a1"], w[m + "a2"] = matrix(a, d), matrix(heads * dk, a)
+            w[m + "dt_bias"] = uniform(heads * dk, -4.0, 0.0)
+            w[m + "g1"], w[m + "g2"] = matrix(b, d), matrix(heads * dv, b)
+            w[m + "o"] = matrix(d, heads * dv)
+        elif layer["type"] == "mlstm":
+            heads, dk, dv = mixer["heads"], mixer["dim"], mixer["vdim"]
+            for name, rows in (("q", heads * dk), ("k", heads * dk), ("v", heads * dv), ("g", heads * dv)):
+                w[m + name] = matrix(rows, d)
+            w[m + "i"], w[m + "i.b"] = matrix(heads, d, 2.0), normal(heads)
+            w[m + "f"], w[m + "f.b"] = matrix(heads, d), uniform(heads, 0.0, 5.0)
+            w[m + "norm"] = 1 + normal(heads * dv, std=0.2)
+            w[m + "o"] = matrix(d, heads * dv)
+        else:
+            left, right = mixer["left"], mixer["right"]
+            a, s = m + "left.", m + "right."
+            w[a + "q"] = matrix(left["heads"] * left["dim"], d)
+            w[a + "k"] = matrix(left["kv_heads"] * left["dim"], d)
+            w[a + "v"] = matrix(left["kv_heads"] * left["vdim"], d)
+            w[a + "pb"] = normal(left["heads"]) - 2.0
+            w[a + "o"] = matrix(d, left["heads"] * left["vdim"])
+            inner = right["heads"] * right["vdim"]
+            channels = inner + 2 * right["groups"] * right["state"]
+            w[s + "in"] = matrix(inner + channels + right["heads"], d)
+            w[s + "conv"] = normal(channels, right["conv"], std=1 / math.sqrt(right["conv"]))
+            w[s + "conv.b"] = normal(channels, std=0.2)
+            w[s + "dt_bias"] = uniform(right["heads"], -4.0, 0.0)
+            w[s + "A_log"] = uniform(right["heads"], -2.0, 1.5)
+            w[s + "D"] = normal(right["heads"])
+            w[s + "norm"] = 1 + normal(inner, std=0.2)
+            w[s + "o"] = matrix(d, inner)
+        if layer.get("mlp") is not None:
+            ff = layer["mlp"]["ff"]
+            w[p + "mlp.gate"], w[p + "mlp.up"], w[p + "mlp.down"] = matrix(ff, d), matrix(ff, d), matrix(d, ff)
+    return w
