@@ -229,10 +229,11 @@ class DecoderModel:
                 else:
                     kernels.stream_step(h, tokens, width, bias=bias, rows=rows)
             block.forward(h, ctx, view)
-            # a block may leave its last write to the block that follows, if that one takes it
+            # a block may leave its last write to the block that follows, if that one takes writes of its kind
             if hasattr(block, "finish"):
                 follower = self.blocks[schedule[index + 1].block] if index + 1 < len(schedule) else None
-                if getattr(follower, "takes_stream_write", False) != block.takes_stream_write:
+                takes = getattr(follower, "takes_stream_write", False)
+                if not takes or takes != block.takes_stream_write:
                     block.finish(h, ctx)
         wanted = logit_rows.numel()
         if wanted == 0:

@@ -288,7 +288,7 @@ def test_gate_with_the_tanh_form_of_gelu(dtype):
     tol = 1e-5 if dtype == torch.float32 else 2e-2
     assert torch.allclose(out.double().cpu(), expected, atol=tol, rtol=tol)
     with pytest.raises(Exception):
-        kernels.silu_gate(both.cuda(), out, "relu")
+        kernels.silu_gate(both.cuda(), out, "softsign")
 
 
 def test_latent_prepare_reads_queries_from_rows_of_their_own():
