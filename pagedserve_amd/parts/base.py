@@ -150,6 +150,16 @@ class Mixer(Part):
         raise NotImplementedError
 
 
+def packed_projection(workspace, core_rows: int, ride: int, tokens: int):
+    """Float rows for a packed product of ``core_rows`` columns and ``ride`` of the caller's, and the caller's columns.
+    (Rows begin at multiples of 32 bytes whatever the columns are: kernels that move 16 bytes at a time take them.)"""
+    total = core_rows + ride
+    _, proj, _ = workspace.column_views("core_proj", -(-total // 8) * 8, torch.float32, tokens, (total, -total % 8))
+    _, _, ridden, _ = workspace.column_views("core_proj", -(-total // 8) * 8, torch.float32, tokens,
+                                             (core_rows, ride, -total % 8))
+    return proj, ridden
+
+
 class CoreMixer(Mixer):
     """A mixer that works between two products: a packed product of the layer's input in float, the mixer's own
     work (``core``) on its columns, and an output product of what that leaves.  Kinds give ``core_rows`` (rows
@@ -204,8 +214,7 @@ class CoreMixer(Mixer):
 
     def forward(self, x, residual, ctx, cache):
         tokens, workspace = ctx.tokens, ctx.workspace
-        proj, _, ridden = workspace.column_views("core_proj", self.core_rows + self.ride, torch.float32, tokens,
-                                                 (self.core_rows, self.ride))
+        proj, ridden = packed_projection(workspace, self.core_rows, self.ride, tokens)
         kernels.linear(x, self.in_weight, None, proj, packed=self.in_packed,
                        memo=site_memo(self._memo_in, workspace), shared=ctx.shared_calls)
         out = workspace.first_rows("core_out", self.core_columns, self.dtype, tokens)

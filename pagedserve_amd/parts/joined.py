@@ -4,7 +4,7 @@ import torch
 
 from ..ops import kernels
 from ..weights.loader import MATRIX, ParamSpec
-from .base import Mixer, site_memo
+from .base import Mixer, packed_projection, site_memo
 from .registry import MIXERS, build_part, register_mixer
 
 
@@ -83,8 +83,7 @@ class JoinedMixers(Mixer):
         tokens, workspace = ctx.tokens, ctx.workspace
         left, right = self.left, self.right
         core_rows = left.core_rows + right.core_rows
-        proj, _, ridden = workspace.column_views("core_proj", core_rows + self.ride, torch.float32, tokens,
-                                                 (core_rows, self.ride))
+        proj, ridden = packed_projection(workspace, core_rows, self.ride, tokens)
         kernels.linear(x, self.in_weight, None, proj, packed=self.in_packed,
                        memo=site_memo(self._memo_in, workspace), shared=ctx.shared_calls)
         columns = left.core_columns + right.core_columns

@@ -93,6 +93,10 @@ class ChannelDelta(CoreMixer):
     def bind_core(self, tensors, device):
         self.conv_weight = tensors["conv.weight"].t().contiguous()
         self.decay_weight = tensors["decay.weight"].unsqueeze(0)
+        # equal sizes: both low-rank products as one block-diagonal one
+        self.low_weights = None
+        if self.decay_rank == self.gate_rank and self.heads * self.key_dim == self.value_cols:
+            self.low_weights = torch.stack([tensors["decay.weight"], tensors["gate.weight"]]).contiguous()
         self.decay_bias = tensors["decay.bias"]
         self.decay_log = tensors["decay.log"]
         self.gate_weight = tensors["gate.weight"].unsqueeze(0)
@@ -106,11 +110,16 @@ class ChannelDelta(CoreMixer):
         heads, dk, dv = self.heads, self.key_dim, self.value_dim
         low_col = col + self.channels
         gate_col = low_col + self.decay_rank
-        raw_decay = workspace.first_rows("delta_raw_decay", heads * dk, torch.float32, tokens)
-        kernels.block_linear(proj[:, low_col:gate_col], 0, self.decay_weight, None, raw_decay, heads * dk)
-        gate = workspace.first_rows("delta_gate", self.value_cols, torch.float32, tokens)
-        kernels.block_linear(proj[:, gate_col:gate_col + self.gate_rank], 0, self.gate_weight, None, gate,
-                             self.value_cols)
+        decays = heads * dk
+        both, raw_decay, gate = workspace.column_views("delta_low", decays + self.value_cols, torch.float32, tokens,
+                                                       (decays, self.value_cols))
+        if self.low_weights is not None:
+            kernels.block_linear(proj[:, low_col:gate_col + self.gate_rank], self.decay_rank, self.low_weights, None,
+                                 both, decays)
+        else:
+            kernels.block_linear(proj[:, low_col:gate_col], 0, self.decay_weight, None, raw_decay, decays)
+            kernels.block_linear(proj[:, gate_col:gate_col + self.gate_rank], 0, self.gate_weight, None, gate,
+                                 self.value_cols)
         mixed, q, k, v = workspace.column_views("delta_inputs", self.channels, torch.float32, tokens,
                                                 (self.key_cols, self.key_cols, self.value_cols))
         decay = workspace.first_rows("delta_decay", heads * dk, torch.float32, tokens)
